@@ -220,14 +220,24 @@ void weight_prefetch(const at::Tensor& W, int64_t nbytes, int64_t wgs, at::Tenso
   check_launch("weight_prefetch");
 }
 
+void set_gated_act(NormEpi& ne, int64_t act) {
+  TORCH_CHECK(act == ACT_SILU || act == ACT_GELU_TANH, "gated activation: 0 silu, 1 gelu (tanh form)");
+  if (act == ACT_GELU_TANH) {
+    ne.act_c0 = GELU_C0;
+    ne.act_c1 = GELU_C1;
+  }
+}
+
 void gemm_silu(const at::Tensor& X, const at::Tensor& W, at::Tensor& Y,
-               const c10::optional<at::Tensor>& ss_in, double norm_eps) {
+               const c10::optional<at::Tensor>& ss_in, double norm_eps, int64_t act) {
   CHECK_BF16_TENSOR(X); CHECK_BF16_TENSOR(W); CHECK_BF16_TENSOR(Y);
   const int K = X.size(-1), M = X.numel() / K, N = W.size(0);
   TORCH_CHECK(W.size(1) == K && N % 64 == 0, "gemm_silu: W [N, K], N % 64 == 0");
   TORCH_CHECK(Y.numel() == (int64_t)M * (N / 2), "gemm_silu: Y [M, N/2]");
   TORCH_CHECK(gemm_tn_check(M, N, K) == 0, "gemm_silu: unsupported shape");
-  NormEpiScope scope(make_norm_epi(M, K, c10::nullopt, ss_in, norm_eps));
+  NormEpi ne = make_norm_epi(M, K, c10::nullopt, ss_in, norm_eps);
+  set_gated_act(ne, act);
+  NormEpiScope scope(ne);
   TORCH_CHECK(launch_gemm_silu(X.data_ptr(), W.data_ptr(), Y.data_ptr(), M, N, K, stream()) == 0,
               "gemm_silu failed");
   check_launch("gemm_silu");
@@ -236,13 +246,15 @@ void gemm_silu(const at::Tensor& X, const at::Tensor& W, at::Tensor& Y,
 // tuning / tests: one SwiGLU path by code (launch_gemm_silu_algo); returns
 // nonzero (nothing launched) where the path does not take the shape
 int64_t gemm_silu_algo(const at::Tensor& X, const at::Tensor& W, at::Tensor& Y, int64_t algo,
-                       const c10::optional<at::Tensor>& ss_in, double norm_eps) {
+                       const c10::optional<at::Tensor>& ss_in, double norm_eps, int64_t act) {
   CHECK_BF16_TENSOR(X); CHECK_BF16_TENSOR(W); CHECK_BF16_TENSOR(Y);
   const int K = X.size(-1), M = X.numel() / K, N = W.size(0);
   TORCH_CHECK(W.size(1) == K && N % 64 == 0, "gemm_silu_algo: W [N, K], N % 64 == 0");
   TORCH_CHECK(Y.numel() == (int64_t)M * (N / 2), "gemm_silu_algo: Y [M, N/2]");
   TORCH_CHECK(gemm_tn_check(M, N, K) == 0, "gemm_silu_algo: unsupported shape");
-  NormEpiScope scope(make_norm_epi(M, K, c10::nullopt, ss_in, norm_eps));
+  NormEpi ne = make_norm_epi(M, K, c10::nullopt, ss_in, norm_eps);
+  set_gated_act(ne, act);
+  NormEpiScope scope(ne);
   const int rc = launch_gemm_silu_algo(X.data_ptr(), W.data_ptr(), Y.data_ptr(), M, N, K, (int)algo,
                                        stream());
   if (rc == 0) check_launch("gemm_silu_algo");
@@ -681,10 +693,21 @@ void prefix_attention(const at::Tensor& q, const at::Tensor& k_cache, const at::
   check_launch("prefix_attention");
 }
 
+// bf16, or f32 in the 32-bit mode: true for f32
+bool low_is_f32(const at::Tensor& t) {
+  TORCH_CHECK(t.scalar_type() == at::kBFloat16 || t.scalar_type() == at::kFloat, "bf16 or f32 tensor");
+  return t.scalar_type() == at::kFloat;
+}
+#define CHECK_TENSOR(t) CHECK_DEV(t); CHECK_CONTIG(t)
+#define CHECK_F32_TENSOR(t) CHECK_TENSOR(t); TORCH_CHECK((t).scalar_type() == at::kFloat, #t " must be f32")
+
 void sample_allowed(const at::Tensor& hidden, const at::Tensor& W, const at::Tensor& allow_ptr,
                     const at::Tensor& allow_ids, const at::Tensor& ctr, double temperature,
-                    int64_t seed, at::Tensor& out_tok, const c10::optional<at::Tensor>& out_logit) {
-  CHECK_BF16_TENSOR(hidden); CHECK_BF16_TENSOR(W);
+                    int64_t seed, at::Tensor& out_tok, const c10::optional<at::Tensor>& out_logit,
+                    double logit_scale, double logit_cap) {
+  CHECK_TENSOR(hidden); CHECK_TENSOR(W);
+  const bool f32 = low_is_f32(hidden);
+  TORCH_CHECK(W.scalar_type() == hidden.scalar_type(), "W dtype");
   CHECK_I32_TENSOR(allow_ptr); CHECK_I32_TENSOR(allow_ids); CHECK_I32_TENSOR(out_tok);
   CHECK_I32_TENSOR(ctr);
   const int S = hidden.size(0), H = hidden.size(1);
@@ -695,18 +718,170 @@ void sample_allowed(const at::Tensor& hidden, const at::Tensor& W, const at::Ten
   launch_sample_allowed(hidden.data_ptr(), W.data_ptr(), allow_ptr.data_ptr<int>(),
                         allow_ids.data_ptr<int>(), ctr.data_ptr<int>(),
                         (float)temperature, (unsigned long long)seed, S, H,
-                        out_tok.data_ptr<int>(), lp, stream());
+                        out_tok.data_ptr<int>(), lp, stream(), (float)logit_scale, (float)logit_cap, f32);
   check_launch("sample_allowed");
 }
 
-void sample_dense(const at::Tensor& logits, const at::Tensor& ctr, double temperature,
-                  int64_t seed, at::Tensor& out_tok) {
-  CHECK_BF16_TENSOR(logits); CHECK_I32_TENSOR(out_tok);
-  CHECK_I32_TENSOR(ctr);
-  launch_sample_dense(logits.data_ptr(), logits.size(0), logits.size(1),
-                      ctr.data_ptr<int>(), (float)temperature,
+void sample_dense(const at::Tensor& logits, const at::Tensor& allow_ptr, const at::Tensor& allow_ids,
+                  const at::Tensor& ctr, double temperature, int64_t seed, at::Tensor& out_tok) {
+  CHECK_F32_TENSOR(logits); CHECK_I32_TENSOR(out_tok); CHECK_I32_TENSOR(ctr);
+  CHECK_I32_TENSOR(allow_ptr); CHECK_I32_TENSOR(allow_ids);
+  const int S = logits.size(0);
+  TORCH_CHECK(logits.dim() == 2 && allow_ptr.numel() == S + 1 && out_tok.numel() == S && ctr.numel() == S,
+              "sample_dense shapes");
+  launch_sample_dense(logits.data_ptr<float>(), S, logits.size(1), allow_ptr.data_ptr<int>(),
+                      allow_ids.data_ptr<int>(), ctr.data_ptr<int>(), (float)temperature,
                       (unsigned long long)seed, out_tok.data_ptr<int>(), stream());
   check_launch("sample_dense");
+}
+
+// x [T, Hp] f32 (in place), y [T, Hp], out [T, >= Hp] rows (a row-strided view
+// is fine), w_post / w_pre [Hp] f32 or none
+void residual_norm(at::Tensor& x, const c10::optional<at::Tensor>& y,
+                   const c10::optional<at::Tensor>& w_post, const c10::optional<at::Tensor>& w_pre,
+                   const c10::optional<at::Tensor>& out, int64_t H, double eps) {
+  CHECK_F32_TENSOR(x);
+  const int Hp = x.size(-1), rows = x.numel() / Hp;
+  bool f32 = false;
+  int ld = 0;
+  if (y.has_value()) {
+    CHECK_TENSOR((*y));
+    f32 = low_is_f32(*y);
+    TORCH_CHECK(y->numel() == x.numel() && w_post.has_value(), "residual_norm: y [T, Hp] with w_post");
+  }
+  for (const auto* w : {&w_post, &w_pre})
+    if (w->has_value()) { CHECK_F32_TENSOR((**w)); TORCH_CHECK((*w)->numel() == Hp, "norm weight [Hp]"); }
+  if (out.has_value()) {
+    CHECK_DEV((*out));
+    const bool of = low_is_f32(*out);
+    TORCH_CHECK(!y.has_value() || of == f32, "y and out: one type");
+    f32 = of;
+    TORCH_CHECK(out->dim() == 2 && out->size(0) == rows && out->size(1) == Hp && out->stride(1) == 1 &&
+                    out->stride(0) % 4 == 0, "residual_norm: out [T, Hp]");
+    ld = out->stride(0);
+  }
+  TORCH_CHECK(launch_residual_norm(x.data_ptr<float>(), y.has_value() ? y->data_ptr() : nullptr,
+                                   w_post.has_value() ? w_post->data_ptr<float>() : nullptr,
+                                   w_pre.has_value() ? w_pre->data_ptr<float>() : nullptr,
+                                   out.has_value() ? out->data_ptr() : nullptr, ld, rows, (int)H, Hp,
+                                   (float)eps, f32, stream()) == 0,
+              "residual_norm: unsupported width ", Hp);
+  check_launch("residual_norm");
+}
+
+void embedding_scaled(const at::Tensor& ids, const at::Tensor& table, double scale, at::Tensor& x,
+                      const c10::optional<at::Tensor>& lo) {
+  CHECK_I32_TENSOR(ids); CHECK_TENSOR(table); CHECK_F32_TENSOR(x);
+  const bool f32 = low_is_f32(table);
+  const int Hp = table.size(1), T = ids.numel();
+  TORCH_CHECK(Hp % 4 == 0 && x.numel() == (int64_t)T * Hp, "embedding_scaled shapes");
+  int ld = 0;
+  if (lo.has_value()) {
+    CHECK_DEV((*lo));
+    TORCH_CHECK(lo->scalar_type() == table.scalar_type() && lo->dim() == 2 && lo->size(0) == T &&
+                    lo->size(1) == Hp && lo->stride(1) == 1 && lo->stride(0) % 4 == 0, "lo [T, Hp]");
+    ld = lo->stride(0);
+  }
+  launch_embedding_scaled(ids.data_ptr<int>(), table.data_ptr(), (float)scale, x.data_ptr<float>(),
+                          lo.has_value() ? lo->data_ptr() : nullptr, ld, T, Hp, f32, stream());
+  check_launch("embedding_scaled");
+}
+
+void logit_finish(at::Tensor& z, double scale, double cap) {
+  CHECK_F32_TENSOR(z);
+  launch_logit_finish(z.data_ptr<float>(), z.numel(), (float)scale, (float)cap, stream());
+  check_launch("logit_finish");
+}
+
+void gemm_f32(const at::Tensor& X, const at::Tensor& W, at::Tensor& Y) {
+  CHECK_F32_TENSOR(X); CHECK_F32_TENSOR(W); CHECK_F32_TENSOR(Y);
+  const int K = X.size(-1), M = X.numel() / K, N = W.size(0);
+  TORCH_CHECK(W.dim() == 2 && W.size(1) == K && Y.numel() == (int64_t)M * N, "gemm_f32 shapes");
+  TORCH_CHECK(launch_gemm_f32(X.data_ptr<float>(), W.data_ptr<float>(), Y.data_ptr<float>(), M, N, K,
+                              stream()) == 0, "gemm_f32: K % 16 == 0, N % 4 == 0");
+  check_launch("gemm_f32");
+}
+
+void gated_act_f32(const at::Tensor& z, at::Tensor& y, int64_t act) {
+  CHECK_F32_TENSOR(z); CHECK_F32_TENSOR(y);
+  const int F = y.size(-1), M = y.numel() / F;
+  TORCH_CHECK(F % 16 == 0 && z.numel() == 2 * y.numel(), "gated_act_f32 shapes");
+  launch_gated_act_f32(z.data_ptr<float>(), y.data_ptr<float>(), M, F, (int)act, stream());
+  check_launch("gated_act_f32");
+}
+
+void rope_kv_any(const at::Tensor& qkv, const c10::optional<at::Tensor>& bias, const at::Tensor& pos,
+                 const at::Tensor& slots, const at::Tensor& cos_sin, at::Tensor& q_out,
+                 at::Tensor& k_cache, at::Tensor& v_cache) {
+  CHECK_TENSOR(qkv); CHECK_I32_TENSOR(pos); CHECK_I32_TENSOR(slots); CHECK_F32_TENSOR(cos_sin);
+  CHECK_TENSOR(q_out); CHECK_TENSOR(k_cache); CHECK_TENSOR(v_cache);
+  const bool f32 = low_is_f32(qkv);
+  for (const auto* t : {&q_out, &k_cache, &v_cache})
+    TORCH_CHECK(t->scalar_type() == qkv.scalar_type(), "rope_kv_any: one type");
+  TORCH_CHECK(q_out.dim() == 3 && k_cache.dim() == 4 && v_cache.dim() == 4, "rope_kv_any dims");
+  const int T = pos.numel(), Hq = q_out.size(1), DK = q_out.size(2), Hkv = k_cache.size(1),
+            BS = k_cache.size(2), DV = v_cache.size(3);
+  const int64_t N = (int64_t)(Hq + Hkv) * DK + (int64_t)Hkv * DV;
+  TORCH_CHECK(q_out.size(0) == T && slots.numel() == T && qkv.numel() == T * N, "rope_kv_any: qkv [T, N]");
+  TORCH_CHECK(k_cache.size(3) == DK && v_cache.size(0) == k_cache.size(0) && v_cache.size(1) == Hkv &&
+                  v_cache.size(2) == BS, "rope_kv_any: caches [nb, Hkv, BS, D]");
+  TORCH_CHECK(cos_sin.dim() == 3 && cos_sin.size(1) == DK / 2 && cos_sin.size(2) == 2, "cos_sin [P, DK/2, 2]");
+  if (bias.has_value()) { CHECK_F32_TENSOR((*bias)); TORCH_CHECK(bias->numel() == N, "bias [N]"); }
+  TORCH_CHECK(launch_rope_kv_any(qkv.data_ptr(), bias.has_value() ? bias->data_ptr<float>() : nullptr,
+                                 pos.data_ptr<int>(), slots.data_ptr<int>(), cos_sin.data_ptr(),
+                                 q_out.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), T, Hq, Hkv, DK,
+                                 DV, BS, f32, stream()) == 0, "rope_kv_any: head sizes % 8");
+  check_launch("rope_kv_any");
+}
+
+MaskedAttnArgs masked_args(const at::Tensor& q, const at::Tensor& k_cache, const at::Tensor& v_cache,
+                           at::Tensor& out, const at::Tensor& q_start, const at::Tensor& q_len,
+                           const at::Tensor& ctx_len, const at::Tensor& block_table, double scale,
+                           double cap, int64_t chunk, bool sink) {
+  CHECK_TENSOR(q); CHECK_TENSOR(k_cache); CHECK_TENSOR(v_cache); CHECK_TENSOR(out);
+  CHECK_I32_TENSOR(q_start); CHECK_I32_TENSOR(q_len); CHECK_I32_TENSOR(ctx_len);
+  CHECK_I32_TENSOR(block_table);
+  for (const auto* t : {&k_cache, &v_cache, (const at::Tensor*)&out})
+    TORCH_CHECK(t->scalar_type() == q.scalar_type(), "masked attention: one type");
+  TORCH_CHECK(q.dim() == 3 && k_cache.dim() == 4 && v_cache.dim() == 4 && out.dim() == 3 &&
+                  block_table.dim() == 2, "masked attention dims");
+  MaskedAttnArgs a{};
+  a.Hq = q.size(1);
+  a.DK = q.size(2);
+  a.Hkv = k_cache.size(1);
+  a.DV = v_cache.size(3);
+  a.S = q_len.numel();
+  a.max_blocks = block_table.size(1);
+  TORCH_CHECK(a.Hq % a.Hkv == 0 && k_cache.size(2) == 64 && v_cache.size(2) == 64 &&
+                  k_cache.size(3) == a.DK && v_cache.size(1) == a.Hkv && v_cache.size(0) == k_cache.size(0),
+              "masked attention: caches [nb, Hkv, 64, D]");
+  TORCH_CHECK(out.size(0) == q.size(0) && out.size(1) == a.Hq && out.size(2) == a.DV, "out [T, Hq, DV]");
+  TORCH_CHECK(q_start.numel() == a.S && ctx_len.numel() == a.S && block_table.size(0) == a.S,
+              "masked attention: per-sequence arrays");
+  TORCH_CHECK(chunk >= 0 && cap >= 0, "masked attention: chunk, cap >= 0");
+  a.q = q.data_ptr();
+  a.kc = k_cache.data_ptr();
+  a.vc = v_cache.data_ptr();
+  a.out = out.data_ptr();
+  a.q_start = q_start.data_ptr<int>();
+  a.q_len = q_len.data_ptr<int>();
+  a.ctx_len = ctx_len.data_ptr<int>();
+  a.block_table = block_table.data_ptr<int>();
+  a.scale = (float)scale;
+  a.cap = (float)cap;
+  a.chunk = (int)chunk;
+  a.sink = sink;
+  return a;
+}
+
+void attention_row(const at::Tensor& q, const at::Tensor& k_cache, const at::Tensor& v_cache,
+                   at::Tensor& out, const at::Tensor& q_start, const at::Tensor& q_len,
+                   const at::Tensor& ctx_len, const at::Tensor& block_table, double scale, double cap,
+                   int64_t chunk, bool sink) {
+  const MaskedAttnArgs a = masked_args(q, k_cache, v_cache, out, q_start, q_len, ctx_len, block_table,
+                                       scale, cap, chunk, sink);
+  TORCH_CHECK(launch_attn_row(a, q.size(0), low_is_f32(q), stream()) == 0, "attention_row: value heads <= 512");
+  check_launch("attention_row");
 }
 
 // decision lookahead: the sampled outcome's tokens / sizes / allowed set into
@@ -730,13 +905,15 @@ void branch_select(const at::Tensor& prev_tok, const at::Tensor& tab, int64_t n,
   check_launch("branch_select");
 }
 
+// data [n, c, nb, Hkv, BS, D] bf16 (a f32 cache as bf16 words of twice the width)
 void copy_blocks(at::Tensor& data, const at::Tensor& src, const at::Tensor& dst) {
   CHECK_BF16_TENSOR(data); CHECK_I32_TENSOR(src); CHECK_I32_TENSOR(dst);
   TORCH_CHECK(data.dim() == 6, "kv data [L, 2, nb, Hkv, BS, D]");
+  TORCH_CHECK(data.size(3) * data.size(4) * data.size(5) % 8 == 0, "block of 16-B vectors");
   TORCH_CHECK(src.numel() == dst.numel(), "pairs");
   const int64_t block_elems = data.size(3) * data.size(4) * data.size(5);
   launch_copy_blocks(data.data_ptr(), src.data_ptr<int>(), dst.data_ptr<int>(), src.numel(),
-                     data.size(0) * 2, data.size(2), block_elems, stream());
+                     data.size(0) * data.size(1), data.size(2), block_elems, stream());
   check_launch("copy_blocks");
 }
 
@@ -878,7 +1055,7 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
         "measured SwiGLU path per 64-row M bucket for one gate|up (N, K) (-1: the rule)");
   m.def("gemm_silu_algo", &gemm_silu_algo, "one SwiGLU GEMM path by code (tuning / tests)",
         py::arg("X"), py::arg("W"), py::arg("Y"), py::arg("algo"), py::arg("ss_in") = py::none(),
-        py::arg("norm_eps") = 0.0);
+        py::arg("norm_eps") = 0.0, py::arg("act") = 0);
   m.def("gemm_plan_set_splits", &gemm_plan_set_splits_py,
         "measured split-K of the 128^2 path for one (N, K): a count per 64-row M bucket (0 = rule)");
   m.def("gemm_plan_split", &gemm_plan_split);
@@ -917,7 +1094,7 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("weight_prefetch", &weight_prefetch, py::arg("W"), py::arg("nbytes"), py::arg("wgs"), py::arg("sink"),
         "read up to nbytes of W once on the current stream (Infinity Cache warm-up)");
   m.def("gemm_silu", &gemm_silu, py::arg("X"), py::arg("W"), py::arg("Y"),
-        py::arg("ss_in") = py::none(), py::arg("norm_eps") = 0.0);
+        py::arg("ss_in") = py::none(), py::arg("norm_eps") = 0.0, py::arg("act") = 0);
   m.def("gemm_f32out", &gemm_f32out);
   m.def("l2norm_rows", &l2norm_rows);
   m.def("topk_fused", &topk_fused, py::arg("Q"), py::arg("E"), py::arg("k"), py::arg("cand_v"),
@@ -948,8 +1125,16 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("attn_tokens_per_item", &attn_tokens_per_item);
   m.def("sample_allowed", &sample_allowed, py::arg("hidden"), py::arg("W"), py::arg("allow_ptr"),
         py::arg("allow_ids"), py::arg("ctr"), py::arg("temperature"), py::arg("seed"),
-        py::arg("out_tok"), py::arg("out_logit") = py::none());
+        py::arg("out_tok"), py::arg("out_logit") = py::none(), py::arg("logit_scale") = 1.0,
+        py::arg("logit_cap") = 0.0);
   m.def("sample_dense", &sample_dense);
+  m.def("residual_norm", &residual_norm);
+  m.def("embedding_scaled", &embedding_scaled);
+  m.def("logit_finish", &logit_finish);
+  m.def("gemm_f32", &gemm_f32);
+  m.def("gated_act_f32", &gated_act_f32);
+  m.def("rope_kv_any", &rope_kv_any);
+  m.def("attention_row", &attention_row);
   m.def("branch_select", &branch_select);
   m.def("add_inplace", &add_inplace);
   m.def("paged_attention_decode_oproj", &paged_attention_decode_oproj,

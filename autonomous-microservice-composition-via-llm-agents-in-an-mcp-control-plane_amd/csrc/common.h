@@ -98,6 +98,12 @@ DEV float norm_row_scale(const NE& ne, int m) {
   const float ss = (float)ne.ss_in[m] * (1.f / SS_FIX);
   return rsqrtf(ss * ne.inv_h + ne.eps);
 }
+// gated activation of the EPI 2 epilogues: g sigmoid(g (c0 + c1 g^2)) u, which is
+// silu(g) u at (1, 0) and the tanh form of gelu at (GELU_C0, GELU_C1)
+template <class NE>
+DEV float gated_act(const NE& ne, float g, float u) {
+  return g / (1.f + __expf(-g * fmaf(ne.act_c1, g * g, ne.act_c0))) * u;
+}
 // the row scales of N rows at once: the wave-uniform "no norm" test is hoisted
 // out and every load issued before the first use (norm_row_scale in an
 // unrolled loop makes hipcc branch around each load and wait vmcnt(0) per
@@ -208,7 +214,7 @@ DEV void store_silu(const f32x4 (&acc)[MT][NT], bf16* __restrict__ Y, int M, int
       const f32x4 gv = acc[mt][2 * p] * rs[mt], uv = acc[mt][2 * p + 1] * rs[mt];
       bf16x4 o;
 #pragma unroll
-      for (int j = 0; j < 4; ++j) o[j] = (bf16)(gv[j] / (1.f + __expf(-gv[j])) * uv[j]);
+      for (int j = 0; j < 4; ++j) o[j] = (bf16)gated_act(ne, gv[j], uv[j]);
       *reinterpret_cast<bf16x4*>(Y + (size_t)m * F + f) = o;
     }
   }
@@ -266,8 +272,8 @@ DEV void store_wide(const f32x4 (&acc)[MT][8], RS rsY, const bf16* __restrict__ 
         const f32x4 gb = acc[mt][4 * p + 2] * s, ub = acc[mt][4 * p + 3] * s;
 #pragma unroll
         for (int e = 0; e < 4; ++e) {
-          oa[e] = (bf16)(ga[e] / (1.f + __expf(-ga[e])) * ua[e]);
-          ob[e] = (bf16)(gb[e] / (1.f + __expf(-gb[e])) * ub[e]);
+          oa[e] = (bf16)gated_act(ne, ga[e], ua[e]);
+          ob[e] = (bf16)gated_act(ne, gb[e], ub[e]);
         }
       } else {
 #pragma unroll
@@ -359,8 +365,8 @@ DEV void store_wide_slab(const f32x4 (&acc)[MT][8], RS rsY, const bf16* __restri
         const f32x4 gb = av(4 * p + 2) * s, ub = av(4 * p + 3) * s;
 #pragma unroll
         for (int e = 0; e < 4; ++e) {
-          oa[e] = (bf16)(ga[e] / (1.f + __expf(-ga[e])) * ua[e]);
-          ob[e] = (bf16)(gb[e] / (1.f + __expf(-gb[e])) * ub[e]);
+          oa[e] = (bf16)gated_act(ne, ga[e], ua[e]);
+          ob[e] = (bf16)gated_act(ne, gb[e], ub[e]);
         }
       } else {
 #pragma unroll

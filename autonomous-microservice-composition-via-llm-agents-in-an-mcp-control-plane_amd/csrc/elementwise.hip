@@ -280,3 +280,72 @@ void launch_copy_blocks(void* data, const int* src, const int* dst, int npairs, 
                                                       block_elems / 8);
 }
 
+// ------------------------- RoPE + KV write, any head sizes, biases, bf16 / f32
+// qkv: [T, Hq DK + Hkv DK + Hkv DV] from the QKV projection, ``bias`` (fp32,
+// one per column, or null) added first.  Queries and keys rotate as halves
+// (dimension j with j + DK / 2; cos_sin [max_pos, DK / 2] float2 holds the
+// identity for pairs that do not rotate), values pass.  One thread per 8
+// elements: 4 + 4 of a q / k head, 8 of a v head.
+template <class T>
+__global__ __launch_bounds__(256) void rope_kv_any_kernel(
+    const T* __restrict__ qkv, const float* __restrict__ bias, const int* __restrict__ pos,
+    const int* __restrict__ slots, const float2* __restrict__ cos_sin, T* __restrict__ q_out,
+    T* __restrict__ k_cache, T* __restrict__ v_cache, int T_, int Hq, int Hkv, int DK, int DV,
+    int BS) {
+  const int uk = DK / 8, uv = DV / 8;
+  const int per = (Hq + Hkv) * uk + Hkv * uv;
+  const int N = (Hq + Hkv) * DK + Hkv * DV;
+  const size_t i = blockIdx.x * 256ull + threadIdx.x;
+  if (i >= (size_t)T_ * per) return;
+  const int t = (int)(i / per);
+  int u = (int)(i % per);
+  const T* src = qkv + (size_t)t * N;
+  if (u >= (Hq + Hkv) * uk) {                          // value head
+    u -= (Hq + Hkv) * uk;
+    const int slot = slots[t];
+    if (slot < 0) return;
+    const int h = u / uv, d = (u % uv) * 8;
+    const int col = (Hq + Hkv) * DK + h * DV + d;
+    T* dst = v_cache + (((size_t)(slot / BS) * Hkv + h) * BS + slot % BS) * DV + d;
+#pragma unroll
+    for (int j = 0; j < 8; ++j) dst[j] = (T)((float)src[col + j] + (bias ? bias[col + j] : 0.f));
+    return;
+  }
+  const int h = u / uk, d = (u % uk) * 4;
+  const int col = h * DK + d;
+  T* dst;
+  if (h < Hq) {
+    dst = q_out + ((size_t)t * Hq + h) * DK + d;
+  } else {
+    const int slot = slots[t];
+    if (slot < 0) return;
+    dst = k_cache + (((size_t)(slot / BS) * Hkv + (h - Hq)) * BS + slot % BS) * DK + d;
+  }
+  const float2* cs = cos_sin + (size_t)pos[t] * (DK / 2) + d;
+#pragma unroll
+  for (int j = 0; j < 4; ++j) {
+    const float2 r = cs[j];
+    const float a = (float)src[col + j] + (bias ? bias[col + j] : 0.f);
+    const float b = (float)src[col + DK / 2 + j] + (bias ? bias[col + DK / 2 + j] : 0.f);
+    dst[j] = (T)(a * r.x - b * r.y);
+    dst[DK / 2 + j] = (T)(b * r.x + a * r.y);
+  }
+}
+
+int launch_rope_kv_any(const void* qkv, const float* bias, const int* pos, const int* slots,
+                       const void* cos_sin, void* q_out, void* k_cache, void* v_cache, int T, int Hq,
+                       int Hkv, int DK, int DV, int BS, bool f32, hipStream_t s) {
+  if (T <= 0) return 0;
+  if (DK % 8 || DV % 8) return 1;
+  const size_t total = (size_t)T * ((Hq + Hkv) * (DK / 8) + Hkv * (DV / 8));
+  const unsigned grid = (unsigned)((total + 255) / 256);
+  if (f32)
+    rope_kv_any_kernel<float><<<grid, 256, 0, s>>>((const float*)qkv, bias, pos, slots,
+                                                   (const float2*)cos_sin, (float*)q_out,
+                                                   (float*)k_cache, (float*)v_cache, T, Hq, Hkv, DK, DV, BS);
+  else
+    rope_kv_any_kernel<bf16><<<grid, 256, 0, s>>>((const bf16*)qkv, bias, pos, slots,
+                                                  (const float2*)cos_sin, (bf16*)q_out,
+                                                  (bf16*)k_cache, (bf16*)v_cache, T, Hq, Hkv, DK, DV, BS);
+  return 0;
+}

@@ -178,7 +178,7 @@ __global__ __launch_bounds__(256) void splitk_reduce(const float* __restrict__ w
     g *= rs;
     u *= rs;
 #pragma unroll
-    for (int j = 0; j < 4; ++j) o[j] = (bf16)(g[j] / (1.f + __expf(-g[j])) * u[j]);
+    for (int j = 0; j < 4; ++j) o[j] = (bf16)gated_act(ne, g[j], u[j]);
   } else {
     const float* p = ws + (size_t)m * N + c;
     f32x4 v = *reinterpret_cast<const f32x4*>(p);

@@ -221,7 +221,7 @@ DEV void mainloop(const bf16* __restrict__ X, const bf16* __restrict__ W, int M,
 // lane holds Y[m][n .. n+3] of each 16x16 fragment
 template <int EPI>
 DEV void epilogue(bf16* __restrict__ Y, const bf16* __restrict__ R, int M, int N, int m0, int n0,
-                  const f32x4 (&acc)[2][4][4]) {
+                  const f32x4 (&acc)[2][4][4], const NormEpi& ne) {
   const int lane = threadIdx.x & 63;
   const int wave = threadIdx.x >> 6;
   const int wm = wave >> 2, wn = wave & 3;
@@ -238,10 +238,11 @@ DEV void epilogue(bf16* __restrict__ Y, const bf16* __restrict__ R, int M, int N
         for (int p = 0; p < 2; ++p) {
           const int f = ((n0 + wn * 64) >> 1) + p * 16 + fq * 4;
           if (f >= F) continue;
-          const f32x4 gv = acc[mh][mt][2 * p], uv = acc[mh][mt][2 * p + 1];
+          const float rs = norm_row_scale(ne, m);
+          const f32x4 gv = acc[mh][mt][2 * p] * rs, uv = acc[mh][mt][2 * p + 1] * rs;
           bf16x4 o;
 #pragma unroll
-          for (int j = 0; j < 4; ++j) o[j] = (bf16)(gv[j] / (1.f + __expf(-gv[j])) * uv[j]);
+          for (int j = 0; j < 4; ++j) o[j] = (bf16)gated_act(ne, gv[j], uv[j]);
           *reinterpret_cast<bf16x4*>(Y + (size_t)m * F + f) = o;
         }
         continue;
@@ -269,14 +270,14 @@ __global__ __launch_bounds__(512, 1) void gemm_tn_256(const bf16* __restrict__ X
                                                       const bf16* __restrict__ W,
                                                       bf16* __restrict__ Y,
                                                       const bf16* __restrict__ R, int M, int N,
-                                                      int K) {
+                                                      int K, const NormEpi ne) {
   __shared__ __attribute__((aligned(16))) bf16 smem[8 * PIECE];
   const int nm = (M + BM - 1) / BM, nn = (N + BN - 1) / BN;
   int m0, n0;
   tile_coords(xcd_remap(blockIdx.x, nm * nn), nm, nn, m0, n0);
   f32x4 acc[2][4][4];
   mainloop<VAR>(X, W, M, N, K, m0, n0, 0, K / BK, smem, acc);
-  epilogue<EPI>(Y, R, M, N, m0, n0, acc);
+  epilogue<EPI>(Y, R, M, N, m0, n0, acc, ne);
 }
 
 // ---------------------------------------------------------------------------
@@ -297,7 +298,7 @@ __global__ __launch_bounds__(512, 1) void gemm_tn_256_splitk(const bf16* __restr
                                                              const bf16* __restrict__ R, int M,
                                                              int N, int K, int splits,
                                                              float* __restrict__ ws,
-                                                             int* __restrict__ cnt) {
+                                                             int* __restrict__ cnt, const NormEpi ne) {
   // ONE __shared__ array: a second LDS object (even the 4-byte last-arriver
   // flag) makes hipcc put vmcnt(0) before every ds_read of the K-loop
   // (cdna_hip_programming.md §5 "Three .s-level traps" (a))
@@ -340,14 +341,14 @@ __global__ __launch_bounds__(512, 1) void gemm_tn_256_splitk(const bf16* __restr
     for (int q = 0; q < 32; ++q)
       (&acc[0][0][0])[q] += wsv[((size_t)c * 32 + q) * 512 + threadIdx.x];
   }
-  epilogue<EPI>(Y, R, M, N, m0, n0, acc);
+  epilogue<EPI>(Y, R, M, N, m0, n0, acc, ne);
 }
 
 template <class VAR>
 void launch_var(const void* X, const void* W, void* Y, int M, int N, int K, hipStream_t s) {
   const int nm = (M + BM - 1) / BM, nn = (N + BN - 1) / BN;
   gemm_tn_256<0, VAR><<<dim3(nm * nn), 512, 0, s>>>((const bf16*)X, (const bf16*)W, (bf16*)Y,
-                                                    nullptr, M, N, K);
+                                                    nullptr, M, N, K, NormEpi{});
 }
 
 }  // namespace
@@ -505,11 +506,12 @@ void launch_256(const void* X, const void* W, void* Y, const void* R, int M, int
   splits = min(splits, max(1, K / BK));
   if (splits > 1 && sk_reserve(sd, tiles, splits)) {
     gemm_tn_256_splitk<EPI, VAR><<<tiles * splits, 512, 0, s>>>(
-        (const bf16*)X, (const bf16*)W, (bf16*)Y, (const bf16*)R, M, N, K, splits, sd.ws, sd.cnt);
+        (const bf16*)X, (const bf16*)W, (bf16*)Y, (const bf16*)R, M, N, K, splits, sd.ws, sd.cnt,
+        norm_epi());
     return;
   }
   gemm_tn_256<EPI, VAR><<<dim3(tiles), 512, 0, s>>>((const bf16*)X, (const bf16*)W, (bf16*)Y,
-                                                    (const bf16*)R, M, N, K);
+                                                    (const bf16*)R, M, N, K, norm_epi());
 }
 
 }  // namespace

@@ -485,7 +485,7 @@ __global__ __launch_bounds__(256, 1) void gemm_tn_256d(const bf16* __restrict__ 
           const f32x4 gv = acc[mt][2 * p] * rsc[mt], uv = acc[mt][2 * p + 1] * rsc[mt];
           bf16x4 o;
 #pragma unroll
-          for (int j = 0; j < 4; ++j) o[j] = (bf16)(gv[j] / (1.f + __expf(-gv[j])) * uv[j]);
+          for (int j = 0; j < 4; ++j) o[j] = (bf16)gated_act(ne, gv[j], uv[j]);
           put(row, p * 16 + fq * 4, o);
         }
       } else {

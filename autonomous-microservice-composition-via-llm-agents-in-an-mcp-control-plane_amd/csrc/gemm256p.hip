@@ -370,7 +370,7 @@ __global__ __launch_bounds__(256, 1) void gemm_tn_256p(const bf16* __restrict__ 
             const f32x4 gv = acc[mt][2 * pp] * rsc[mt], uv = acc[mt][2 * pp + 1] * rsc[mt];
             bf16x4 o;
 #pragma unroll
-            for (int e = 0; e < 4; ++e) o[e] = (bf16)(gv[e] / (1.f + __expf(-gv[e])) * uv[e]);
+            for (int e = 0; e < 4; ++e) o[e] = (bf16)gated_act(ne, gv[e], uv[e]);
             put(row, pp * 16 + fq * 4, o);
           }
         } else {

@@ -97,7 +97,7 @@ DEV void store_row(bf16* __restrict__ Y, int M, int N, int m0, int n0, int wm, i
       const f32x4 gv = v(2 * p) * in.rs, uv = v(2 * p + 1) * in.rs;
       bf16x4 o;
 #pragma unroll
-      for (int j = 0; j < 4; ++j) o[j] = (bf16)(gv[j] / (1.f + __expf(-gv[j])) * uv[j]);
+      for (int j = 0; j < 4; ++j) o[j] = (bf16)gated_act(ne, gv[j], uv[j]);
       *reinterpret_cast<bf16x4*>(Y + (size_t)m * F2 + f) = o;
     }
     return;

@@ -166,7 +166,7 @@ __global__ __launch_bounds__(64 * WV) void gemm_skinny(const bf16* __restrict__ 
 #pragma unroll
       for (int q = 0; q < 4; ++q) {
         const float gv = tot[0][q] * rs, uv = up[q] * rs;
-        o[q] = (bf16)(gv / (1.f + __expf(-gv)) * uv);
+        o[q] = (bf16)gated_act(ne, gv, uv);
       }
       *reinterpret_cast<bf16x4*>(Y + (size_t)m * (N >> 1) + 8 * bx + 4 * g) = o;
       continue;
@@ -179,7 +179,7 @@ __global__ __launch_bounds__(64 * WV) void gemm_skinny(const bf16* __restrict__ 
 #pragma unroll
       for (int q = 0; q < 4; ++q) {
         const float gv = tot[0][q] * rs, uv = tot[1][q] * rs;
-        o[q] = (bf16)(gv / (1.f + __expf(-gv)) * uv);
+        o[q] = (bf16)gated_act(ne, gv, uv);
       }
       *reinterpret_cast<bf16x4*>(Y + (size_t)m * F + f) = o;
     } else {

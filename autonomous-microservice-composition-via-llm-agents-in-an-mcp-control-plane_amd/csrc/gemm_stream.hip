@@ -292,7 +292,7 @@ __global__ __launch_bounds__(256 * MH, MH == 1 ? 2 : 1) void gemm_stream(const b
       const f32x4 gv = sum[a][0] * rs, uv = sum[a][1] * rs;
       bf16x4 o;
 #pragma unroll
-      for (int i = 0; i < 4; ++i) o[i] = (bf16)(gv[i] / (1.f + __expf(-gv[i])) * uv[i]);
+      for (int i = 0; i < 4; ++i) o[i] = (bf16)gated_act(ne, gv[i], uv[i]);
       *reinterpret_cast<bf16x4*>(Y + (size_t)m * (N >> 1) + (n0 >> 1) + 8 * f0 + 4 * g) = o;
     } else if constexpr (EPI == 3) {
       const int head = tile >> 1;

@@ -17,7 +17,12 @@ struct NormEpi {
   unsigned long long* ss_out = nullptr;     // [M] fixed point (common.h SS_FIX), zeroed by the caller
   const unsigned long long* ss_in = nullptr;
   float inv_h = 0.f, eps = 0.f;
+  // gated activation of EPI 2 (common.h gated_act): g sigmoid(g (act_c0 + act_c1 g^2)) u;
+  // (1, 0) is SwiGLU, the pair below the tanh form of gelu
+  float act_c0 = 1.f, act_c1 = 0.f;
 };
+// 0.5 g (1 + tanh(sqrt(2 / pi) (g + 0.044715 g^3))) = g sigmoid(2 sqrt(2 / pi) (g + 0.044715 g^3))
+constexpr float GELU_C0 = 1.5957691216057308f, GELU_C1 = 1.5957691216057308f * 0.044715f;
 NormEpi& norm_epi();                     // the current launch's (host, not thread-shared)
 struct NormEpiScope {
   NormEpi saved;
@@ -38,6 +43,43 @@ void launch_rope_kv(const void* qkv, const int* pos, const int* slots, const voi
                     void* q_out, void* k_cache, void* v_cache, int T, int Hq, int Hkv, int D,
                     int BS, hipStream_t s);
 void launch_add_inplace(void* y, const void* x, size_t n, hipStream_t s);
+
+// any head sizes, q / k / v biases (fp32 or null), bf16 or f32; nonzero: head sizes not multiples of 8
+int launch_rope_kv_any(const void* qkv, const float* bias, const int* pos, const int* slots,
+                       const void* cos_sin, void* q_out, void* k_cache, void* v_cache, int T, int Hq,
+                       int Hkv, int DK, int DV, int BS, bool f32, hipStream_t s);
+
+// residual.hip: fp32 residual stream, norms on both sides of a sublayer
+constexpr int RESIDUAL_MAX_WIDTH = 16384;
+int launch_residual_norm(float* x, const void* y, const float* w_post, const float* w_pre,
+                         void* out, int ld, int rows, int H, int Hp, float eps, bool f32,
+                         hipStream_t s);
+void launch_embedding_scaled(const int* ids, const void* table, float scale, float* x, void* lo,
+                             int ld, int T, int Hp, bool f32, hipStream_t s);
+void launch_logit_finish(float* z, size_t n, float scale, float cap, hipStream_t s);
+
+// gemm_f32.hip: the 32-bit mode's products
+enum GatedAct { ACT_SILU = 0, ACT_GELU_TANH = 1 };
+int launch_gemm_f32(const float* X, const float* W, float* Y, int M, int N, int K, hipStream_t s);
+void launch_gated_act_f32(const float* z, float* y, int M, int F, int act, hipStream_t s);
+
+// attention_masked.hip
+struct MaskedAttnArgs {
+  const void* q;
+  const void* kc;
+  const void* vc;
+  void* out;
+  const int* q_start;
+  const int* q_len;
+  const int* ctx_len;
+  const int* block_table;
+  int max_blocks, S;
+  int Hq, Hkv, DK, DV;
+  float scale, cap;          // cap 0: no soft cap
+  int chunk;                 // 0: plain causal
+  int sink;
+};
+int launch_attn_row(const MaskedAttnArgs& a, int T, bool f32, hipStream_t s);
 
 // QKV projection + RoPE + paged K/V write fused in the GEMM epilogue (K1+K4+K10)
 // serving-size M: tile shape per (M, N) filling one wave of workgroups (gemm_flex.hip)
@@ -210,8 +252,11 @@ int launch_prefix_attention(const void* q, const void* k_cache, const void* v_ca
 void launch_sample_allowed(const void* hidden, const void* W, const int* allow_ptr,
                            const int* allow_ids, const int* ctr, float temperature,
                            unsigned long long seed, int S, int H, int* out_tok, float* out_logit,
-                           hipStream_t s);
-void launch_sample_dense(const void* logits, int S, int V, const int* ctr, float temperature,
+                           hipStream_t s, float logit_scale = 1.f, float logit_cap = 0.f,
+                           bool f32 = false);
+// over finished fp32 logits [S, V]; an allowed set of the one id -1 is the whole vocabulary
+void launch_sample_dense(const float* logits, int S, int V, const int* allow_ptr,
+                         const int* allow_ids, const int* ctr, float temperature,
                          unsigned long long seed, int* out_tok, hipStream_t s);
 int launch_branch_select(const int* prev_tok, const int* tab, int n, int* ids, int* slots, int* q_len,
                          int* ctx_len, int* rows, int* aptr, int aptr_len, int* aids, int* err,

@@ -114,7 +114,8 @@ void append_ints(std::vector<int32_t>& dst, const py::handle& seq, Py_ssize_t li
 // One ragged step.  seqs: list of (tokens, take, start, blocks, kv_begin,
 // sample) - the first `take` of `tokens` enter at positions
 // [start, start + take) of a sequence whose KV blocks are `blocks`; `sample`
-// marks that its last token's hidden state is sampled.  Returns
+// marks that its last token's hidden state is sampled, or lists the places
+// among the new tokens whose hidden rows the step returns.  Returns
 // (host int32 array, layout) exactly like engine.batch.pack_host.
 py::tuple pack_step(const py::list& seqs, int block_size, int group, const py::object& copies,
                     const py::object& pre_bt, int pre_tokens, const py::object& allowed,
@@ -144,8 +145,17 @@ py::tuple pack_step(const py::list& seqs, int block_size, int group, const py::o
     q_len[s] = take;
     ctx_len[s] = start + take;
     kv_begin[s] = it[4].cast<int>();
+    if (PyList_Check(it[5].ptr()) || PyTuple_Check(it[5].ptr())) {
+      const size_t r0 = rows.size();
+      append_ints(rows, it[5]);
+      for (size_t r = r0; r < rows.size(); ++r) {
+        if (rows[r] < 0 || rows[r] >= take) throw std::invalid_argument("pack_step: row outside the span");
+        rows[r] += T;
+      }
+    } else if (it[5].cast<bool>()) {
+      rows.push_back(T + take - 1);
+    }
     T += take;
-    if (it[5].cast<bool>()) rows.push_back(T - 1);
     maxb = std::max(maxb, tab.size());
   }
   // attention work lists (engine.batch.build_work)

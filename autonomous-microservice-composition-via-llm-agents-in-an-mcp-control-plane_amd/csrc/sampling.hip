@@ -11,28 +11,40 @@
 #include "common.h"
 #include "kernels.h"
 
-__global__ __launch_bounds__(256) void sample_allowed_kernel(
-    const bf16* __restrict__ hidden, const bf16* __restrict__ W, const int* __restrict__ allow_ptr,
-    const int* __restrict__ allow_ids, const int* __restrict__ ctr, float inv_temp,
-    unsigned long long seed, int H, int* __restrict__ out_tok, float* __restrict__ out_logit) {
-  const int s = blockIdx.x;
-  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-  const int a0 = allow_ptr[s], a1 = allow_ptr[s + 1];
-  const bf16* h = hidden + (size_t)s * H;
-  const int nvec = H >> 3;
-  float best = -INFINITY, best_logit = 0.f;
-  int best_tok = -1;
-  for (int a = a0 + wave; a < a1; a += 4) {
-    const int tok = allow_ids[a];
-    const bf16* w = W + (size_t)tok * H;
-    float acc = 0.f;
-    for (int c = lane; c < nvec; c += 64) {
+// A model that scales or soft-caps its logits (z <- cap tanh(z scale / cap))
+// passes both; 1 and 0 leave the dot products as they are.
+template <class T>
+DEV float row_dot(const T* __restrict__ h, const T* __restrict__ w, int H, int lane) {
+  float acc = 0.f;
+  if constexpr (sizeof(T) == 2) {
+    for (int c = lane; c < (H >> 3); c += 64) {
       const bf16x8 x = reinterpret_cast<const bf16x8*>(h)[c];
       const bf16x8 y = reinterpret_cast<const bf16x8*>(w)[c];
 #pragma unroll
       for (int j = 0; j < 8; ++j) acc += (float)x[j] * (float)y[j];
     }
-    acc = wave_sum(acc);
+  } else {
+    for (int c = lane; c < H; c += 64) acc += h[c] * w[c];
+  }
+  return wave_sum(acc);
+}
+
+template <class T>
+__global__ __launch_bounds__(256) void sample_allowed_kernel(
+    const T* __restrict__ hidden, const T* __restrict__ W, const int* __restrict__ allow_ptr,
+    const int* __restrict__ allow_ids, const int* __restrict__ ctr, float inv_temp,
+    unsigned long long seed, int H, int* __restrict__ out_tok, float* __restrict__ out_logit,
+    float logit_scale, float logit_cap) {
+  const int s = blockIdx.x;
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const int a0 = allow_ptr[s], a1 = allow_ptr[s + 1];
+  const T* h = hidden + (size_t)s * H;
+  float best = -INFINITY, best_logit = 0.f;
+  int best_tok = -1;
+  for (int a = a0 + wave; a < a1; a += 4) {
+    const int tok = allow_ids[a];
+    float acc = row_dot(h, W + (size_t)tok * H, H, lane) * logit_scale;
+    if (logit_cap > 0.f) acc = logit_cap * tanhf(acc / logit_cap);
     float score = acc;
     if (inv_temp > 0.f) {
       const float u = uniform01(seed, (unsigned long long)(unsigned)ctr[s], (unsigned long long)tok);
@@ -64,51 +76,76 @@ __global__ __launch_bounds__(256) void sample_allowed_kernel(
 void launch_sample_allowed(const void* hidden, const void* W, const int* allow_ptr,
                            const int* allow_ids, const int* ctr, float temperature,
                            unsigned long long seed, int S, int H, int* out_tok, float* out_logit,
-                           hipStream_t s) {
+                           hipStream_t s, float logit_scale, float logit_cap, bool f32) {
   if (S <= 0) return;
   const float inv_t = temperature > 0.f ? 1.f / temperature : 0.f;
-  sample_allowed_kernel<<<S, 256, 0, s>>>((const bf16*)hidden, (const bf16*)W, allow_ptr,
-                                          allow_ids, ctr, inv_t, seed, H, out_tok, out_logit);
+  if (f32)
+    sample_allowed_kernel<float><<<S, 256, 0, s>>>((const float*)hidden, (const float*)W, allow_ptr,
+                                                   allow_ids, ctr, inv_t, seed, H, out_tok, out_logit,
+                                                   logit_scale, logit_cap);
+  else
+    sample_allowed_kernel<bf16><<<S, 256, 0, s>>>((const bf16*)hidden, (const bf16*)W, allow_ptr,
+                                                  allow_ids, ctr, inv_t, seed, H, out_tok, out_logit,
+                                                  logit_scale, logit_cap);
 }
 
-// Dense variant: logits [S, V] (fp32 or bf16 via the GEMM), optional -inf mask
-// folded in by the caller.  One block per row, Gumbel-max over the full vocab.
-__global__ __launch_bounds__(256) void sample_dense_kernel(const bf16* __restrict__ logits, int V,
-                                                           const int* __restrict__ ctr,
-                                                           float inv_temp,
-                                                           unsigned long long seed,
-                                                           int* __restrict__ out_tok) {
+// Dense form: finished fp32 logits [S, V] (free generation, where a step's
+// allowed set is the vocabulary).  One block per row; the row's allowed set is
+// {-1} for the whole vocabulary, a list of ids, or empty (token -1).
+__global__ __launch_bounds__(1024) void sample_dense_kernel(
+    const float* __restrict__ logits, int V, const int* __restrict__ allow_ptr,
+    const int* __restrict__ allow_ids, const int* __restrict__ ctr, float inv_temp,
+    unsigned long long seed, int* __restrict__ out_tok) {
   const int s = blockIdx.x;
-  const bf16* row = logits + (size_t)s * V;
+  const float* row = logits + (size_t)s * V;
+  const int a0 = allow_ptr[s], na = allow_ptr[s + 1] - a0;
+  const bool all = na == 1 && allow_ids[a0] < 0;
+  const int n = all ? V : na;
   float best = -INFINITY;
-  int bt = 0;
-  for (int i = threadIdx.x; i < V; i += 256) {
-    const float l = (float)row[i];
-    float sc = l;
-    if (inv_temp > 0.f) sc = l * inv_temp - __logf(-__logf(uniform01(seed, (unsigned long long)(unsigned)ctr[s], (unsigned long long)i)));
-    if (sc > best) { best = sc; bt = i; }
+  int bt = -1;
+  for (int i = threadIdx.x; i < n; i += 1024) {
+    const int tok = all ? i : allow_ids[a0 + i];
+    float sc = row[tok];
+    if (inv_temp > 0.f)
+      sc = sc * inv_temp -
+           __logf(-__logf(uniform01(seed, (unsigned long long)(unsigned)ctr[s], (unsigned long long)tok)));
+    if (sc > best || bt < 0) {
+      best = sc;
+      bt = tok;
+    }
   }
+  auto better = [](float ob, int ot, float b, int t) {
+    return ot >= 0 && (t < 0 || ob > b || (ob == b && ot < t));
+  };
   for (int o = 32; o > 0; o >>= 1) {
     const float ob = __shfl_xor(best, o, 64);
     const int ot = __shfl_xor(bt, o, 64);
-    if (ob > best || (ob == best && ot < bt)) { best = ob; bt = ot; }
+    if (better(ob, ot, best, bt)) {
+      best = ob;
+      bt = ot;
+    }
   }
-  __shared__ float sb[4];
-  __shared__ int st[4];
-  if ((threadIdx.x & 63) == 0) { sb[threadIdx.x >> 6] = best; st[threadIdx.x >> 6] = bt; }
+  __shared__ float sb[16];
+  __shared__ int st[16];
+  if ((threadIdx.x & 63) == 0) {
+    sb[threadIdx.x >> 6] = best;
+    st[threadIdx.x >> 6] = bt;
+  }
   __syncthreads();
   if (threadIdx.x == 0) {
     int bi = 0;
-    for (int i = 1; i < 4; ++i) if (sb[i] > sb[bi]) bi = i;
+    for (int i = 1; i < 16; ++i)
+      if (better(sb[i], st[i], sb[bi], st[bi])) bi = i;
     out_tok[s] = st[bi];
   }
 }
 
-void launch_sample_dense(const void* logits, int S, int V, const int* ctr, float temperature,
+void launch_sample_dense(const float* logits, int S, int V, const int* allow_ptr,
+                         const int* allow_ids, const int* ctr, float temperature,
                          unsigned long long seed, int* out_tok, hipStream_t s) {
   if (S <= 0) return;
   const float inv_t = temperature > 0.f ? 1.f / temperature : 0.f;
-  sample_dense_kernel<<<S, 256, 0, s>>>((const bf16*)logits, V, ctr, inv_t, seed, out_tok);
+  sample_dense_kernel<<<S, 1024, 0, s>>>(logits, V, allow_ptr, allow_ids, ctr, inv_t, seed, out_tok);
 }
 
 // Decision lookahead (engine MCP_LOOKAHEAD): the next forward was launched

@@ -273,6 +273,8 @@ def pack_step_py(entries, block_size: int, group: int, copies=None, pre_bt=None,
 
     ``entries``: (tokens, take, start, blocks, kv_begin, sample) per sequence;
     the first ``take`` tokens enter at positions [start, start + take).
+    ``sample``: True = the last of them feeds the sampler, or a list of places
+    among them whose hidden rows the step returns (in that order).
     Returns ``(host, layout)`` like ``pack_host``."""
     ids, pos, slots, rows = [], [], [], []
     q_start, q_len, ctx_len, kvb, tables = [], [], [], [], []
@@ -292,9 +294,13 @@ def pack_step_py(entries, block_size: int, group: int, copies=None, pre_bt=None,
         ctx_len.append(start + take)
         kvb.append(kv_begin)
         tables.append(blocks)
+        if isinstance(sample, (list, tuple)):
+            if any(not 0 <= r < take for r in sample):
+                raise ValueError("pack_step: row outside the span")
+            rows += [T + r for r in sample]
+        elif sample:
+            rows.append(T + take - 1)
         T += take
-        if sample:
-            rows.append(T - 1)
     S = len(entries)
     maxb = max([len(t) for t in tables] + [1])
     bt = np.zeros((S, maxb), np.int32)

@@ -33,6 +33,7 @@ import torch
 from .. import ops
 from ..utils.metrics import METRICS
 from ..utils.tracing import span
+from .decoders import FedDecoder
 from .batch import BLOCK_SIZE, HostStager, choose_kv_splits, pack_step, step_from_host, views
 from .kv_cache import KVCache
 
@@ -93,6 +94,10 @@ class Sequence:
         self.t_first = None
         self.t_done = None
         self.is_prefix_job = decoder is None
+        self.samples = getattr(decoder, "samples", True)   # False: tokens come from ``feed``
+        self.dense = getattr(decoder, "dense", False)      # samples from the whole vocabulary
+        self.want: List[int] = []              # positions whose logits are asked for, ascending
+        self.logits: Dict[int, np.ndarray] = {}   # position -> [vocab] fp32 logits
         self.cohort = 0                        # launch cohort (pipelined engine)
         if decoder is not None:
             first = decoder.advance()
@@ -101,7 +106,7 @@ class Sequence:
 
     @property
     def wants_sample(self) -> bool:
-        return self.decoder is not None and not self.decoder.done
+        return self.decoder is not None and self.samples and not self.decoder.done
 
 
 @dataclasses.dataclass
@@ -118,6 +123,8 @@ class _Launch:
     # per sequence, token -> (token, appended tokens, done, next allowed, decoder)
     seqs: Optional[list] = None
     branches: Optional[list] = None
+    scored: Optional[list] = None       # (sequence, position) of each row of ``logits``
+    logits: Optional[torch.Tensor] = None
 
 
 # MCP_SPIN_WAIT=1: busy-poll the sampled-token event (one host core per GPU
@@ -157,6 +164,17 @@ def tp_graph_safe(model) -> bool:
     return True
 
 
+def sample_step(model, hidden, dstep, temperature: float, seed: int, dense: bool = False):
+    """Tokens of a step's returned rows, drawn on the device."""
+    if dense:
+        return ops.sample_dense(model.logits(hidden).contiguous(), dstep.allow_ptr, dstep.allow_ids,
+                                dstep.sample_ctr, temperature, seed)
+    return ops.sample_allowed(hidden, model.w.lm_head, dstep.allow_ptr, dstep.allow_ids,
+                              dstep.sample_ctr, temperature, seed,
+                              logit_scale=getattr(model, "logit_scale", 1.0),
+                              logit_cap=getattr(model, "logit_cap", 0.0))
+
+
 _FEED_ADVANCE = False
 
 
@@ -178,10 +196,12 @@ class LLMEngine:
                  seed: int = 0, bcast=None, cascade: bool = True, pipeline: Optional[bool] = None,
                  graphs: Optional[bool] = None, lookahead: Optional[bool] = None):
         self.model = model
-        cfg = model.cfg
         self.device = model.device
         self.bcast = bcast          # parallel.comm.StepBroadcaster on a TP driver, else None
-        self.cascade = cascade and os.environ.get("MCP_CASCADE", "1") == "1"   # shared-prefix attention
+        # shared-prefix attention (a model whose attention has no one prefix for
+        # every later query opts out; its prefix blocks are shared all the same)
+        self.cascade = (cascade and os.environ.get("MCP_CASCADE", "1") == "1"
+                        and getattr(model, "supports_cascade", True))
         # optional two launch cohorts in flight: the host schedules / updates one
         # cohort while the GPU runs the other's forward.  Every cohort step
         # streams all the weights again, so a request waits two weight-bound
@@ -216,12 +236,10 @@ class LLMEngine:
                 graphs = bcast is not None and tp_graph_safe(model)
         self._graphs_wanted = graphs
         self.graphs = None          # engine.graphs.GraphRunner, created after the KV cache
-        if num_blocks is not None:
-            self.kv = KVCache(cfg.layers, model.hkv, cfg.head_dim, num_blocks, self.device)
-        else:
-            self.kv = KVCache.sized_for(cfg.layers, model.hkv, cfg.head_dim, self.device,
-                                        budget_bytes=kv_budget_bytes)
+        self.kv = KVCache.for_model(model, num_blocks, kv_budget_bytes)
         self.alloc = self.kv.allocator
+        # keys a span of new tokens attends (None: all of its context)
+        self._attended = getattr(model, "attended_keys", None)
         self.max_batch = max_batch
         self.max_step_tokens = max_step_tokens
         # chunked prefill (MCP_PREFILL_CHUNK tokens per step, 0 = off): while
@@ -507,6 +525,33 @@ class LLMEngine:
         self.waiting.append(seq)
         return seq
 
+    def open(self) -> Sequence:
+        """A request fed from outside: it takes tokens through ``feed``, never
+        samples, and holds its blocks until ``close``."""
+        return self.submit(FedDecoder(), [])
+
+    def feed(self, seq: Sequence, tokens: Seq[int], want: Seq[int] = ()) -> None:
+        """The next ``tokens`` of an ``open`` request; ``want``: places among
+        them whose logits ``step`` leaves in ``seq.logits`` (by position)."""
+        at = seq.base + len(seq.tokens)
+        max_pos = getattr(self.model.cfg, "max_pos", None)
+        if max_pos is not None and at + len(tokens) > max_pos:
+            raise ValueError(f"{at + len(tokens)} tokens do not fit the model's {max_pos}-token context")
+        if any(not 0 <= w < len(tokens) for w in want):
+            raise ValueError("feed: a wanted place is outside the tokens")
+        seq.want += sorted(at + w for w in want)
+        seq.pending += tokens
+        seq.tokens += tokens
+
+    def close(self, seq: Sequence) -> None:
+        """End an ``open`` request; its blocks go back to the pool."""
+        if seq.pending and not seq.done:
+            raise ValueError("close: the request still has tokens to run")
+        if not seq.done:
+            self._finish(seq)
+        self.running = [q for q in self.running if q is not seq]
+        self.waiting = [q for q in self.waiting if q is not seq]
+
     def abort_all(self, reason: str = "aborted") -> int:
         """Fail every queued and running request (their blocks go back to the
         allocator) and forget the prefix cache: the planner's recovery after a
@@ -598,7 +643,7 @@ class LLMEngine:
         seq.blocks = []
         if seq.is_prefix_job:
             seq.prefix_entry.computed = True
-        else:
+        elif seq.samples:
             t_parse = time.perf_counter()
             if seq.error is None:
                 try:
@@ -740,6 +785,7 @@ class LLMEngine:
                 (first if (q.prefix is casc and q.materialized) else rest).append(q)
             order = first + rest
         pre_tokens = 0
+        scored, kinds = [], []                 # (sequence, position); per returned row: sampled?
         casc_keys = (casc.length // BLOCK_SIZE) * BLOCK_SIZE if casc is not None else 0
         alloc, pool_free = self.alloc.alloc, self.alloc
         blocked = None
@@ -790,8 +836,17 @@ class LLMEngine:
             else:
                 ck = 0
             dec = seq.decoder
-            sample = take == n and dec is not None and not dec.done
-            add_entry((pend, take, start, blocks, ck, sample))
+            sample = take == n and dec is not None and seq.samples and not dec.done
+            rows = sample
+            if seq.want:                       # rows whose logits are asked for, then the sampled one
+                now = [p for p in seq.want if p < start + take]
+                seq.want = seq.want[len(now):]
+                scored += [(seq, p) for p in now]
+                kinds += [False] * len(now)
+                rows = [p - start for p in now] + ([take - 1] if sample else [])
+            if sample:
+                kinds.append(True)
+            add_entry((pend, take, start, blocks, ck, rows))
             add_batch((seq, take))
             if sample:
                 add_sample(seq)
@@ -832,14 +887,22 @@ class LLMEngine:
                 else:
                     allowed = [d.allowed() for d in decs]
             ctr = [(q.uid * 4096 + q.n_samples) & 0x7FFFFFFF for q in sample_seqs]
+        picks = None                           # rows of the step that are sampled (None: all)
+        if scored and sample_seqs:             # scored rows carry an empty allowed set
+            picks = [i for i, smp in enumerate(kinds) if smp]
+            it, ic = iter(allowed), iter(ctr)
+            allowed = [next(it) if smp else [] for smp in kinds]
+            ctr = [next(ic) if smp else 0 for smp in kinds]
+        dense = any(q.dense for q in sample_seqs)
         # a step that fits a captured bucket replays its hipGraph (prefix
         # copy-on-write, cascade and split-KV attention included)
         use_graph = (self.graphs is not None and T <= self.graphs.buckets[-1] and T <= _GRAPH_MAX_T
-                     and self.temperature == self.graphs.temperature)
+                     and self.temperature == self.graphs.temperature and not scored)
         cascade = pre_tokens > 0
         # split-KV for few long-context decode sequences (K6), over the keys
         # each sequence attends itself (after the cascade prefix, if any)
-        own_keys = [e[2] + e[1] - (e[4] if cascade else 0) for e in entries]
+        own_keys = [e[2] + e[1] - (e[4] if cascade else 0) for e in entries] \
+            if self._attended is None else [self._attended(e[2], e[1]) for e in entries]
         kv_splits = choose_kv_splits(
             [e[1] for e in entries], own_keys,
             group, self.model.hkv, hq=self.model.hq) if self.device.type == "cuda" else 1
@@ -855,8 +918,9 @@ class LLMEngine:
                 self.stats["kv_split_steps"] += 1
         t0 = time.perf_counter()
         self.stats["schedule_s"] += t0 - t_sched
-        tok_dev = self.graphs.run(step_from_host(host, layout), copies, kv_splits) \
+        tok_dev = self.graphs.run(step_from_host(host, layout), copies, kv_splits, dense=dense) \
             if use_graph else None
+        logits = None
         if tok_dev is not None:            # replayed hipGraph: forward + sampling
             self.stats["graph_steps"] += 1
             self.stats["graph_cow_steps"] += bool(copies)
@@ -867,7 +931,13 @@ class LLMEngine:
                 tokens, event = self._fetch(tok_dev[:len(sample_seqs)])
         else:
             hidden, dstep = self._launch(host, layout)
-            tok_dev = self._sample(hidden, dstep, len(sample_seqs))
+            if scored:
+                idx = [i for i, smp in enumerate(kinds) if not smp]
+                logits = self.model.logits(hidden if len(idx) == len(kinds) else
+                                           hidden[torch.tensor(idx, device=hidden.device)])
+            tok_dev = self._sample(hidden, dstep, len(sample_seqs), dense)
+            if picks is not None:
+                tok_dev = tok_dev[torch.tensor(picks, device=tok_dev.device)]
             tokens, event = self._fetch(tok_dev) if tok_dev is not None else (None, None)
         self.stats["launch_s"] += time.perf_counter() - t0
         if self.graphs is not None:
@@ -876,7 +946,8 @@ class LLMEngine:
         self.stats["tokens"] += T
         self.stats["steps"] += 1
         self.steps += 1
-        return _Launch(batch_seqs, sample_seqs, tokens, event, T, tok_dev=tok_dev)
+        return _Launch(batch_seqs, sample_seqs, tokens, event, T, tok_dev=tok_dev,
+                       scored=scored or None, logits=logits)
 
     # ------------------------------------------------------ decision lookahead
     LOOKAHEAD_MAX_SEQS = int(os.environ.get("MCP_LOOKAHEAD_MAX_SEQS", "8"))
@@ -1030,7 +1101,8 @@ class LLMEngine:
                 rel.append(rel[-1] + len(a))
             tab += [len(tail_sets)] + rel + [x for a in tail_sets for x in a]
         group = self.model.cfg.group
-        own_keys = [p[2] + p[3] for p in per] + [seq.num_cached + take for seq, take, _ in explicit]
+        spans = [(p[2], p[3]) for p in per] + [(seq.num_cached, take) for seq, take, _ in explicit]
+        own_keys = [sum(sp) if self._attended is None else self._attended(*sp) for sp in spans]
         q_lens = [p[3] for p in per] + [take for _, take, _ in explicit]
         kv_splits = choose_kv_splits(q_lens, own_keys, group, self.model.hkv,
                                      hq=self.model.hq) if self.device.type == "cuda" else 1
@@ -1226,6 +1298,10 @@ class LLMEngine:
         self.stats["sample_s"] += t2 - t1
         if self.bcast is not None:          # TP: a collective that timed out fails the step
             self.model.comm_check()
+        if L.scored:
+            rows = L.logits.float().cpu().numpy()
+            for (seq, pos), row in zip(L.scored, rows):
+                seq.logits[pos] = row
         batch_seqs, sample_seqs = L.batch_seqs, L.sample_seqs
         with span("retire.update"):
             self._update(batch_seqs, sample_seqs, new_tokens, booked=L.booked)
@@ -1281,7 +1357,7 @@ class LLMEngine:
         if pre is not None:
             pre(dstep)
         if csrc.numel():
-            ops.copy_blocks(self.kv.data, csrc, cdst)
+            self.kv.copy_blocks(csrc, cdst)
         if dstep.token_ids.numel() == 0:
             return None, dstep
         with span("launch.forward"):
@@ -1291,17 +1367,16 @@ class LLMEngine:
         if self.bcast is not None:
             self.bcast.stop()
 
-    def _sample(self, hidden: torch.Tensor, dstep, n: int) -> Optional[torch.Tensor]:
+    def _sample(self, hidden: torch.Tensor, dstep, n: int, dense: bool = False) -> Optional[torch.Tensor]:
         """Fused LM-head-rows + grammar mask + Gumbel-max sampling (K9) on the
-        allowed sets that travelled with the step descriptor.  The RNG counter
-        (request uid, sample index) makes every draw unique, so the seed is
-        constant (the same kernel runs inside captured hipGraphs)."""
+        allowed sets that travelled with the step descriptor; with ``dense``
+        (some request samples from the whole vocabulary) over full logits.  The
+        RNG counter (request uid, sample index) makes every draw unique, so the
+        seed is constant (the same kernel runs inside captured hipGraphs)."""
         if n == 0:
             return None
-        tok = ops.sample_allowed(hidden, self.model.w.lm_head, dstep.allow_ptr, dstep.allow_ids,
-                                 dstep.sample_ctr, self.temperature, self.seed)
         self.stats["samples"] += n
-        return tok
+        return sample_step(self.model, hidden, dstep, self.temperature, self.seed, dense)
 
     @staticmethod
     def _fetch(tok: torch.Tensor):

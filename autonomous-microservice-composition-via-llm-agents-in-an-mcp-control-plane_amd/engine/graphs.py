@@ -9,7 +9,8 @@ Python the launches, not the GPU, set the step time.  Steps with at most
 (``torch.cuda.CUDAGraph`` is the HIP graph API on ROCm).  A graph is keyed by
 (token bucket, sequence-capacity class, block-table width class, split-KV
 factor, cascade on / off), captured at start-up (``warm``) or lazily on first
-use, after one eager warm-up of the same static step.  Every step of
+use, after one eager warm-up of the same static step (the key's last entry also
+says whether the step samples from full logits: free generation).  Every step of
 a key uses ONE fixed int32 layout (``pack_static``):
 
 * tokens padded to the bucket size (padding writes no KV: slot -1), sequence
@@ -44,7 +45,6 @@ from typing import Dict, List, Optional, Sequence, Tuple
 import numpy as np
 import torch
 
-from .. import ops
 from ..utils.tracing import span
 from .batch import BLOCK_SIZE, HostStager, StepInputs, build_work, tokens_per_item, views
 
@@ -233,13 +233,13 @@ class GraphRunner:
 
     # ---------------------------------------------------------------- graphs
     def _body(self, e: _Bucket):
-        ops.copy_blocks(self.kv.data, e.csrc, e.cdst)
+        self.kv.copy_blocks(e.csrc, e.cdst)
         hidden = self.model.forward(e.dstep, self.kv)
         if not self.sample:
             return None
-        return ops.sample_allowed(hidden, self.model.w.lm_head, e.dstep.allow_ptr,
-                                  e.dstep.allow_ids, e.dstep.sample_ctr, self.temperature,
-                                  self.seed)
+        from .engine import sample_step
+        return sample_step(self.model, hidden, e.dstep, self.temperature, self.seed,
+                           dense=bool(e.key[4] & 2))
 
     def get(self, key) -> _Bucket:
         """The captured graph of ``key`` (capturing it on first use)."""
@@ -255,7 +255,8 @@ class GraphRunner:
         if e is not None:
             return e
         t0 = time.perf_counter()
-        b, sb, w, ns, casc = key
+        b, sb, w, ns, flags = key
+        casc = flags & 1
         sizes = self._sizes(b, w, sb)
         S_b = self._caps(b, sb)[0]
         buf = torch.zeros(sum(sizes), dtype=torch.int32, device=self.device)
@@ -311,7 +312,7 @@ class GraphRunner:
             for sb in self.seq_classes(b):
                 for w in widths:
                     for ns in kv_splits:
-                        for casc in (0, 1):
+                        for casc in self._warm_flags():
                             cap((b, sb, w, int(ns), casc), b, w, sb)
             if b <= self.WARM_SPLIT_MAX_TOKENS and self.device.type == "cuda":
                 for sb in self.seq_classes(b)[:self.WARM_SPLIT_SEQ_CLASSES]:
@@ -319,13 +320,16 @@ class GraphRunner:
                         for ns in self.WARM_SPLITS:
                             if ns in kv_splits:
                                 continue
-                            for casc in (0, 1):
+                            for casc in self._warm_flags():
                                 cap((b, sb, w, int(ns), casc), b, w, sb)
         self.warmed = True
         return self.captures - n0
 
+    def _warm_flags(self):
+        return (0, 1) if getattr(self.model, "supports_cascade", True) else (0,)
+
     def run(self, step: StepInputs, copies: Sequence = (), kv_splits: int = 1,
-            pre=None) -> Optional[torch.Tensor]:
+            pre=None, dense: bool = False) -> Optional[torch.Tensor]:
         """Replays the graph for ``step`` (after the prefix copy-on-write
         ``copies``); returns the device tensor of sampled tokens (first
         ``len(step.logit_rows)`` entries valid), or None when the step does
@@ -343,8 +347,9 @@ class GraphRunner:
             host = self.pack_static(step, b, w, copies, sb)
         if host is None:
             return None
-        casc = int(step.pre_tokens > 0 and step.pre_bt is not None and len(step.pre_bt) > 0)
-        key = (b, sb, w, int(kv_splits), casc)
+        flags = int(step.pre_tokens > 0 and step.pre_bt is not None and len(step.pre_bt) > 0)
+        flags |= 2 * bool(dense)
+        key = (b, sb, w, int(kv_splits), flags)
         if kv_splits > 1 and self.warmed and key not in self._b:
             return None        # an uncommon split key: eager, never a lazy capture mid-serving
         if self.bcast is not None:

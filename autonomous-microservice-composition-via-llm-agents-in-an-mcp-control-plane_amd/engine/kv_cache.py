@@ -8,6 +8,12 @@ Llama-3-8B needs 128 KiB per token, so ~200 GB holds ~1.6 M tokens.
 
 Blocks are reference counted so many requests can share the registry-prompt
 prefix blocks (prefix caching).
+
+A model whose cached layers differ in head count or head size, whose keys and
+values differ, or that runs a layer more than once (each run caches its own keys)
+gives one (kv_heads, key_dim, value_dim) per cached layer instead
+(``KVCache.from_specs``): same blocks and block ids, one stacked tensor per
+distinct (kv_heads, dim).
 """
 from __future__ import annotations
 
@@ -15,6 +21,7 @@ from typing import List, Optional
 
 import torch
 
+from .. import ops
 from . import native
 from .batch import BLOCK_SIZE
 
@@ -81,10 +88,56 @@ class KVCache:
         self.num_blocks = num_blocks
         self.data = torch.zeros(layers, 2, num_blocks, kv_heads, BLOCK_SIZE, head_dim,
                                 device=device, dtype=dtype)
+        self.stacks = [self.data]              # every tensor of the cache, [n, c, num_blocks, ...]
+        self._layer = [(self.data[l, 0], self.data[l, 1]) for l in range(layers)]
         self.allocator = make_allocator(num_blocks)
 
+    @classmethod
+    def from_specs(cls, specs, num_blocks: int, device, dtype=torch.bfloat16) -> "KVCache":
+        """``specs``: (kv_heads, key_dim, value_dim) of every cached layer."""
+        self = cls.__new__(cls)
+        self.layers, self.num_blocks, self.data = len(specs), num_blocks, None
+        place, count = [], {}
+        for h, dk, dv in specs:
+            for d in (dk, dv):
+                place.append(((h, d), count.get((h, d), 0)))
+                count[(h, d)] = count.get((h, d), 0) + 1
+        stack = {(h, d): torch.zeros(n, 1, num_blocks, h, BLOCK_SIZE, d, device=device, dtype=dtype)
+                 for (h, d), n in count.items()}
+        self.stacks = list(stack.values())
+        at = [stack[k][i, 0] for k, i in place]
+        self._layer = list(zip(at[0::2], at[1::2]))
+        self.allocator = make_allocator(num_blocks)
+        return self
+
+    @classmethod
+    def for_model(cls, model, num_blocks: Optional[int] = None, budget_bytes: Optional[int] = None):
+        """The cache of ``model``: its ``kv_specs`` when it has them, else equal
+        layers from its config.  ``num_blocks`` None: sized from free memory."""
+        specs = getattr(model, "kv_specs", None)
+        if specs is None:
+            cfg = model.cfg
+            if num_blocks is not None:
+                return cls(cfg.layers, model.hkv, cfg.head_dim, num_blocks, model.device)
+            return cls.sized_for(cfg.layers, model.hkv, cfg.head_dim, model.device,
+                                 budget_bytes=budget_bytes)
+        if num_blocks is None:
+            size = torch.empty(0, dtype=model.dtype).element_size()
+            per = sum(h * (dk + dv) for h, dk, dv in specs) * BLOCK_SIZE * size
+            num_blocks = cls._blocks_in_budget(per, model.device, budget_bytes)
+        return cls.from_specs(specs, num_blocks, model.device, model.dtype)
+
     def layer(self, l: int):
-        return self.data[l, 0], self.data[l, 1]
+        return self._layer[l]
+
+    def copy_blocks(self, src, dst) -> None:
+        """Block src[i] -> dst[i] in every cached layer (negative pairs: none)."""
+        for t in self.stacks:
+            ops.copy_blocks(t, src, dst)
+
+    @property
+    def nbytes(self) -> int:
+        return sum(t.numel() * t.element_size() for t in self.stacks)
 
     @staticmethod
     def bytes_per_block(layers, kv_heads, head_dim, dtype_bytes=2) -> int:
@@ -94,6 +147,14 @@ class KVCache:
     def sized_for(cls, layers, kv_heads, head_dim, device, budget_bytes: Optional[int] = None,
                   max_blocks: Optional[int] = None, reserve_frac: float = 0.1):
         per = cls.bytes_per_block(layers, kv_heads, head_dim)
+        n = cls._blocks_in_budget(per, device, budget_bytes, reserve_frac)
+        if max_blocks is not None:
+            n = min(n, max_blocks)
+        return cls(layers, kv_heads, head_dim, n, device)
+
+    @staticmethod
+    def _blocks_in_budget(per: int, device, budget_bytes: Optional[int],
+                          reserve_frac: float = 0.1) -> int:
         dev = torch.device(device)
         if budget_bytes is None:
             if dev.type == "cuda":
@@ -101,7 +162,4 @@ class KVCache:
                 budget_bytes = int(free - reserve_frac * total)
             else:
                 budget_bytes = 256 * per
-        n = max(16, budget_bytes // per)
-        if max_blocks is not None:
-            n = min(n, max_blocks)
-        return cls(layers, kv_heads, head_dim, int(n), device)
+        return int(max(16, budget_bytes // per))

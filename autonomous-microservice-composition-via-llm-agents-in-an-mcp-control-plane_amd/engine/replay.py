@@ -1,0 +1,103 @@
+"""Replay of a token trace: given ids through a model, step by step, logits out.
+
+    python -m mcp_amd.engine.replay --model DIR --dtype bfloat16|float32 --out DIR --max-tokens N
+
+(``bin/trace_run`` builds the kernels if needed and runs this.)  Steps come on
+standard input, one JSON object a line:
+
+    {"step": 0, "entries": [{"id": "a", "tokens": [5, 17], "want": [1]}], "end": []}
+
+Each entry brings a request's next tokens; ``want`` lists the places among them
+whose logits are wanted, ``end`` the requests that are over after the step.  All
+entries of a step run as one batch of the engine, from its paged cache.  A step
+with wanted places writes ``<out>/<step>.f32`` (entry order, little-endian fp32,
+[wanted, vocab]); every step prints ``done <step>``.
+
+The engine is the serving engine: its scheduler batches the entries
+(``LLMEngine.feed``), its block allocator places them, its model runs them; the
+pool holds ``--max-tokens`` tokens in whole blocks, so finished requests' blocks
+are used again.
+"""
+from __future__ import annotations
+
+import argparse
+import json
+import os
+import sys
+
+import numpy as np
+import torch
+
+MAX_LIVE = 4                     # live requests of a trace
+
+
+class Replay:
+    def __init__(self, model, max_tokens: int, vocab: int, max_live: int = MAX_LIVE):
+        from .batch import BLOCK_SIZE
+        from .engine import LLMEngine
+        self.vocab = vocab
+        blocks = max(1, -(-max_tokens // BLOCK_SIZE))
+        self.engine = LLMEngine(model, num_blocks=blocks, max_batch=max_live,
+                                max_step_tokens=blocks * BLOCK_SIZE, temperature=0.0,
+                                graphs=False, lookahead=False, pipeline=False)
+        self.live = {}
+
+    def step(self, entries, end=()):
+        """Run one step's entries as one batch; [wanted, vocab] fp32 or None."""
+        eng, order = self.engine, []
+        for e in entries:
+            seq = self.live.get(e["id"])
+            if seq is None:
+                seq = self.live[e["id"]] = eng.open()
+            at = seq.base + len(seq.tokens)
+            eng.feed(seq, e["tokens"], e["want"])
+            order += [(seq, at + w) for w in e["want"]]
+        idle = 0
+        while any(q.pending for q in self.live.values()):
+            idle = idle + 1 if eng.step() == 0 else 0
+            if idle > 8:
+                raise RuntimeError(f"no room for the step's tokens: {eng.alloc.num_free} of "
+                                   f"{eng.kv.num_blocks} blocks free")
+        for q in self.live.values():
+            if q.error:
+                raise RuntimeError(q.error)
+        out = np.stack([seq.logits[p] for seq, p in order]) if order else None
+        for seq, _ in order:
+            seq.logits.clear()
+        for i in end:
+            eng.close(self.live.pop(i))
+        return out
+
+
+def main(argv=None) -> int:
+    ap = argparse.ArgumentParser(description="replay a token trace, writing logits")
+    ap.add_argument("--model", required=True, help="checkpoint directory")
+    ap.add_argument("--dtype", choices=("bfloat16", "float32"), default="bfloat16")
+    ap.add_argument("--out", required=True, help="directory of the logits files")
+    ap.add_argument("--max-tokens", type=int, required=True,
+                    help="most tokens live requests hold at a time (the cache pool)")
+    a = ap.parse_args(argv)
+    from ..models.registry import load_model
+    if not torch.cuda.is_available():
+        raise RuntimeError("no GPU: the kernels run on gfx950")
+    try:
+        model = load_model(a.model, "cuda:0", dtype=getattr(torch, a.dtype), max_pos=a.max_tokens + 64)
+    except NotImplementedError as e:
+        if a.dtype == "float32":
+            print(e, file=sys.stderr)
+            return 3
+        raise
+    run = Replay(model, a.max_tokens, model.cfg.vocab_size)
+    for line in sys.stdin:
+        if not line.strip():
+            continue
+        s = json.loads(line)
+        z = run.step(s["entries"], s.get("end", ()))
+        if z is not None:
+            z.astype("<f4").tofile(os.path.join(a.out, f"{s['step']}.f32"))
+        print(f"done {s['step']}", flush=True)
+    return 0
+
+
+if __name__ == "__main__":
+    sys.exit(main())

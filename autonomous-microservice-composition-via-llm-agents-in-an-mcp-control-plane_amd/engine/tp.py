@@ -15,7 +15,6 @@ from __future__ import annotations
 import torch
 import torch.distributed as dist
 
-from .. import ops
 from ..parallel.comm import StepBroadcaster
 from .batch import views
 
@@ -64,7 +63,7 @@ def worker_loop(model, kv, bcast: StepBroadcaster) -> int:
             continue
         dstep, csrc, cdst = views(payload, layout)
         if csrc.numel():
-            ops.copy_blocks(kv.data, csrc, cdst)
+            kv.copy_blocks(csrc, cdst)
         if dstep.token_ids.numel():
             model.forward(dstep, kv)
         model.comm_check()          # K12 peer timeout -> hard failure (lags <= 1 step)

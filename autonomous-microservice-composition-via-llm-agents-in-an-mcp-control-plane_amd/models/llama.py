@@ -355,6 +355,10 @@ class LlamaModel:
         if chk is not None:
             chk()
 
+    def logits(self, hidden: torch.Tensor) -> torch.Tensor:
+        """[R, V] fp32 logits of ``forward``'s rows (free generation, scoring)."""
+        return ops.gemm_f32out(hidden, self.w.lm_head)
+
     # --------------------------------------------------------------- forward
     def _residual_gemm(self, a: torch.Tensor, w: torch.Tensor, x: torch.Tensor) -> torch.Tensor:
         """x + a w^T with the residual add fused in the GEMM epilogue; for TP the

@@ -195,11 +195,18 @@ def save_llama_safetensors(cfg: LlamaConfig, w: LlamaWeights, path, shard_layers
            if cfg.rope_scaling else {})}, indent=1))
 
 
-def model_from_checkpoint(path, device, tp_rank: int = 0, tp: int = 1, tp_group=None):
+def llama_from_checkpoint(path, device, tp_rank: int = 0, tp: int = 1, tp_group=None):
     """LlamaModel over an HF safetensors checkpoint directory."""
     from .llama import LlamaModel
     cfg, w = load_llama_safetensors(path, device, tp_rank=tp_rank, tp=tp)
     return LlamaModel(cfg, w, device, tp_rank, tp, tp_group)
+
+
+def model_from_checkpoint(path, device, tp_rank: int = 0, tp: int = 1, tp_group=None):
+    """The model of whatever architecture the checkpoint directory holds
+    (``models.registry``)."""
+    from .registry import load_model
+    return load_model(path, device, tp_rank, tp, tp_group)
 
 
 def checkpoint_dir_from_env() -> Optional[str]:

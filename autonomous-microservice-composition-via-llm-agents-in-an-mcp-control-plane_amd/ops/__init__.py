@@ -173,12 +173,60 @@ def gemm(X, W, R=None, out=None, algo: int = -1, ss_out=None):
         if _TRACE is not None:
             _trace(X, W, "gemm" if R is None else "gemm+res")
         out = X.new_empty(*X.shape[:-1], W.shape[0]) if out is None else out
-        lib().gemm(X, W, out, R, algo, ss_out)
+        if X.dtype == torch.float32:              # the 32-bit mode: plain products only
+            if R is not None or ss_out is not None:
+                raise NotImplementedError("float32 gemm: no residual epilogue")
+            lib().gemm_f32(X, W, out)
+        else:
+            lib().gemm(X, W, out, R, algo, ss_out)
         return out
     r = ref.gemm(X, W, R)
     if ss_out is not None:
         ss_out[:r.shape[0]] += ref.row_sumsq(r)
     return r if out is None else out.copy_(r)
+
+
+def gemm_f32out(X, W, out=None):
+    """Y = X @ W^T with the fp32 accumulators stored as they are (bf16 or f32
+    operands): products that enter an fp32 stream or the logits."""
+    if X.is_cuda:
+        out = torch.empty(*X.shape[:-1], W.shape[0], device=X.device, dtype=torch.float32) \
+            if out is None else out
+        (lib().gemm_f32 if X.dtype == torch.float32 else lib().gemm_f32out)(X, W, out)
+        return out
+    r = X.float() @ W.float().t()
+    return r if out is None else out.copy_(r)
+
+
+def embedding_scaled(ids, table, scale: float, lo=None):
+    """table[ids] * scale as the fp32 residual; ``lo`` ([T, H], row-strided
+    views too) also gets the rows in its own type."""
+    if table.is_cuda:
+        x = torch.empty(ids.numel(), table.shape[1], device=table.device, dtype=torch.float32)
+        lib().embedding_scaled(ids, table, float(scale), x, lo)
+        return x
+    x = table[ids.long()].float() * scale
+    if lo is not None:
+        lo.copy_(x)
+    return x
+
+
+def residual_norm(x, H: int, eps: float, y=None, w_post=None, w_pre=None, out=None):
+    """One pass over the fp32 residual ``x`` [T, Hp] (in place; means over the
+    first ``H`` columns, the rest are zero): x += rms(y) * w_post when ``y`` is
+    given, then ``out`` = rms(x) * w_pre, or x itself without ``w_pre``."""
+    if x.is_cuda:
+        lib().residual_norm(x, y, w_post, w_pre, out, int(H), float(eps))
+        return out
+    return ref.residual_norm(x, H, eps, y, w_post, w_pre, out)
+
+
+def logit_finish(z, scale: float = 1.0, cap: float = 0.0):
+    """z <- cap tanh(z scale / cap) in place (``cap`` 0: z scale)."""
+    if z.is_cuda:
+        lib().logit_finish(z, float(scale), float(cap))
+        return z
+    return z.copy_(ref.soft_cap(z * scale, cap))
 
 
 _PF_SINK = {}
@@ -205,18 +253,27 @@ def weight_prefetch_init(device):
     return sink
 
 
-def gemm_silu(X, W, out=None, ss_in=None, eps: float = 0.0):
-    """SwiGLU projection: silu(X Wg^T) * (X Wu^T) with W = interleave_gate_up(Wg, Wu)
-    ([2F, K], 16-row groups); the activation is fused into the MFMA GEMM epilogue.
+GATED_ACTS = {"silu": 0, "gelu_tanh": 1}        # csrc/kernels.h GatedAct
+
+
+def gemm_silu(X, W, out=None, ss_in=None, eps: float = 0.0, act: str = "silu"):
+    """Gated projection: act(X Wg^T) * (X Wu^T) with W = interleave_gate_up(Wg, Wu)
+    ([2F, K], 16-row groups); the activation (``silu``: SwiGLU, or ``gelu_tanh``)
+    is fused into the MFMA GEMM epilogue.
     ``ss_in`` (int64 [M]): fused RMSNorm - the accumulators of row m are scaled
     by rsqrt(ss_in[m] / K + eps) first (the norm weight folded into W)."""
     if X.is_cuda:
         if _TRACE is not None:
             _trace(X, W, "swiglu")
         out = X.new_empty(*X.shape[:-1], W.shape[0] // 2) if out is None else out
-        lib().gemm_silu(X, W, out, ss_in, eps)
+        if X.dtype == torch.float32:
+            z = X.new_empty(*X.shape[:-1], W.shape[0])
+            lib().gemm_f32(X, W, z)
+            lib().gated_act_f32(z, out, GATED_ACTS[act])
+        else:
+            lib().gemm_silu(X, W, out, ss_in, eps, GATED_ACTS[act])
         return out
-    r = ref.gemm_silu(X, W, ss_in, eps)
+    r = ref.gemm_silu(X, W, ss_in, eps, act)
     return r if out is None else out.copy_(r)
 
 
@@ -250,6 +307,21 @@ def qkv_rope(h, wqkv, pos, slots, cos_sin, q_out, k_cache, v_cache, Hq, Hkv, D, 
     else:
         qkv = ref.gemm(h, wqkv)
     ref.rope_kv(qkv, pos, slots, cos_sin, q_out, k_cache, v_cache, Hq, Hkv, D)
+    return q_out
+
+
+def qkv_rope_bias(h, wqkv, bias, pos, slots, cos_sin, q_out, k_cache, v_cache):
+    """``qkv_rope`` with projection biases (fp32 [N]) and key / value heads of
+    any sizes (multiples of 8): sizes come from q_out [T, Hq, DK] and the
+    caches.  Pairs that do not rotate hold (1, 0) in ``cos_sin``."""
+    if h.is_cuda:
+        qkv = gemm(h, wqkv)
+        lib().rope_kv_any(qkv, bias, pos, slots, cos_sin, q_out, k_cache, v_cache)
+        return q_out
+    qkv = h.float() @ wqkv.float().t()
+    if bias is not None:
+        qkv = qkv + bias
+    ref.rope_kv_any(qkv, pos, slots, cos_sin, q_out, k_cache, v_cache)
     return q_out
 
 
@@ -515,17 +587,55 @@ def paged_attention(q, k_cache, v_cache, meta, scale, out=None):
     return r if out is None else out.copy_(r)
 
 
+def masked_attention(q, k_cache, v_cache, meta, scale, soft_cap: float = 0.0, chunk: int = 0,
+                     sink: bool = False):
+    """Paged causal attention, q [T, Hq, DK] -> [T, Hq, DV], with the score
+    soft cap (s <- cap tanh(s / cap); 0 = none), the chunked mask (keys of the
+    query's own ``chunk``-token stretch of the sequence; 0 = all earlier keys)
+    and the softmax sink (one added to the denominator)."""
+    if q.is_cuda:
+        out = torch.empty(q.shape[0], q.shape[1], v_cache.shape[3], device=q.device, dtype=q.dtype)
+        lib().attention_row(q, k_cache, v_cache, out, meta.q_start, meta.q_len, meta.ctx_len,
+                            meta.block_table, float(scale), float(soft_cap), int(chunk), bool(sink))
+        return out
+    return ref.masked_attention(q, k_cache, v_cache, meta.q_start, meta.q_len, meta.ctx_len,
+                                meta.block_table, scale, soft_cap, chunk, sink)
+
+
+def sample_dense(logits, allow_ptr, allow_ids, ctr, temperature, seed):
+    """Gumbel-max (greedy at temperature 0) over finished fp32 logits [R, V];
+    a row's allowed set is a list of ids or {-1}, the whole vocabulary."""
+    if logits.is_cuda:
+        out = torch.empty(logits.shape[0], dtype=torch.int32, device=logits.device)
+        lib().sample_dense(logits, allow_ptr, allow_ids, ctr, temperature, seed, out)
+        return out
+    rows = []
+    for i in range(logits.shape[0]):
+        ids = allow_ids[int(allow_ptr[i]):int(allow_ptr[i + 1])].long()
+        if len(ids) == 1 and int(ids[0]) < 0:
+            ids = torch.arange(logits.shape[1])
+        rows.append((ids, logits[i, ids]))
+    return _draw(rows, ctr, temperature, seed)
+
+
 def sample_allowed(hidden, W, allow_ptr, allow_ids, ctr, temperature, seed, out_tok=None,
-                   out_logit=None):
+                   out_logit=None, logit_scale: float = 1.0, logit_cap: float = 0.0):
     if hidden.is_cuda:
         out_tok = torch.empty(hidden.shape[0], dtype=torch.int32, device=hidden.device) \
             if out_tok is None else out_tok
         lib().sample_allowed(hidden, W, allow_ptr, allow_ids, ctr, temperature, seed, out_tok,
-                             out_logit)
+                             out_logit, logit_scale, logit_cap)
         return out_tok
+    rows = [(ids, ref.soft_cap(z * logit_scale, logit_cap)) for ids, z in
+            ref.sample_allowed_logits(hidden, W, allow_ptr, allow_ids)]
+    t = _draw(rows, ctr, temperature, seed)
+    return t if out_tok is None else out_tok.copy_(t)
+
+
+def _draw(rows, ctr, temperature, seed):
     # CPU: same Gumbel-max semantics with torch's RNG, one stream per (seed, counter)
     toks = []
-    for i, (ids, logits) in enumerate(ref.sample_allowed_logits(hidden, W, allow_ptr, allow_ids)):
+    for i, (ids, logits) in enumerate(rows):
         if len(ids) == 0:
             toks.append(-1)
             continue
@@ -536,8 +646,7 @@ def sample_allowed(hidden, W, allow_ptr, allow_ids, ctr, temperature, seed, out_
         else:
             sc = logits
         toks.append(int(ids[int(torch.argmax(sc))]))
-    t = torch.tensor(toks, dtype=torch.int32)
-    return t if out_tok is None else out_tok.copy_(t)
+    return torch.tensor(toks, dtype=torch.int32)
 
 
 def branch_select(prev_tok, tab, n: int, dstep, err):
@@ -670,7 +779,9 @@ def topk_cosine(queries, corpus, k: int, seg_len: int = 4096, n_valid: Optional[
 def copy_blocks(kv_data, src, dst):
     """kv_data [L, 2, nb, Hkv, BS, D]: copy block src[i] -> dst[i] (all layers, K and V)."""
     if kv_data.is_cuda:
-        lib().copy_blocks(kv_data, src, dst)
+        # (a float32 cache moves as bf16 words of twice the width)
+        lib().copy_blocks(kv_data if kv_data.dtype == torch.bfloat16 else kv_data.view(torch.bfloat16),
+                          src, dst)
     else:
         keep = (src >= 0) & (dst >= 0)          # negative pairs are padding
         kv_data[:, :, dst[keep].long()] = kv_data[:, :, src[keep].long()]

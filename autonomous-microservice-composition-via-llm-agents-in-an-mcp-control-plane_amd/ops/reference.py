@@ -59,14 +59,19 @@ def norm_row_scale(ss: torch.Tensor, H: int, eps: float) -> torch.Tensor:
     return torch.rsqrt(ss.double().div(SS_FIX).float() / H + eps).unsqueeze(-1)
 
 
-def gemm_silu(X, W_interleaved, ss_in=None, eps: float = 0.0):
+def gelu_tanh(z):
+    return 0.5 * z * (1 + torch.tanh(math.sqrt(2 / math.pi) * (z + 0.044715 * z ** 3)))
+
+
+def gemm_silu(X, W_interleaved, ss_in=None, eps: float = 0.0, act: str = "silu"):
     y = (X.float() @ W_interleaved.float().t())
     if ss_in is not None:                      # fused RMSNorm: rows scaled after the GEMM
         y = y * norm_row_scale(ss_in[:X.shape[0]], X.shape[-1], eps)
     T, F2 = y.shape
     y = y.view(T, F2 // (2 * GU_GROUP), 2, GU_GROUP)
     g, u = y[:, :, 0], y[:, :, 1]
-    return (torch.nn.functional.silu(g) * u).reshape(T, F2 // 2).to(X.dtype)
+    f = {"silu": torch.nn.functional.silu, "gelu_tanh": gelu_tanh}[act]
+    return (f(g) * u).reshape(T, F2 // 2).to(X.dtype)
 
 
 def gemm(X, W, R: Optional[torch.Tensor] = None):
@@ -151,6 +156,65 @@ def paged_attention(q, k_cache, v_cache, q_start, q_len, ctx_len, block_table, s
         S = S.masked_fill(kpos > qpos, float("-inf"))
         P = torch.softmax(S, dim=-1)
         out[qs:qs + ql] = (P @ V).transpose(0, 1).to(q.dtype)
+    return out
+
+
+def soft_cap(z, cap: float):
+    return cap * torch.tanh(z / cap) if cap > 0 else z
+
+
+def residual_norm(x, H, eps, y=None, w_post=None, w_pre=None, out=None):
+    def norm(v, w):
+        v = v.float()
+        return v / torch.sqrt((v[:, :H] ** 2).mean(-1, keepdim=True) + eps) * w
+    if y is not None:
+        x += norm(y, w_post)
+    if out is not None:
+        out.copy_(x if w_pre is None else norm(x, w_pre))
+    return out
+
+
+def rope_kv_any(qkv, pos, slots, cos_sin, q_out, k_cache, v_cache):
+    """qkv [T, Hq DK + Hkv DK + Hkv DV] fp32; halves rotate (dimension j with
+    j + DK / 2), values pass."""
+    T, Hq, DK = q_out.shape
+    Hkv, BS, DV = k_cache.shape[1], k_cache.shape[2], v_cache.shape[3]
+    q, k, v = torch.split(qkv, [Hq * DK, Hkv * DK, Hkv * DV], dim=-1)
+    q_out.copy_(apply_rope(q.reshape(T, Hq, DK), pos, cos_sin))
+    k = apply_rope(k.reshape(T, Hkv, DK), pos, cos_sin).to(k_cache.dtype)
+    v = v.reshape(T, Hkv, DV).to(v_cache.dtype)
+    on = slots >= 0
+    b, o = (slots[on] // BS).long(), (slots[on] % BS).long()
+    k_cache[b, :, o] = k[on]
+    v_cache[b, :, o] = v[on]
+
+
+def masked_attention(q, k_cache, v_cache, q_start, q_len, ctx_len, block_table, scale,
+                     cap=0.0, chunk=0, sink=False):
+    T, Hq, DK = q.shape
+    Hkv, BS, DV = k_cache.shape[1], k_cache.shape[2], v_cache.shape[3]
+    out = q.new_zeros(T, Hq, DV)
+    for s in range(q_start.numel()):
+        qs, ql, cl = int(q_start[s]), int(q_len[s]), int(ctx_len[s])
+        if ql == 0:
+            continue
+        blocks = block_table[s, :(cl + BS - 1) // BS].long()
+        K = k_cache[blocks].permute(1, 0, 2, 3).reshape(Hkv, -1, DK)[:, :cl].float()
+        V = v_cache[blocks].permute(1, 0, 2, 3).reshape(Hkv, -1, DV)[:, :cl].float()
+        Q = q[qs:qs + ql].float().view(ql, Hkv, Hq // Hkv, DK).permute(1, 2, 0, 3)
+        S = soft_cap(Q @ K.unsqueeze(1).transpose(2, 3) * scale, cap)
+        i = torch.arange(cl - ql, cl).unsqueeze(1)
+        j = torch.arange(cl).unsqueeze(0)
+        ok = j <= i
+        if chunk:
+            ok = ok & (j // chunk == i // chunk)
+        S = S.masked_fill(~ok, float("-inf"))
+        m = S.amax(-1, keepdim=True)
+        if sink:
+            m = m.clamp(min=0)
+        P = torch.exp(S - m)
+        den = P.sum(-1, keepdim=True) + (torch.exp(-m) if sink else 0)
+        out[qs:qs + ql] = (P / den @ V.unsqueeze(1)).permute(2, 0, 1, 3).reshape(ql, Hq, DV).to(q.dtype)
     return out
 
 

@@ -139,7 +139,6 @@ def _replica_main(idx: int, device: str, cfg: ReplicaConfig, records: list, vers
         return
     import torch
     from ..engine.engine import LLMEngine
-    from ..models.llama import LlamaModel
     from ..planner.local import LocalPlanner
     from ..registry import MemoryRegistry, RedisRegistry
     from ..retrieval.store import SchemaIndex
@@ -157,15 +156,16 @@ def _replica_main(idx: int, device: str, cfg: ReplicaConfig, records: list, vers
                                   cfg.full_weights_seed)
         kw = {"num_blocks": nb}
     else:
-        if os.path.isdir(cfg.model):                   # an HF checkpoint directory
+        if os.path.isdir(cfg.model):                   # a checkpoint directory
             from ..models.weights import model_from_checkpoint
             m = model_from_checkpoint(cfg.model, device)
         elif cfg.full_weights_seed is not None:
-            from ..models.llama import get_config, random_weights
+            from ..models.llama import LlamaModel, get_config, random_weights
             mc = get_config(cfg.model)
             m = LlamaModel(mc, random_weights(mc, device, seed=cfg.full_weights_seed), device)
         else:
-            m = LlamaModel.random(cfg.model, device, seed=cfg.seed)
+            from ..models.registry import random_model
+            m = random_model(cfg.model, device, seed=cfg.seed)
         kw = {"num_blocks": cfg.num_blocks} if cfg.num_blocks else {}
     eng = LLMEngine(m, max_batch=cfg.max_batch, max_step_tokens=cfg.max_step_tokens,
                     temperature=cfg.temperature, seed=cfg.seed + idx, bcast=bcast, **kw)

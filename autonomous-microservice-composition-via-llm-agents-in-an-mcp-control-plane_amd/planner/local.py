@@ -85,14 +85,14 @@ class LocalPlanner(Planner):
     def from_settings(cls, settings, registry):
         import torch
         from ..engine.engine import LLMEngine
-        from ..models.llama import LlamaModel
+        from ..models.registry import random_model
         from ..retrieval.store import SchemaIndex
         from ..models.weights import model_from_checkpoint
         dev = "cuda:0" if torch.cuda.is_available() else "cpu"
-        if os.path.isdir(settings.model):        # an HF safetensors checkpoint directory
+        if os.path.isdir(settings.model):        # a safetensors checkpoint directory
             model = model_from_checkpoint(settings.model, dev)
         else:                                     # a named architecture, random-init weights
-            model = LlamaModel.random(settings.model, dev, seed=settings.seed)
+            model = random_model(settings.model, dev, seed=settings.seed)
         kw = {} if dev != "cpu" else {"num_blocks": 512}
         if getattr(settings, "kv_blocks", 0):
             kw["num_blocks"] = settings.kv_blocks

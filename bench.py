@@ -131,7 +131,7 @@ def main():
     engine = LLMEngine(model, max_batch=2 * args.batch + 8, max_step_tokens=args.max_step_tokens,
                        temperature=0.2, seed=args.seed + rank, **kw)
     log(f"[rank {rank}] KV cache: {engine.kv.num_blocks} blocks x 64 tokens "
-        f"({engine.kv.data.numel() * 2 / 1e9:.1f} GB)")
+        f"({engine.kv.nbytes / 1e9:.1f} GB)")
     reg = MemoryRegistry(synthetic_registry(args.services, seed=1))
     planner = LocalPlanner(engine, reg, max_nodes=args.max_nodes, min_nodes=args.min_nodes)
     names = [s.name for s in reg.list_services()]
