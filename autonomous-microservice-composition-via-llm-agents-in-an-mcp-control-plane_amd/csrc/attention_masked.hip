@@ -6,12 +6,137 @@
 //
 // Layouts: q [T, Hq, DK], k cache [num_blocks, Hkv, 64, DK], v cache
 // [num_blocks, Hkv, 64, DV], out [T, Hq, DV].
+//
+// Three forms:
+//   tile   4-wave work items (prompt portions): the item's tokens x G heads are
+//          rows, 16 per wave; K / V tiles of one 64-key block go through LDS
+//          (LDS-DMA) and are shared by the waves;
+//   split  1-wave work items (decode): one 16-row tile, the keys shared out over
+//          the 4 waves of a block and over gridDim.z blocks, K straight into MFMA
+//          registers, V through a per-wave LDS buffer; merged in LDS, then (z > 1)
+//          by attn_split_merge;
+//   row    one wave per (token, head), fp32: the 32-bit mode, odd head sizes.
+// Both MFMA forms compute S^T = K Q^T (v_mfma_f32_16x16x32_bf16; a lane owns one
+// query row), then O^T += V^T P^T with P^T straight from the S^T accumulators and
+// V^T from transposed LDS reads, as attention.hip does.
+//
+// Softmax.  The sink is a key of score 0 without a value: a running sum that
+// starts at m = 0, l = 1.  A soft cap bounds every score by +-cap, so while
+// e^cap is far inside fp32 (cap <= NOMAX_CAP) the weights e^s need no running
+// maximum at all: no row reductions and no rescaling inside the key loop, and
+// partial sums over keys (waves, splits) simply add.
 #include "common.h"
 #include "kernels.h"
 
 namespace {
 
 constexpr int KT = 64;                        // keys per cache block
+
+typedef __attribute__((ext_vector_type(4))) short s16x4;
+constexpr float LOG2E = 1.4426950408889634f;
+constexpr float NOMAX_CAP = 60.f;             // e^60 x 1e6 keys is far below fp32's range
+
+enum { PLAIN = 0, CAPPED = 1, CAPPED_NOMAX = 2 };   // score forms
+
+DEV bf16x4 tr_read(const bf16* p) {
+  s16x4 v = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) s16x4*)(p));
+  return __builtin_bit_cast(bf16x4, v);
+}
+
+// Score constants (log2 units): PLAIN s = acc a; CAPPED s = C tanh(acc scale / cap)
+// = C - 2 C / (1 + 2^(acc a)), a = 2 log2(e) scale / cap, C = cap log2(e)
+struct ScoreConst {
+  float a, c;
+};
+template <int MODE>
+DEV ScoreConst score_const(const MaskedAttnArgs& p) {
+  if constexpr (MODE == PLAIN) return {p.scale * LOG2E, 0.f};
+  return {2.f * LOG2E * p.scale / p.cap, p.cap * LOG2E};
+}
+template <int MODE>
+DEV float score(float acc, const ScoreConst& k) {
+  if constexpr (MODE == PLAIN) return acc * k.a;
+  return fmaf(-2.f * k.c, __builtin_amdgcn_rcpf(1.f + fexp2(acc * k.a)), k.c);
+}
+
+// running softmax state of one query row (the lane's)
+struct Run {
+  float m, l;                                 // maximum (log2 units; 0 in CAPPED_NOMAX), this lane's sum
+};
+
+// One 64-key tile of the lane's row (keys 16 nt + 4 fq + r): scores -> weights
+// (bf16 MFMA fragments, key order as in the accumulators).  MASKED: keys outside
+// [lo, hi] (tile-relative) drop out.  Returns the factor O is to be rescaled by.
+template <int MODE, bool MASKED>
+DEV float tile_weights(f32x4 (&sacc)[4], bf16x8 (&pf)[2], Run& st, const ScoreConst& k, int lo, int hi,
+                       int fq) {
+  float alpha = 1.f;
+  float tmax = -INFINITY;
+#pragma unroll
+  for (int nt = 0; nt < 4; ++nt)
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      float v = score<MODE>(sacc[nt][r], k);
+      if constexpr (MASKED) {
+        const int key = nt * 16 + fq * 4 + r;
+        v = (key >= lo && key <= hi) ? v : -INFINITY;
+      }
+      sacc[nt][r] = v;
+      if constexpr (MODE != CAPPED_NOMAX) tmax = fmaxf(tmax, v);
+    }
+  float mu = 0.f;
+  if constexpr (MODE != CAPPED_NOMAX) {
+    tmax = fmaxf(tmax, __shfl_xor(tmax, 16, 64));
+    tmax = fmaxf(tmax, __shfl_xor(tmax, 32, 64));
+    const float m_new = fmaxf(st.m, tmax);
+    mu = m_new == -INFINITY ? 0.f : m_new;    // every key masked so far
+    alpha = fexp2(st.m - mu);
+    st.m = m_new;
+  }
+  float sum = 0.f;
+#pragma unroll
+  for (int nt = 0; nt < 4; ++nt)
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const float p = fexp2(sacc[nt][r] - mu);
+      sum += p;
+      pf[nt >> 1][(nt & 1) * 4 + r] = (bf16)p;
+    }
+  st.l = st.l * alpha + sum;
+  return alpha;
+}
+
+// O^T += V^T P^T over one tile; Vl: [64][DV] with 16-B chunk swizzle ^= row & 7
+template <int DV>
+DEV void tile_pv(const bf16* Vl, const bf16x8 (&pf)[2], f32x4 (&o)[DV / 16], int lane) {
+  const int fq = lane >> 4, tq = (lane & 15) >> 2, tp = lane & 3;
+#pragma unroll
+  for (int dt = 0; dt < DV / 16; ++dt) {
+    const int chunk = dt * 2 + (tp >> 1), half = (tp & 1) * 4;
+#pragma unroll
+    for (int k2 = 0; k2 < 2; ++k2) {
+      const int key0 = k2 * 32 + fq * 4 + tq;
+      const int key1 = key0 + 16;
+      const bf16x4 v0 = tr_read(Vl + key0 * DV + ((chunk ^ (key0 & 7)) << 3) + half);
+      const bf16x4 v1 = tr_read(Vl + key1 * DV + ((chunk ^ (key1 & 7)) << 3) + half);
+      const bf16x8 vf = bf16x8{v0[0], v0[1], v0[2], v0[3], v1[0], v1[1], v1[2], v1[3]};
+      o[dt] = mfma16x16x32(vf, pf[k2], o[dt]);
+    }
+  }
+}
+
+// LDS-DMA of pieces [p0, p1) (1 KiB each) of a [64][D] block, swizzled
+template <int D, int P0, int P1>
+DEV void stage_rows(const bf16* src, bf16* dst, int first, int lane) {
+  constexpr int NC = D / 8;                   // 16-B chunks per row
+#pragma unroll
+  for (int i = P0; i < P1; ++i) {
+    const int p = first + i;
+    const int c = p * 64 + lane;
+    const int row = c / NC, chunk = c % NC;
+    glds16(src + row * D + ((chunk ^ (row & 7)) << 3), dst + p * 512);
+  }
+}
 
 DEV int chunk_start(int pos, int chunk) { return chunk > 0 ? pos / chunk * chunk : 0; }
 
@@ -89,7 +214,328 @@ __global__ __launch_bounds__(64) void attn_row_kernel(const MaskedAttnArgs a) {
   }
 }
 
+
+// ------------------------------------------------------------------ tile form
+// blockIdx.x = work item, blockIdx.y = key head x 64-row group of the item
+template <int DK, int DV, int MODE>
+__global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(DK + DV <= 256 ? 3 : 1)))
+void attn_tile_kernel(const MaskedAttnArgs a) {
+  __shared__ __attribute__((aligned(16))) bf16 smem[KT * (DK + DV)];
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const int fr = lane & 15, fq = lane >> 4;
+  const int Hkv = a.Hkv, G = a.Hq / Hkv;
+  const int kvh = blockIdx.y % Hkv, rg = blockIdx.y / Hkv;
+  const int s = a.work_seq[blockIdx.x], q0 = a.work_q0[blockIdx.x];
+  const int ql = a.q_len[s], cl = a.ctx_len[s], qs = a.q_start[s];
+  const int ntok = min(a.item_tokens, ql - q0);         // the item's tokens (<= 0: padding)
+  const int row0 = rg * 64;
+  if (row0 >= ntok * G) return;                          // whole block, before any barrier
+  const int rows = min(ntok * G - row0, 64);
+  const int row = wave * 16 + fr;
+  const bool valid = row < rows;
+  const int rr = row0 + (valid ? row : 0);
+  const int tok = q0 + rr / G, head = kvh * G + rr % G;
+  const int base = cl - ql;                              // position of the span's first token
+  const int qpos = base + tok;
+  const int first = chunk_start(qpos, a.chunk);          // first key of this lane's row
+  // key tiles of the block, and of this wave's rows
+  const int b_lo = chunk_start(base + q0 + row0 / G, a.chunk), b_hi = base + q0 + (row0 + rows - 1) / G;
+  const int w0 = min(row0 + wave * 16, row0 + rows - 1), w1 = min(row0 + wave * 16 + 15, row0 + rows - 1);
+  const int wp0 = base + q0 + w0 / G, wp1 = base + q0 + w1 / G;   // the wave's positions
+  const int w_lo = chunk_start(wp0, a.chunk), w_in = chunk_start(wp1, a.chunk);
+  const bool w_on = wave * 16 < rows;
+
+  bf16x8 qf[DK / 32];
+  {
+    const bf16* qp = (const bf16*)a.q + ((size_t)(qs + tok) * a.Hq + head) * DK + 8 * fq;
+#pragma unroll
+    for (int ks = 0; ks < DK / 32; ++ks) qf[ks] = *reinterpret_cast<const bf16x8*>(qp + 32 * ks);
+  }
+  const ScoreConst kc = score_const<MODE>(a);
+  Run st;
+  st.m = MODE == CAPPED_NOMAX || a.sink ? 0.f : -INFINITY;
+  st.l = a.sink && fq == 0 ? 1.f : 0.f;
+  f32x4 o[DV / 16];
+#pragma unroll
+  for (int i = 0; i < DV / 16; ++i) o[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+
+  bf16* Kl = smem;
+  bf16* Vl = smem + KT * DK;
+  const int kt0 = b_lo / KT, kt1 = b_hi / KT;
+  const int* bt = a.block_table + (size_t)s * a.max_blocks;
+  int base_kt = kt0, bt_v = kt0 + lane <= kt1 ? bt[kt0 + lane] : 0;   // 64 table entries per load
+  for (int kt = kt0; kt <= kt1; ++kt) {
+    if (kt - base_kt >= 64) {
+      base_kt = kt;
+      bt_v = kt + lane <= kt1 ? bt[kt + lane] : 0;
+    }
+    const size_t blk = (size_t)__builtin_amdgcn_readlane(bt_v, kt - base_kt) * Hkv + kvh;
+    stage_rows<DK, 0, DK / 32>((const bf16*)a.kc + blk * (KT * DK), Kl, wave * (DK / 32), lane);
+    stage_rows<DV, 0, DV / 32>((const bf16*)a.vc + blk * (KT * DV), Vl, wave * (DV / 32), lane);
+    __syncthreads();                                     // drains the LDS-DMA
+    if (b_hi - kt * KT < KT - 1) {                       // rows past the last key: zero their values
+      const int r0 = b_hi - kt * KT + 1;
+      for (int c = r0 * (DV / 8) + threadIdx.x; c < KT * (DV / 8); c += 256)
+        *reinterpret_cast<u32x4*>(Vl + c * 8) = u32x4{0, 0, 0, 0};
+      __syncthreads();
+    }
+    const int k_lo = kt * KT, k_hi = k_lo + KT - 1;
+    if (w_on && k_lo <= wp1 && k_hi >= w_lo) {           // (wave-uniform) some row of the wave sees it
+      f32x4 sacc[4];
+#pragma unroll
+      for (int nt = 0; nt < 4; ++nt) {
+        sacc[nt] = f32x4{0.f, 0.f, 0.f, 0.f};
+        const int kr = nt * 16 + fr;
+#pragma unroll
+        for (int ks = 0; ks < DK / 32; ++ks) {
+          const bf16x8 kf = *reinterpret_cast<const bf16x8*>(Kl + kr * DK + (((ks * 4 + fq) ^ (kr & 7)) << 3));
+          sacc[nt] = mfma16x16x32(kf, qf[ks], sacc[nt]);
+        }
+      }
+      bf16x8 pf[2];
+      const float alpha = (k_hi <= wp0 && k_lo >= w_in)
+                              ? tile_weights<MODE, false>(sacc, pf, st, kc, 0, 0, fq)
+                              : tile_weights<MODE, true>(sacc, pf, st, kc, first - k_lo, qpos - k_lo, fq);
+      if constexpr (MODE != CAPPED_NOMAX) {
+#pragma unroll
+        for (int dt = 0; dt < DV / 16; ++dt) o[dt] *= alpha;
+      }
+      tile_pv<DV>(Vl, pf, o, lane);
+    }
+    __syncthreads();
+  }
+  float l = st.l + __shfl_xor(st.l, 16, 64);
+  l += __shfl_xor(l, 32, 64);
+  if (!valid) return;
+  const float inv = l > 0.f ? 1.f / l : 0.f;
+  bf16* op = (bf16*)a.out + ((size_t)(qs + tok) * a.Hq + head) * DV + 4 * fq;
+#pragma unroll
+  for (int dt = 0; dt < DV / 16; ++dt) {
+    bf16x4 w;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) w[r] = (bf16)(o[dt][r] * inv);
+    *reinterpret_cast<bf16x4*>(op + dt * 16) = w;
+  }
+}
+
+// ----------------------------------------------------------------- split form
+// blockIdx.x = work item, .y = key head x 16-row group, .z = key split.  Wave w
+// of split z takes every (4 nz)-th tile of the item, from 4 z + w on.
+template <int DK, int DV, int MODE>
+__global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(DK + DV <= 256 ? 2 : 1)))
+void attn_split_kernel(const MaskedAttnArgs a) {
+  constexpr int NWV = 4;
+  __shared__ __attribute__((aligned(16))) bf16 smem[NWV * KT * DV];   // V tiles, then the waves' O
+  __shared__ float red_m[NWV][16], red_l[NWV][16];
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const int fr = lane & 15, fq = lane >> 4;
+  const int Hkv = a.Hkv, G = a.Hq / Hkv;
+  const int kvh = blockIdx.y % Hkv, rg = blockIdx.y / Hkv;
+  const int z = blockIdx.z, nz = gridDim.z;
+  const int s = a.work_seq[blockIdx.x], q0 = a.work_q0[blockIdx.x];
+  const int ql = a.q_len[s], cl = a.ctx_len[s], qs = a.q_start[s];
+  const int ntok = min(a.item_tokens, ql - q0);
+  const int row0 = rg * 16;
+  if (row0 >= ntok * G) return;                          // whole block, before any barrier
+  const int rows = min(ntok * G - row0, 16);
+  const bool valid = fr < rows;
+  const int rr = row0 + (valid ? fr : 0);
+  const int tok = q0 + rr / G, head = kvh * G + rr % G;
+  const int base = cl - ql, qpos = base + tok;
+  const int first = chunk_start(qpos, a.chunk);
+  const int p0 = base + q0 + row0 / G, p1 = base + q0 + (row0 + rows - 1) / G;
+  const int lo = chunk_start(p0, a.chunk), in = chunk_start(p1, a.chunk);
+
+  bf16x8 qf[DK / 32];
+  {
+    const bf16* qp = (const bf16*)a.q + ((size_t)(qs + tok) * a.Hq + head) * DK + 8 * fq;
+#pragma unroll
+    for (int ks = 0; ks < DK / 32; ++ks) qf[ks] = *reinterpret_cast<const bf16x8*>(qp + 32 * ks);
+  }
+  const ScoreConst kc = score_const<MODE>(a);
+  const bool sink = a.sink && z == 0 && wave == 0;
+  Run st;
+  st.m = MODE == CAPPED_NOMAX || sink ? 0.f : -INFINITY;
+  st.l = sink && fq == 0 ? 1.f : 0.f;
+  f32x4 o[DV / 16];
+#pragma unroll
+  for (int i = 0; i < DV / 16; ++i) o[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+
+  bf16* Vl = smem + wave * (KT * DV);
+  const int kt0 = lo / KT, kt1 = p1 / KT, step = NWV * nz;
+  const int* bt = a.block_table + (size_t)s * a.max_blocks;
+  int kt = kt0 + z * NWV + wave, left = 0, bt_v = 0;
+  for (; kt <= kt1; kt += step, --left) {
+    if (left == 0) {                                     // the wave's next 64 table entries
+      const int i = kt + lane * step;
+      bt_v = i <= kt1 ? bt[i] : 0;
+      left = 64;
+    }
+    const size_t blk = (size_t)__builtin_amdgcn_readlane(bt_v, 64 - left) * Hkv + kvh;
+    const bf16* kp = (const bf16*)a.kc + blk * (KT * DK) + fr * DK + 8 * fq;
+    bf16x8 kf[4][DK / 32];
+#pragma unroll
+    for (int nt = 0; nt < 4; ++nt)
+#pragma unroll
+      for (int ks = 0; ks < DK / 32; ++ks)
+        kf[nt][ks] = *reinterpret_cast<const bf16x8*>(kp + nt * 16 * DK + 32 * ks);
+    stage_rows<DV, 0, DV / 8>((const bf16*)a.vc + blk * (KT * DV), Vl, 0, lane);
+    f32x4 sacc[4];
+#pragma unroll
+    for (int nt = 0; nt < 4; ++nt) {
+      sacc[nt] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int ks = 0; ks < DK / 32; ++ks) sacc[nt] = mfma16x16x32(kf[nt][ks], qf[ks], sacc[nt]);
+    }
+    const int k_lo = kt * KT, k_hi = k_lo + KT - 1;
+    bf16x8 pf[2];
+    const float alpha = (k_hi <= p0 && k_lo >= in)
+                            ? tile_weights<MODE, false>(sacc, pf, st, kc, 0, 0, fq)
+                            : tile_weights<MODE, true>(sacc, pf, st, kc, first - k_lo, qpos - k_lo, fq);
+    if constexpr (MODE != CAPPED_NOMAX) {
+#pragma unroll
+      for (int dt = 0; dt < DV / 16; ++dt) o[dt] *= alpha;
+    }
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");     // the wave's V tile is in LDS
+    if (p1 - k_lo < KT - 1) {                            // rows past the last key: zero their values
+      for (int c = (p1 - k_lo + 1) * (DV / 8) + lane; c < KT * (DV / 8); c += 64)
+        *reinterpret_cast<u32x4*>(Vl + c * 8) = u32x4{0, 0, 0, 0};
+      asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+    }
+    tile_pv<DV>(Vl, pf, o, lane);
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");   // V is read before the next DMA lands
+  }
+
+  // ---- merge the waves: O [16][DV] fp32 per wave in its own V buffer
+  float l = st.l + __shfl_xor(st.l, 16, 64);
+  l += __shfl_xor(l, 32, 64);
+  if (fq == 0) {
+    red_m[wave][fr] = st.m;
+    red_l[wave][fr] = l;
+  }
+  float* Ow = reinterpret_cast<float*>(Vl);
+#pragma unroll
+  for (int dt = 0; dt < DV / 16; ++dt)
+    *reinterpret_cast<f32x4*>(Ow + fr * DV + dt * 16 + 4 * fq) = o[dt];
+  __syncthreads();
+  const int r = threadIdx.x >> 4, c0 = (threadIdx.x & 15) * 4;
+  if (r >= rows) return;
+  float m = red_m[0][r], wgt[NWV], lt = 0.f;
+#pragma unroll
+  for (int w = 1; w < NWV; ++w) m = fmaxf(m, red_m[w][r]);
+  const float mu = m == -INFINITY ? 0.f : m;
+#pragma unroll
+  for (int w = 0; w < NWV; ++w) {
+    wgt[w] = MODE == CAPPED_NOMAX ? 1.f : fexp2(red_m[w][r] - mu);
+    lt += wgt[w] * red_l[w][r];
+  }
+  const int r2 = row0 + r;
+  const size_t orow = (size_t)(qs + q0 + r2 / G) * a.Hq + kvh * G + r2 % G;
+  const float inv = nz == 1 ? (lt > 0.f ? 1.f / lt : 0.f) : 1.f;
+#pragma unroll
+  for (int c = c0; c < DV; c += 64) {
+    f32x4 v = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int w = 0; w < NWV; ++w)
+      v += *reinterpret_cast<const f32x4*>(reinterpret_cast<const float*>(smem + w * (KT * DV)) + r * DV + c) *
+           wgt[w];
+    v *= inv;
+    if (nz == 1) {
+      bf16x4 b;
+#pragma unroll
+      for (int j = 0; j < 4; ++j) b[j] = (bf16)v[j];
+      *reinterpret_cast<bf16x4*>((bf16*)a.out + orow * DV + c) = b;
+    } else {
+      *reinterpret_cast<f32x4*>(a.split_o + ((size_t)z * a.rows + orow) * DV + c) = v;
+    }
+  }
+  if (nz > 1 && (threadIdx.x & 15) == 0) {
+    a.split_ml[((size_t)z * a.rows + orow) * 2] = m;
+    a.split_ml[((size_t)z * a.rows + orow) * 2 + 1] = lt;
+  }
+}
+
+// Sum of the splits' partials (unnormalised O, m, l): one thread per 4 columns
+// of a row of the split form's items (blockIdx.y = key head x 16-row group).
+template <int MODE>
+__global__ __launch_bounds__(256) void attn_split_merge(const MaskedAttnArgs a, int nz) {
+  const int G = a.Hq / a.Hkv, kvh = blockIdx.y % a.Hkv, rg = blockIdx.y / a.Hkv;
+  const int s = a.work_seq[blockIdx.x], q0 = a.work_q0[blockIdx.x];
+  const int ntok = min(a.item_tokens, a.q_len[s] - q0);
+  const int r = rg * 16 + (threadIdx.x >> 4);
+  if (r >= ntok * G) return;
+  const size_t row = (size_t)(a.q_start[s] + q0 + r / G) * a.Hq + kvh * G + r % G;
+  float mu = 0.f;
+  if constexpr (MODE != CAPPED_NOMAX) {
+    float m = -INFINITY;
+    for (int z = 0; z < nz; ++z) m = fmaxf(m, a.split_ml[((size_t)z * a.rows + row) * 2]);
+    mu = m == -INFINITY ? 0.f : m;
+  }
+  for (int c = (threadIdx.x & 15) * 4; c < a.DV; c += 64) {
+    float l = 0.f;
+    f32x4 v = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
+    for (int z = 0; z < nz; ++z) {
+      const size_t i = (size_t)z * a.rows + row;
+      const float w = MODE == CAPPED_NOMAX ? 1.f : fexp2(a.split_ml[i * 2] - mu);
+      l += w * a.split_ml[i * 2 + 1];
+      v += *reinterpret_cast<const f32x4*>(a.split_o + i * a.DV + c) * w;
+    }
+    const float inv = l > 0.f ? 1.f / l : 0.f;
+    bf16x4 b;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) b[j] = (bf16)(v[j] * inv);
+    *reinterpret_cast<bf16x4*>((bf16*)a.out + row * a.DV + c) = b;
+  }
+}
+
+template <int DK, int DV, int MODE>
+void launch_mode(const MaskedAttnArgs& a, int nwork, int form, int nz, hipStream_t s) {
+  const int G = a.Hq / a.Hkv;
+  if (form == 4) {
+    const int groups = (a.item_tokens * G + 63) / 64;
+    attn_tile_kernel<DK, DV, MODE><<<dim3(nwork, a.Hkv * groups), 256, 0, s>>>(a);
+    return;
+  }
+  const int groups = (a.item_tokens * G + 15) / 16;
+  attn_split_kernel<DK, DV, MODE><<<dim3(nwork, a.Hkv * groups, nz), 256, 0, s>>>(a);
+  if (nz > 1) attn_split_merge<MODE><<<dim3(nwork, a.Hkv * groups), 256, 0, s>>>(a, nz);
+}
+
+template <int DK, int DV>
+void launch_dims(const MaskedAttnArgs& a, int nwork, int form, int nz, hipStream_t s) {
+  if (a.cap <= 0.f) launch_mode<DK, DV, PLAIN>(a, nwork, form, nz, s);
+  else if (a.cap <= NOMAX_CAP) launch_mode<DK, DV, CAPPED_NOMAX>(a, nwork, form, nz, s);
+  else launch_mode<DK, DV, CAPPED>(a, nwork, form, nz, s);
+}
+
+template <int DK>
+int launch_dk(const MaskedAttnArgs& a, int nwork, int form, int nz, hipStream_t s) {
+  switch (a.DV) {
+    case 64: launch_dims<DK, 64>(a, nwork, form, nz, s); return 0;
+    case 128: launch_dims<DK, 128>(a, nwork, form, nz, s); return 0;
+    case 192: launch_dims<DK, 192>(a, nwork, form, nz, s); return 0;
+    case 256: launch_dims<DK, 256>(a, nwork, form, nz, s); return 0;
+    default: return 3;
+  }
+}
+
 }  // namespace
+
+// One work list (form 4: the 4-wave items, 1: the 1-wave items, whose keys go
+// over nz splits); nonzero: head sizes outside 64 / 128 / 192 / 256
+int launch_attn_masked(const MaskedAttnArgs& a, int nwork, int form, int nz, hipStream_t s) {
+  if (nwork <= 0) return 0;
+  if (form != 1 && form != 4) return 1;
+  if (nz < 1 || (form == 4 && nz != 1) || (nz > 1 && (!a.split_o || !a.split_ml))) return 2;
+  switch (a.DK) {
+    case 64: return launch_dk<64>(a, nwork, form, nz, s);
+    case 128: return launch_dk<128>(a, nwork, form, nz, s);
+    case 192: return launch_dk<192>(a, nwork, form, nz, s);
+    case 256: return launch_dk<256>(a, nwork, form, nz, s);
+    default: return 3;
+  }
+}
 
 int launch_attn_row(const MaskedAttnArgs& a, int T, bool f32, hipStream_t s) {
   if (T <= 0) return 0;

@@ -874,6 +874,38 @@ MaskedAttnArgs masked_args(const at::Tensor& q, const at::Tensor& k_cache, const
   return a;
 }
 
+// one work list of the MFMA forms (form 4 / 1, attention_masked.hip); false: head
+// sizes outside them, nothing launched
+bool attention_masked(const at::Tensor& q, const at::Tensor& k_cache, const at::Tensor& v_cache,
+                      at::Tensor& out, const at::Tensor& q_start, const at::Tensor& q_len,
+                      const at::Tensor& ctx_len, const at::Tensor& block_table,
+                      const at::Tensor& work_seq, const at::Tensor& work_q0, int64_t form,
+                      int64_t item_tokens, double scale, double cap, int64_t chunk, bool sink,
+                      int64_t nz, const c10::optional<at::Tensor>& split_o,
+                      const c10::optional<at::Tensor>& split_ml) {
+  MaskedAttnArgs a = masked_args(q, k_cache, v_cache, out, q_start, q_len, ctx_len, block_table,
+                                 scale, cap, chunk, sink);
+  CHECK_BF16(q); CHECK_I32_TENSOR(work_seq); CHECK_I32_TENSOR(work_q0);
+  TORCH_CHECK(work_seq.numel() == work_q0.numel() && item_tokens > 0, "attention_masked: work list");
+  a.work_seq = work_seq.data_ptr<int>();
+  a.work_q0 = work_q0.data_ptr<int>();
+  a.item_tokens = (int)item_tokens;
+  a.rows = (int)(q.size(0) * q.size(1));
+  if (nz > 1) {
+    TORCH_CHECK(split_o.has_value() && split_ml.has_value(), "attention_masked: split buffers");
+    CHECK_F32_TENSOR((*split_o)); CHECK_F32_TENSOR((*split_ml));
+    TORCH_CHECK(split_o->numel() >= nz * a.rows * (int64_t)a.DV && split_ml->numel() >= nz * a.rows * 2,
+                "attention_masked: split_o [nz, T, Hq, DV], split_ml [nz, T, Hq, 2]");
+    a.split_o = split_o->data_ptr<float>();
+    a.split_ml = split_ml->data_ptr<float>();
+  }
+  const int rc = launch_attn_masked(a, work_seq.numel(), (int)form, (int)nz, stream());
+  if (rc == 3) return false;
+  TORCH_CHECK(rc == 0, "attention_masked: code ", rc);
+  check_launch("attention_masked");
+  return true;
+}
+
 void attention_row(const at::Tensor& q, const at::Tensor& k_cache, const at::Tensor& v_cache,
                    at::Tensor& out, const at::Tensor& q_start, const at::Tensor& q_len,
                    const at::Tensor& ctx_len, const at::Tensor& block_table, double scale, double cap,
@@ -1135,6 +1167,11 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("gated_act_f32", &gated_act_f32);
   m.def("rope_kv_any", &rope_kv_any);
   m.def("attention_row", &attention_row);
+  m.def("attention_masked", &attention_masked, py::arg("q"), py::arg("k_cache"), py::arg("v_cache"),
+        py::arg("out"), py::arg("q_start"), py::arg("q_len"), py::arg("ctx_len"), py::arg("block_table"),
+        py::arg("work_seq"), py::arg("work_q0"), py::arg("form"), py::arg("item_tokens"),
+        py::arg("scale"), py::arg("cap"), py::arg("chunk"), py::arg("sink"), py::arg("nz") = 1,
+        py::arg("split_o") = py::none(), py::arg("split_ml") = py::none());
   m.def("branch_select", &branch_select);
   m.def("add_inplace", &add_inplace);
   m.def("paged_attention_decode_oproj", &paged_attention_decode_oproj,

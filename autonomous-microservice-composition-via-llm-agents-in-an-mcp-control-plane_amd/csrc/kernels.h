@@ -78,7 +78,16 @@ struct MaskedAttnArgs {
   float scale, cap;          // cap 0: no soft cap
   int chunk;                 // 0: plain causal
   int sink;
+  // work-list forms: items of item_tokens tokens
+  const int* work_seq;
+  const int* work_q0;
+  int item_tokens;
+  // split form with nz > 1: [nz][rows][DV] unnormalised O, [nz][rows] (m, l); rows = T Hq
+  float* split_o;
+  float* split_ml;
+  int rows;
 };
+int launch_attn_masked(const MaskedAttnArgs& a, int nwork, int form, int nz, hipStream_t s);
 int launch_attn_row(const MaskedAttnArgs& a, int T, bool f32, hipStream_t s);
 
 // QKV projection + RoPE + paged K/V write fused in the GEMM epilogue (K1+K4+K10)

@@ -394,7 +394,8 @@ class DozazenModel:
             ops.qkv_rope_bias(h, lw.wqkv, lw.bqkv, step.positions, step.slots, self.cos_sin[i], q, kc, vc)
             if last and rows.numel() == 0 and tap is None:
                 return h.new_empty(0, Wp)              # every key is in the cache; nothing is read
-            a = ops.masked_attention(q, kc, vc, step.attn, m.scale, m.soft_cap, m.chunk, True)
+            a = ops.masked_attention(q, kc, vc, step.attn, m.scale, cfg.group, m.soft_cap,
+                                     m.chunk, True)
             a = a.view(T, -1)
             if last and tap is None:                   # only the asked-for rows go on
                 ri = rows.long()

@@ -587,16 +587,37 @@ def paged_attention(q, k_cache, v_cache, meta, scale, out=None):
     return r if out is None else out.copy_(r)
 
 
-def masked_attention(q, k_cache, v_cache, meta, scale, soft_cap: float = 0.0, chunk: int = 0,
-                     sink: bool = False):
+MASKED_MAX_HEAD = 256           # largest head of the MFMA forms (csrc/attention_masked.hip)
+# scheduler split counts are for one wave per split: blocks of 4 waves take fewer
+_MASKED_SPLIT_DIV = int(os.environ.get("MCP_MASKED_SPLIT_DIV", "2"))
+
+
+def masked_attention(q, k_cache, v_cache, meta, scale, group: int, soft_cap: float = 0.0,
+                     chunk: int = 0, sink: bool = False):
     """Paged causal attention, q [T, Hq, DK] -> [T, Hq, DV], with the score
     soft cap (s <- cap tanh(s / cap); 0 = none), the chunked mask (keys of the
     query's own ``chunk``-token stretch of the sequence; 0 = all earlier keys)
-    and the softmax sink (one added to the denominator)."""
+    and the softmax sink (one added to the denominator).  ``group``: the GQA
+    group the step's work lists were cut for (16 / group tokens per 1-wave
+    item); the heads' own group may be another."""
     if q.is_cuda:
         out = torch.empty(q.shape[0], q.shape[1], v_cache.shape[3], device=q.device, dtype=q.dtype)
-        lib().attention_row(q, k_cache, v_cache, out, meta.q_start, meta.q_len, meta.ctx_len,
-                            meta.block_table, float(scale), float(soft_cap), int(chunk), bool(sink))
+        L = lib()
+        a = (q, k_cache, v_cache, out, meta.q_start, meta.q_len, meta.ctx_len, meta.block_table)
+        k = (float(scale), float(soft_cap), int(chunk), bool(sink))
+        if q.dtype == torch.bfloat16 and max(q.shape[2], v_cache.shape[3]) <= MASKED_MAX_HEAD:
+            for nw, ws, wq in meta.work_lists():
+                nz, so, sm = 1, None, None
+                if nw == 1 and int(meta.kv_splits) > 1:
+                    # a block's 4 waves share the keys already
+                    nz = max(1, int(meta.kv_splits) // _MASKED_SPLIT_DIV)
+                if nz > 1:
+                    so = torch.empty(nz, *out.shape, device=q.device, dtype=torch.float32)
+                    sm = torch.empty(nz, q.shape[0], q.shape[1], 2, device=q.device, dtype=torch.float32)
+                if not L.attention_masked(*a, ws, wq, nw, nw * (16 // group), *k, nz, so, sm):
+                    raise ValueError(f"masked attention: head sizes {q.shape[2]} / {v_cache.shape[3]}")
+            return out
+        L.attention_row(*a, *k)
         return out
     return ref.masked_attention(q, k_cache, v_cache, meta.q_start, meta.q_len, meta.ctx_len,
                                 meta.block_table, scale, soft_cap, chunk, sink)
