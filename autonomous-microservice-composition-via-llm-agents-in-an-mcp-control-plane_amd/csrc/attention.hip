@@ -954,7 +954,7 @@ void attn_dispatch(int nw, const AttnArgs& a, int nwork, hipStream_t s, int nspl
 // per-device arrival tickets of the fused split-KV launch (zeroed once here,
 // at library load - never inside a graph capture; each last arriver re-arms
 // its own ticket)
-constexpr int SPLIT_CNT_MAX = 1 << 16;
+constexpr int SPLIT_CNT_MAX = ATTN_SPLIT_TICKETS;
 int* g_split_cnt[64] = {};
 
 int* split_counters() {

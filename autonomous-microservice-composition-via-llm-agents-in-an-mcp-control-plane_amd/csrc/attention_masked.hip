@@ -327,6 +327,7 @@ void attn_split_kernel(const MaskedAttnArgs a) {
   constexpr int NWV = 4;
   __shared__ __attribute__((aligned(16))) bf16 smem[NWV * KT * DV];   // V tiles, then the waves' O
   __shared__ float red_m[NWV][16], red_l[NWV][16];
+  __shared__ int s_last;
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int fr = lane & 15, fq = lane >> 4;
   const int Hkv = a.Hkv, G = a.Hq / Hkv;
@@ -419,7 +420,7 @@ void attn_split_kernel(const MaskedAttnArgs a) {
     *reinterpret_cast<f32x4*>(Ow + fr * DV + dt * 16 + 4 * fq) = o[dt];
   __syncthreads();
   const int r = threadIdx.x >> 4, c0 = (threadIdx.x & 15) * 4;
-  if (r >= rows) return;
+  const bool live = r < rows;
   float m = red_m[0][r], wgt[NWV], lt = 0.f;
 #pragma unroll
   for (int w = 1; w < NWV; ++w) m = fmaxf(m, red_m[w][r]);
@@ -429,64 +430,80 @@ void attn_split_kernel(const MaskedAttnArgs a) {
     wgt[w] = MODE == CAPPED_NOMAX ? 1.f : fexp2(red_m[w][r] - mu);
     lt += wgt[w] * red_l[w][r];
   }
-  const int r2 = row0 + r;
+  const int r2 = row0 + (live ? r : 0);
   const size_t orow = (size_t)(qs + q0 + r2 / G) * a.Hq + kvh * G + r2 % G;
-  const float inv = nz == 1 ? (lt > 0.f ? 1.f / lt : 0.f) : 1.f;
+  f32x4 v[DV / 64];
 #pragma unroll
-  for (int c = c0; c < DV; c += 64) {
-    f32x4 v = f32x4{0.f, 0.f, 0.f, 0.f};
+  for (int i = 0; i < DV / 64; ++i) {
+    v[i] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int w = 0; w < NWV; ++w)
-      v += *reinterpret_cast<const f32x4*>(reinterpret_cast<const float*>(smem + w * (KT * DV)) + r * DV + c) *
-           wgt[w];
-    v *= inv;
-    if (nz == 1) {
+      v[i] += *reinterpret_cast<const f32x4*>(reinterpret_cast<const float*>(smem + w * (KT * DV)) + r * DV +
+                                              c0 + 64 * i) * wgt[w];
+  }
+  bf16* op = (bf16*)a.out + orow * DV + c0;
+  auto put = [&](float inv) {
+#pragma unroll
+    for (int i = 0; i < DV / 64; ++i) {
       bf16x4 b;
 #pragma unroll
-      for (int j = 0; j < 4; ++j) b[j] = (bf16)v[j];
-      *reinterpret_cast<bf16x4*>((bf16*)a.out + orow * DV + c) = b;
-    } else {
-      *reinterpret_cast<f32x4*>(a.split_o + ((size_t)z * a.rows + orow) * DV + c) = v;
+      for (int j = 0; j < 4; ++j) b[j] = (bf16)(v[i][j] * inv);
+      *reinterpret_cast<bf16x4*>(op + 64 * i) = b;
     }
+  };
+  if (nz == 1) {
+    if (live) put(lt > 0.f ? 1.f / lt : 0.f);
+    return;
   }
-  if (nz > 1 && (threadIdx.x & 15) == 0) {
-    a.split_ml[((size_t)z * a.rows + orow) * 2] = m;
-    a.split_ml[((size_t)z * a.rows + orow) * 2 + 1] = lt;
-  }
-}
-
-// Sum of the splits' partials (unnormalised O, m, l): one thread per 4 columns
-// of a row of the split form's items (blockIdx.y = key head x 16-row group).
-template <int MODE>
-__global__ __launch_bounds__(256) void attn_split_merge(const MaskedAttnArgs a, int nz) {
-  const int G = a.Hq / a.Hkv, kvh = blockIdx.y % a.Hkv, rg = blockIdx.y / a.Hkv;
-  const int s = a.work_seq[blockIdx.x], q0 = a.work_q0[blockIdx.x];
-  const int ntok = min(a.item_tokens, a.q_len[s] - q0);
-  const int r = rg * 16 + (threadIdx.x >> 4);
-  if (r >= ntok * G) return;
-  const size_t row = (size_t)(a.q_start[s] + q0 + r / G) * a.Hq + kvh * G + r % G;
-  float mu = 0.f;
-  if constexpr (MODE != CAPPED_NOMAX) {
-    float m = -INFINITY;
-    for (int z = 0; z < nz; ++z) m = fmaxf(m, a.split_ml[((size_t)z * a.rows + row) * 2]);
-    mu = m == -INFINITY ? 0.f : m;
-  }
-  for (int c = (threadIdx.x & 15) * 4; c < a.DV; c += 64) {
-    float l = 0.f;
-    f32x4 v = f32x4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll 4
-    for (int z = 0; z < nz; ++z) {
-      const size_t i = (size_t)z * a.rows + row;
-      const float w = MODE == CAPPED_NOMAX ? 1.f : fexp2(a.split_ml[i * 2] - mu);
-      l += w * a.split_ml[i * 2 + 1];
-      v += *reinterpret_cast<const f32x4*>(a.split_o + i * a.DV + c) * w;
-    }
-    const float inv = l > 0.f ? 1.f / l : 0.f;
-    bf16x4 b;
+  // ---- merge the splits: every block stores its unnormalised O and (m, l)
+  // write-through (sc1), drains them and takes the item's ticket; the last one
+  // adds all partials up, read back in split order (sc1), so the result does not
+  // depend on the order of arrival.  Every wave reaches both barriers.
+  const auto rso = __builtin_amdgcn_make_buffer_rsrc(a.split_o, (short)0, 0x7FFFFFFF, 0x00020000);
+  const auto rsm = __builtin_amdgcn_make_buffer_rsrc(a.split_ml, (short)0, 0x7FFFFFFF, 0x00020000);
+  if (live) {
 #pragma unroll
-    for (int j = 0; j < 4; ++j) b[j] = (bf16)(v[j] * inv);
-    *reinterpret_cast<bf16x4*>((bf16*)a.out + row * a.DV + c) = b;
+    for (int i = 0; i < DV / 64; ++i)
+      __builtin_amdgcn_raw_buffer_store_b128(__builtin_bit_cast(u32x4, v[i]), rso,
+                                             (unsigned)((((size_t)z * a.rows + orow) * DV + c0 + 64 * i) * 4), 0, 16);
+    if ((threadIdx.x & 15) == 0)
+      __builtin_amdgcn_raw_buffer_store_b64(u32x2{__builtin_bit_cast(unsigned, m), __builtin_bit_cast(unsigned, lt)},
+                                            rsm, (unsigned)(((size_t)z * a.rows + orow) * 8), 0, 16);
   }
+  asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+  __syncthreads();
+  if (threadIdx.x == 0) {
+    int* cnt = a.tickets + (size_t)blockIdx.x * gridDim.y + blockIdx.y;
+    const int old = __hip_atomic_fetch_add(cnt, 1, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+    if (old == nz - 1) __hip_atomic_store(cnt, 0, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+    s_last = old == nz - 1;
+  }
+  __syncthreads();
+  if (!s_last || !live) return;
+  auto ml = [&](int j) {
+    return __builtin_amdgcn_raw_buffer_load_b64(rsm, (unsigned)(((size_t)j * a.rows + orow) * 8), 0, 16);
+  };
+  float mx = 0.f;
+  if constexpr (MODE != CAPPED_NOMAX) {
+    mx = -INFINITY;
+#pragma unroll 8
+    for (int j = 0; j < nz; ++j) mx = fmaxf(mx, __builtin_bit_cast(float, (unsigned)ml(j)[0]));
+    mx = mx == -INFINITY ? 0.f : mx;
+  }
+  lt = 0.f;
+#pragma unroll
+  for (int i = 0; i < DV / 64; ++i) v[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
+  for (int j = 0; j < nz; ++j) {
+    const auto p = ml(j);
+    const float w = MODE == CAPPED_NOMAX ? 1.f : fexp2(__builtin_bit_cast(float, (unsigned)p[0]) - mx);
+    lt += w * __builtin_bit_cast(float, (unsigned)p[1]);
+#pragma unroll
+    for (int i = 0; i < DV / 64; ++i)
+      v[i] += __builtin_bit_cast(f32x4, __builtin_amdgcn_raw_buffer_load_b128(
+                  rso, (unsigned)((((size_t)j * a.rows + orow) * DV + c0 + 64 * i) * 4), 0, 16)) * w;
+  }
+  put(lt > 0.f ? 1.f / lt : 0.f);
 }
 
 template <int DK, int DV, int MODE>
@@ -499,7 +516,6 @@ void launch_mode(const MaskedAttnArgs& a, int nwork, int form, int nz, hipStream
   }
   const int groups = (a.item_tokens * G + 15) / 16;
   attn_split_kernel<DK, DV, MODE><<<dim3(nwork, a.Hkv * groups, nz), 256, 0, s>>>(a);
-  if (nz > 1) attn_split_merge<MODE><<<dim3(nwork, a.Hkv * groups), 256, 0, s>>>(a, nz);
 }
 
 template <int DK, int DV>
@@ -524,10 +540,19 @@ int launch_dk(const MaskedAttnArgs& a, int nwork, int form, int nz, hipStream_t 
 
 // One work list (form 4: the 4-wave items, 1: the 1-wave items, whose keys go
 // over nz splits); nonzero: head sizes outside 64 / 128 / 192 / 256
-int launch_attn_masked(const MaskedAttnArgs& a, int nwork, int form, int nz, hipStream_t s) {
+int launch_attn_masked(const MaskedAttnArgs& args, int nwork, int form, int nz, hipStream_t s) {
+  MaskedAttnArgs a = args;
   if (nwork <= 0) return 0;
   if (form != 1 && form != 4) return 1;
   if (nz < 1 || (form == 4 && nz != 1) || (nz > 1 && (!a.split_o || !a.split_ml))) return 2;
+  if (nz > 1) {
+    // tickets: one per item, key head and row group (the split-KV tickets of attention.hip)
+    const long long groups = (a.item_tokens * (a.Hq / a.Hkv) + 15) / 16;
+    a.tickets = attn_split_counters();
+    if (!a.tickets || nwork * a.Hkv * groups > ATTN_SPLIT_TICKETS ||
+        (long long)nz * a.rows * a.DV * 4 >= (1ll << 31))
+      nz = 1;                                            // one block per item walks all its keys
+  }
   switch (a.DK) {
     case 64: return launch_dk<64>(a, nwork, form, nz, s);
     case 128: return launch_dk<128>(a, nwork, form, nz, s);

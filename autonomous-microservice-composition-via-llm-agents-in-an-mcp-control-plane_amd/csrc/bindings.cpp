@@ -120,7 +120,8 @@ void rope_kv(const at::Tensor& qkv, const at::Tensor& pos, const at::Tensor& slo
 int64_t qkv_rope_impl(const at::Tensor& X, const at::Tensor& W, at::Tensor& qkv, const at::Tensor& pos,
                       const at::Tensor& slots, const at::Tensor& cos_sin, at::Tensor& q_out,
                       at::Tensor& k_cache, at::Tensor& v_cache, int64_t Hq, int64_t Hkv, int64_t D,
-                      const c10::optional<at::Tensor>& ss_in, double norm_eps, int64_t algo) {
+                      const c10::optional<at::Tensor>& ss_in, double norm_eps, int64_t algo,
+                      const c10::optional<at::Tensor>& bias) {
   CHECK_BF16_TENSOR(X); CHECK_BF16_TENSOR(W); CHECK_BF16_TENSOR(qkv);
   CHECK_I32_TENSOR(pos); CHECK_I32_TENSOR(slots);
   CHECK_BF16_TENSOR(q_out); CHECK_BF16_TENSOR(k_cache); CHECK_BF16_TENSOR(v_cache);
@@ -140,6 +141,11 @@ int64_t qkv_rope_impl(const at::Tensor& X, const at::Tensor& W, at::Tensor& qkv,
   RopeArgs ra{pos.data_ptr<int>(), slots.data_ptr<int>(), cos_sin.data_ptr<float>(),
               q_out.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), (int)Hq, (int)Hkv,
               (int)k_cache.size(2)};
+  if (bias.has_value()) {
+    CHECK_DEV((*bias)); CHECK_CONTIG((*bias));
+    TORCH_CHECK(bias->scalar_type() == at::kFloat && bias->numel() == N, "bias [N] f32");
+    ra.bias = bias->data_ptr<float>();
+  }
   NormEpiScope scope(make_norm_epi(M, K, c10::nullopt, ss_in, norm_eps));
   if (algo >= 0) {             // tuning / tests: one path by code, nonzero = not taken
     const int rc = launch_qkv_rope_algo(X.data_ptr(), W.data_ptr(), qkv.data_ptr(), M, N, K, (int)D,
@@ -155,19 +161,20 @@ int64_t qkv_rope_impl(const at::Tensor& X, const at::Tensor& W, at::Tensor& qkv,
 void qkv_rope(const at::Tensor& X, const at::Tensor& W, at::Tensor& qkv, const at::Tensor& pos,
               const at::Tensor& slots, const at::Tensor& cos_sin, at::Tensor& q_out,
               at::Tensor& k_cache, at::Tensor& v_cache, int64_t Hq, int64_t Hkv, int64_t D,
-              const c10::optional<at::Tensor>& ss_in, double norm_eps) {
+              const c10::optional<at::Tensor>& ss_in, double norm_eps,
+              const c10::optional<at::Tensor>& bias) {
   qkv_rope_impl(X, W, qkv, pos, slots, cos_sin, q_out, k_cache, v_cache, Hq, Hkv, D, ss_in,
-                norm_eps, -1);
+                norm_eps, -1, bias);
 }
 
 int64_t qkv_rope_algo(const at::Tensor& X, const at::Tensor& W, at::Tensor& qkv,
                       const at::Tensor& pos, const at::Tensor& slots, const at::Tensor& cos_sin,
                       at::Tensor& q_out, at::Tensor& k_cache, at::Tensor& v_cache, int64_t Hq,
                       int64_t Hkv, int64_t D, int64_t algo, const c10::optional<at::Tensor>& ss_in,
-                      double norm_eps) {
+                      double norm_eps, const c10::optional<at::Tensor>& bias) {
   TORCH_CHECK(algo >= 0, "qkv_rope_algo: algo >= 0");
   return qkv_rope_impl(X, W, qkv, pos, slots, cos_sin, q_out, k_cache, v_cache, Hq, Hkv, D, ss_in,
-                       norm_eps, algo);
+                       norm_eps, algo, bias);
 }
 
 void gemm_plan_set_rope_py(int64_t N, int64_t K, const std::vector<int64_t>& codes) {
@@ -830,7 +837,7 @@ void rope_kv_any(const at::Tensor& qkv, const c10::optional<at::Tensor>& bias, c
   TORCH_CHECK(launch_rope_kv_any(qkv.data_ptr(), bias.has_value() ? bias->data_ptr<float>() : nullptr,
                                  pos.data_ptr<int>(), slots.data_ptr<int>(), cos_sin.data_ptr(),
                                  q_out.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), T, Hq, Hkv, DK,
-                                 DV, BS, f32, stream()) == 0, "rope_kv_any: head sizes % 8");
+                                 DV, BS, f32, stream()) == 0, "rope_kv_any: head sizes % 16");
   check_launch("rope_kv_any");
 }
 
@@ -1073,14 +1080,14 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("qkv_rope", &qkv_rope, py::arg("X"), py::arg("W"), py::arg("qkv"), py::arg("pos"),
         py::arg("slots"), py::arg("cos_sin"), py::arg("q_out"), py::arg("k_cache"),
         py::arg("v_cache"), py::arg("Hq"), py::arg("Hkv"), py::arg("D"),
-        py::arg("ss_in") = py::none(), py::arg("norm_eps") = 0.0);
+        py::arg("ss_in") = py::none(), py::arg("norm_eps") = 0.0, py::arg("bias") = py::none());
   m.def("gemm_variant", &gemm_variant);
   m.def("gemm_plan_set", &gemm_plan_set_py, "measured tile plan for one (N, K): a code per 64-row M bucket");
   m.def("qkv_rope_algo", &qkv_rope_algo, "one QKV + RoPE path by code (tuning / tests)",
         py::arg("X"), py::arg("W"), py::arg("qkv"), py::arg("pos"), py::arg("slots"),
         py::arg("cos_sin"), py::arg("q_out"), py::arg("k_cache"), py::arg("v_cache"),
         py::arg("Hq"), py::arg("Hkv"), py::arg("D"), py::arg("algo"),
-        py::arg("ss_in") = py::none(), py::arg("norm_eps") = 0.0);
+        py::arg("ss_in") = py::none(), py::arg("norm_eps") = 0.0, py::arg("bias") = py::none());
   m.def("gemm_plan_set_rope", &gemm_plan_set_rope_py,
         "measured QKV + RoPE path per 64-row M bucket for one qkv (N, K) (-1: the rule)");
   m.def("gemm_plan_set_silu", &gemm_plan_set_silu_py,

@@ -165,7 +165,8 @@ template <int D>
 __global__ __launch_bounds__(256) void rope_kv_kernel(
     const bf16* __restrict__ qkv, const int* __restrict__ pos, const int* __restrict__ slots,
     const float2* __restrict__ cos_sin, bf16* __restrict__ q_out, bf16* __restrict__ k_cache,
-    bf16* __restrict__ v_cache, int T, int Hq, int Hkv, int BS, const NormEpi ne) {
+    bf16* __restrict__ v_cache, int T, int Hq, int Hkv, int BS, const NormEpi ne,
+    const float* __restrict__ bias) {
   constexpr int CH = D / 16;                 // 8-wide chunks in the first half
   const int heads = Hq + 2 * Hkv;
   const size_t total = (size_t)T * heads * CH;
@@ -185,11 +186,11 @@ __global__ __launch_bounds__(256) void rope_kv_kernel(
     const int hv = h - Hq - Hkv;
     bf16* dst = v_cache + (((size_t)(slot / BS) * Hkv + hv) * BS + (slot % BS)) * D;
     bf16x8 vlo = lo, vhi = hi;
-    if (ne.ss_in) {
+    if (ne.ss_in || bias) {
 #pragma unroll
       for (int j = 0; j < 8; ++j) {
-        vlo[j] = (bf16)((float)lo[j] * rs);
-        vhi[j] = (bf16)((float)hi[j] * rs);
+        vlo[j] = (bf16)((float)lo[j] * rs + (bias ? bias[h * D + d0 + j] : 0.f));
+        vhi[j] = (bf16)((float)hi[j] * rs + (bias ? bias[h * D + d0 + D / 2 + j] : 0.f));
       }
     }
     *reinterpret_cast<bf16x8*>(dst + d0) = vlo;
@@ -201,7 +202,8 @@ __global__ __launch_bounds__(256) void rope_kv_kernel(
 #pragma unroll
   for (int j = 0; j < 8; ++j) {
     const float2 r = cs[j];
-    const float a = (float)lo[j] * rs, b = (float)hi[j] * rs;
+    const float a = (float)lo[j] * rs + (bias ? bias[h * D + d0 + j] : 0.f);
+    const float b = (float)hi[j] * rs + (bias ? bias[h * D + d0 + D / 2 + j] : 0.f);
     olo[j] = (bf16)(a * r.x - b * r.y);
     ohi[j] = (bf16)(b * r.x + a * r.y);
   }
@@ -220,18 +222,18 @@ __global__ __launch_bounds__(256) void rope_kv_kernel(
 
 void launch_rope_kv(const void* qkv, const int* pos, const int* slots, const void* cos_sin,
                     void* q_out, void* k_cache, void* v_cache, int T, int Hq, int Hkv, int D,
-                    int BS, hipStream_t s) {
+                    int BS, hipStream_t s, const float* bias) {
   if (T <= 0) return;
   const size_t total = (size_t)T * (Hq + 2 * Hkv) * (D / 16);
   const int grid = (int)((total + 255) / 256);
   if (D == 128)
     rope_kv_kernel<128><<<grid, 256, 0, s>>>((const bf16*)qkv, pos, slots, (const float2*)cos_sin,
                                              (bf16*)q_out, (bf16*)k_cache, (bf16*)v_cache, T, Hq,
-                                             Hkv, BS, norm_epi());
+                                             Hkv, BS, norm_epi(), bias);
   else if (D == 64)
     rope_kv_kernel<64><<<grid, 256, 0, s>>>((const bf16*)qkv, pos, slots, (const float2*)cos_sin,
                                             (bf16*)q_out, (bf16*)k_cache, (bf16*)v_cache, T, Hq,
-                                            Hkv, BS, norm_epi());
+                                            Hkv, BS, norm_epi(), bias);
 }
 
 // ------------------------------------------------------------ residual add
@@ -284,60 +286,96 @@ void launch_copy_blocks(void* data, const int* src, const int* dst, int npairs, 
 // qkv: [T, Hq DK + Hkv DK + Hkv DV] from the QKV projection, ``bias`` (fp32,
 // one per column, or null) added first.  Queries and keys rotate as halves
 // (dimension j with j + DK / 2; cos_sin [max_pos, DK / 2] float2 holds the
-// identity for pairs that do not rotate), values pass.  One thread per 8
-// elements: 4 + 4 of a q / k head, 8 of a v head.
+// identity for pairs that do not rotate), values pass.  One thread per 16
+// elements: 8 + 8 of a q / k head, 2 x 8 of a v head.
+DEV void load8(const bf16* p, float (&v)[8]) {
+  const bf16x8 x = *reinterpret_cast<const bf16x8*>(p);
+#pragma unroll
+  for (int j = 0; j < 8; ++j) v[j] = (float)x[j];
+}
+DEV void load8(const float* p, float (&v)[8]) {
+#pragma unroll
+  for (int h = 0; h < 2; ++h) {
+    const f32x4 x = reinterpret_cast<const f32x4*>(p)[h];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) v[4 * h + j] = x[j];
+  }
+}
+DEV void store8(bf16* p, const float (&v)[8]) {
+  bf16x8 x;
+#pragma unroll
+  for (int j = 0; j < 8; ++j) x[j] = (bf16)v[j];
+  *reinterpret_cast<bf16x8*>(p) = x;
+}
+DEV void store8(float* p, const float (&v)[8]) {
+#pragma unroll
+  for (int h = 0; h < 2; ++h)
+    reinterpret_cast<f32x4*>(p)[h] = f32x4{v[4 * h], v[4 * h + 1], v[4 * h + 2], v[4 * h + 3]};
+}
+
 template <class T>
 __global__ __launch_bounds__(256) void rope_kv_any_kernel(
     const T* __restrict__ qkv, const float* __restrict__ bias, const int* __restrict__ pos,
     const int* __restrict__ slots, const float2* __restrict__ cos_sin, T* __restrict__ q_out,
     T* __restrict__ k_cache, T* __restrict__ v_cache, int T_, int Hq, int Hkv, int DK, int DV,
     int BS) {
-  const int uk = DK / 8, uv = DV / 8;
+  const int uk = DK / 16, uv = DV / 16;
   const int per = (Hq + Hkv) * uk + Hkv * uv;
   const int N = (Hq + Hkv) * DK + Hkv * DV;
   const size_t i = blockIdx.x * 256ull + threadIdx.x;
   if (i >= (size_t)T_ * per) return;
   const int t = (int)(i / per);
   int u = (int)(i % per);
-  const T* src = qkv + (size_t)t * N;
-  if (u >= (Hq + Hkv) * uk) {                          // value head
-    u -= (Hq + Hkv) * uk;
-    const int slot = slots[t];
-    if (slot < 0) return;
-    const int h = u / uv, d = (u % uv) * 8;
-    const int col = (Hq + Hkv) * DK + h * DV + d;
-    T* dst = v_cache + (((size_t)(slot / BS) * Hkv + h) * BS + slot % BS) * DV + d;
-#pragma unroll
-    for (int j = 0; j < 8; ++j) dst[j] = (T)((float)src[col + j] + (bias ? bias[col + j] : 0.f));
-    return;
-  }
-  const int h = u / uk, d = (u % uk) * 4;
-  const int col = h * DK + d;
+  const bool is_v = u >= (Hq + Hkv) * uk;
+  if (is_v) u -= (Hq + Hkv) * uk;
+  const int ph = is_v ? uv : uk, h = u / ph, d = (u % ph) * 8;
+  const int second = is_v ? DV / 2 : DK / 2;           // the thread's other 8 elements
+  const int col = is_v ? (Hq + Hkv) * DK + h * DV + d : h * DK + d;
   T* dst;
-  if (h < Hq) {
+  if (!is_v && h < Hq) {
     dst = q_out + ((size_t)t * Hq + h) * DK + d;
   } else {
     const int slot = slots[t];
     if (slot < 0) return;
-    dst = k_cache + (((size_t)(slot / BS) * Hkv + (h - Hq)) * BS + slot % BS) * DK + d;
+    const size_t blk = (size_t)(slot / BS) * Hkv;
+    dst = is_v ? v_cache + ((blk + h) * BS + slot % BS) * DV + d
+               : k_cache + ((blk + h - Hq) * BS + slot % BS) * DK + d;
   }
-  const float2* cs = cos_sin + (size_t)pos[t] * (DK / 2) + d;
+  float a[8], b[8];
+  load8(qkv + (size_t)t * N + col, a);
+  load8(qkv + (size_t)t * N + col + second, b);
+  if (bias) {
+    float ba[8], bb[8];
+    load8(bias + col, ba);
+    load8(bias + col + second, bb);
 #pragma unroll
-  for (int j = 0; j < 4; ++j) {
-    const float2 r = cs[j];
-    const float a = (float)src[col + j] + (bias ? bias[col + j] : 0.f);
-    const float b = (float)src[col + DK / 2 + j] + (bias ? bias[col + DK / 2 + j] : 0.f);
-    dst[j] = (T)(a * r.x - b * r.y);
-    dst[DK / 2 + j] = (T)(b * r.x + a * r.y);
+    for (int j = 0; j < 8; ++j) {
+      a[j] += ba[j];
+      b[j] += bb[j];
+    }
   }
+  if (!is_v) {
+    const float4* cs = reinterpret_cast<const float4*>(cos_sin + (size_t)pos[t] * (DK / 2) + d);
+#pragma unroll
+    for (int j = 0; j < 8; j += 2) {
+      const float4 r = cs[j / 2];                      // (cos, sin) of two pairs
+      const float a0 = a[j], b0 = b[j], a1 = a[j + 1], b1 = b[j + 1];
+      a[j] = a0 * r.x - b0 * r.y;
+      b[j] = b0 * r.x + a0 * r.y;
+      a[j + 1] = a1 * r.z - b1 * r.w;
+      b[j + 1] = b1 * r.z + a1 * r.w;
+    }
+  }
+  store8(dst, a);
+  store8(dst + second, b);
 }
 
 int launch_rope_kv_any(const void* qkv, const float* bias, const int* pos, const int* slots,
                        const void* cos_sin, void* q_out, void* k_cache, void* v_cache, int T, int Hq,
                        int Hkv, int DK, int DV, int BS, bool f32, hipStream_t s) {
   if (T <= 0) return 0;
-  if (DK % 8 || DV % 8) return 1;
-  const size_t total = (size_t)T * ((Hq + Hkv) * (DK / 8) + Hkv * (DV / 8));
+  if (DK % 16 || DV % 16) return 1;
+  const size_t total = (size_t)T * ((Hq + Hkv) * (DK / 16) + Hkv * (DV / 16));
   const unsigned grid = (unsigned)((total + 255) / 256);
   if (f32)
     rope_kv_any_kernel<float><<<grid, 256, 0, s>>>((const float*)qkv, bias, pos, slots,

@@ -607,6 +607,14 @@ __global__ __launch_bounds__(256) void splitk_reduce_rope(const float* __restric
     hi[j] = hi0[j] * rs;
     hi[4 + j] = hi1[j] * rs;
   }
+  if (ra.bias) {
+    const float* b = ra.bias + h * D + d0;
+#pragma unroll
+    for (int j = 0; j < 8; ++j) {
+      lo[j] += b[j];
+      hi[j] += b[D / 2 + j];
+    }
+  }
   bf16x8 olo, ohi;
   bf16* dst;
   if (h >= ra.Hq + ra.Hkv) {                           // V: copy into the cache
@@ -694,9 +702,22 @@ static void launch_gemm_tn_128(const void* X, const void* W, void* Y, const void
                                         K, norm_epi());
 }
 
-// fp32-output variant (retrieval scores: bf16 would tie near-equal cosines)
+static bool skinny_first(int M, int N, int K);
+
+// fp32-output variant (retrieval scores: bf16 would tie near-equal cosines;
+// products that enter an fp32 residual; logits).  Decode-sized M and too few
+// 128^2 tiles for the CUs: the weight-streaming kernels with fp32 stores.
 void launch_gemm_tn_f32out(const void* X, const void* W, float* Y, int M, int N, int K,
                            hipStream_t s) {
+  if (M <= GEMM_STREAM_MAX_M && (N + BN - 1) / BN < gemm256_num_cus()) {
+    NormEpi ne;
+    ne.y32 = Y;
+    NormEpiScope scope(ne);
+    if (skinny_first(M, N, K) && launch_gemm_skinny(X, W, nullptr, nullptr, M, N, K, 0, s) == 0) return;
+    if (gemm_stream_enabled() && launch_gemm_stream(X, W, nullptr, nullptr, M, N, K, 0, RopeArgs{}, s) == 0)
+      return;
+    if (launch_gemm_skinny(X, W, nullptr, nullptr, M, N, K, 0, s) == 0) return;
+  }
   const int nm = (M + BM - 1) / BM, nn = (N + BN - 1) / BN;
   gemm_tn_128<0, float><<<dim3(nm * nn), 256, 0, s>>>((const bf16*)X, (const bf16*)W, Y,
                                                       nullptr, M, N, K, NormEpi{});

@@ -441,6 +441,17 @@ __global__ __launch_bounds__(256, 1) void gemm_tn_256d(const bf16* __restrict__ 
 #pragma unroll
       for (int mt = 0; mt < MTW; ++mt) rpos[mt] = ra.pos[min(m0 + wm * WROWS + mt * 16 + fr, M - 1)];
     }
+    // EPI 3: projection biases of the lane's columns (0 when none)
+    f32x4 bia[EPI == 3 ? 8 : 1];
+    if constexpr (EPI == 3) {
+#pragma unroll
+      for (int nt_ = 0; nt_ < 8; ++nt_) bia[nt_] = f32x4{0.f, 0.f, 0.f, 0.f};
+      if (ra.bias) {
+#pragma unroll
+        for (int nt_ = 0; nt_ < 8; ++nt_)
+          bia[nt_] = *reinterpret_cast<const f32x4*>(ra.bias + head * 128 + nt_ * 16 + fq * 4);
+      }
+    }
     // EPI 2 / 3: fused RMSNorm of the input rows (1 when none), loaded up front
     float rsc[EPI >= 2 ? MTW : 1];
     if constexpr (EPI >= 2) {
@@ -470,7 +481,8 @@ __global__ __launch_bounds__(256, 1) void gemm_tn_256d(const bf16* __restrict__ 
           for (int j = 0; j < 4; ++j) {
             const f32x4 cc = c4[nt_][j >> 1];
             const float rc = cc[(j & 1) * 2], rs = cc[(j & 1) * 2 + 1];
-            const float x1 = acc[mt][nt_][j] * rsc[mt], x2 = acc[mt][nt_ + 4][j] * rsc[mt];
+            const float x1 = acc[mt][nt_][j] * rsc[mt] + bia[EPI == 3 ? nt_ : 0][j];
+            const float x2 = acc[mt][nt_ + 4][j] * rsc[mt] + bia[EPI == 3 ? nt_ + 4 : 0][j];
             o1[j] = (bf16)(x1 * rc - x2 * rs);
             o2[j] = (bf16)(x2 * rc + x1 * rs);
           }
@@ -493,7 +505,8 @@ __global__ __launch_bounds__(256, 1) void gemm_tn_256d(const bf16* __restrict__ 
         for (int nt_ = 0; nt_ < 8; ++nt_) {
           bf16x4 o;
 #pragma unroll
-          for (int j = 0; j < 4; ++j) o[j] = (bf16)(EPI == 3 ? acc[mt][nt_][j] * rsc[mt] : acc[mt][nt_][j]);
+          for (int j = 0; j < 4; ++j) o[j] = (bf16)(EPI == 3 ? acc[mt][nt_][j] * rsc[mt] + bia[EPI == 3 ? nt_ : 0][j]
+                                                          : acc[mt][nt_][j]);
           put(row, nt_ * 16 + fq * 4, o);
         }
       }
@@ -767,7 +780,7 @@ int launch_qkv_rope_algo(const void* X, const void* W, void* qkv, int M, int N, 
   if (algo == 500) {
     launch_gemm_tn(X, W, qkv, nullptr, M, N, K, s);
     launch_rope_kv(qkv, ra.pos, ra.slots, ra.cos_sin, ra.q_out, ra.k_cache, ra.v_cache, M, ra.Hq,
-                   ra.Hkv, D, ra.BS, s);
+                   ra.Hkv, D, ra.BS, s, ra.bias);
     return 0;
   }
   if (algo == 200) return launch_gemm_stream(X, W, nullptr, nullptr, M, N, K, 3, ra, s);
@@ -799,7 +812,7 @@ void launch_qkv_rope(const void* X, const void* W, void* qkv, int M, int N, int 
     return;
   launch_gemm_tn(X, W, qkv, nullptr, M, N, K, s);
   launch_rope_kv(qkv, ra.pos, ra.slots, ra.cos_sin, ra.q_out, ra.k_cache, ra.v_cache, M, ra.Hq,
-                 ra.Hkv, D, ra.BS, s);
+                 ra.Hkv, D, ra.BS, s, ra.bias);
 }
 
 int launch_gemm_tn_256d(const void* X, const void* W, void* Y, const void* R, int M, int N, int K,

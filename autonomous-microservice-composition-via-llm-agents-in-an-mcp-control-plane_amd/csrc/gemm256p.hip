@@ -297,6 +297,16 @@ __global__ __launch_bounds__(256, 1) void gemm_tn_256p(const bf16* __restrict__ 
         rres[i] = *reinterpret_cast<const bf16x8*>(R + (size_t)m * ldy + col0 + lc * 8);
       }
     }
+    f32x4 bia[EPI == 3 ? 8 : 1];                     // projection biases (0 when none)
+    if constexpr (EPI == 3) {
+#pragma unroll
+      for (int nt_ = 0; nt_ < 8; ++nt_) bia[nt_] = f32x4{0.f, 0.f, 0.f, 0.f};
+      if (ra.bias) {
+#pragma unroll
+        for (int nt_ = 0; nt_ < 8; ++nt_)
+          bia[nt_] = *reinterpret_cast<const f32x4*>(ra.bias + head * 128 + nt_ * 16 + fq * 4);
+      }
+    }
     int rpos[MTW];
     if (EPI == 3 && rotate) {
 #pragma unroll
@@ -355,7 +365,8 @@ __global__ __launch_bounds__(256, 1) void gemm_tn_256p(const bf16* __restrict__ 
             for (int e = 0; e < 4; ++e) {
               const f32x4 cc = c4[nt_][e >> 1];
               const float rc = cc[(e & 1) * 2], rs = cc[(e & 1) * 2 + 1];
-              const float x1 = acc[mt][nt_][e] * rsc[mt], x2 = acc[mt][nt_ + 4][e] * rsc[mt];
+              const float x1 = acc[mt][nt_][e] * rsc[mt] + bia[EPI == 3 ? nt_ : 0][e];
+              const float x2 = acc[mt][nt_ + 4][e] * rsc[mt] + bia[EPI == 3 ? nt_ + 4 : 0][e];
               o1[e] = (bf16)(x1 * rc - x2 * rs);
               o2[e] = (bf16)(x2 * rc + x1 * rs);
             }
@@ -378,7 +389,8 @@ __global__ __launch_bounds__(256, 1) void gemm_tn_256p(const bf16* __restrict__ 
           for (int nt_ = 0; nt_ < 8; ++nt_) {
             bf16x4 o;
 #pragma unroll
-            for (int e = 0; e < 4; ++e) o[e] = (bf16)(EPI == 3 ? acc[mt][nt_][e] * rsc[mt] : acc[mt][nt_][e]);
+            for (int e = 0; e < 4; ++e) o[e] = (bf16)(EPI == 3 ? acc[mt][nt_][e] * rsc[mt] + bia[EPI == 3 ? nt_ : 0][e]
+                                                            : acc[mt][nt_][e]);
             put(row, nt_ * 16 + fq * 4, o);
           }
         }

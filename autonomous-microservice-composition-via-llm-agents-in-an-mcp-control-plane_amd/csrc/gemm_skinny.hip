@@ -189,6 +189,12 @@ __global__ __launch_bounds__(64 * WV) void gemm_skinny(const bf16* __restrict__ 
 #pragma unroll
         for (int q = 0; q < 4; ++q) v[q] += (float)pre_rr[mb][q];
       }
+      if constexpr (EPI == 0) {
+        if (ne.y32) {
+          *reinterpret_cast<f32x4*>(ne.y32 + (size_t)m * N + n) = v;
+          continue;
+        }
+      }
       bf16x4 o;
 #pragma unroll
       for (int q = 0; q < 4; ++q) o[q] = (bf16)v[q];

@@ -263,8 +263,19 @@ __global__ __launch_bounds__(256 * MH, MH == 1 ? 2 : 1) void gemm_stream(const b
   //      of token m = 16 mm + r.  Its row inputs were loaded at kernel entry;
   //      EPI 3's (cos, sin) pairs (they need the position) go out together here
   static_assert(UPW_ == UPW && FPU_ == FPU, "prefetch geometry");
-  f32x4 pre_cs[EPI == 3 ? UPW : 1][2];
+  f32x4 pre_cs[EPI == 3 ? UPW : 1][2], pre_b[EPI == 3 ? UPW : 1][2];
   if constexpr (EPI == 3) {
+#pragma unroll
+    for (int a = 0; a < UPW; ++a) pre_b[a][0] = pre_b[a][1] = f32x4{0.f, 0.f, 0.f, 0.f};
+    if (ra.bias) {
+#pragma unroll
+      for (int a = 0; a < UPW; ++a) {
+        const int u = min(wave + a * SW_WAVES, NU - 1);
+        const int d = 32 * (tile & 1) + 16 * ((2 * (u / MF)) >> 1) + 4 * g;
+        pre_b[a][0] = *reinterpret_cast<const f32x4*>(ra.bias + (tile >> 1) * 128 + d);
+        pre_b[a][1] = *reinterpret_cast<const f32x4*>(ra.bias + (tile >> 1) * 128 + d + 64);
+      }
+    }
     if ((tile >> 1) < ra.Hq + ra.Hkv) {              // q / k heads rotate (v heads do not)
 #pragma unroll
       for (int a = 0; a < UPW; ++a) {
@@ -297,7 +308,8 @@ __global__ __launch_bounds__(256 * MH, MH == 1 ? 2 : 1) void gemm_stream(const b
     } else if constexpr (EPI == 3) {
       const int head = tile >> 1;
       const int d = 32 * (tile & 1) + 16 * (f0 >> 1) + 4 * g;       // first of 4 dims (< 64)
-      const f32x4 x1 = sum[a][0] * rs, x2 = sum[a][1] * rs;
+      const f32x4 x1 = sum[a][0] * rs + pre_b[EPI == 3 ? a : 0][0];
+      const f32x4 x2 = sum[a][1] * rs + pre_b[EPI == 3 ? a : 0][1];
       bf16x4 o1, o2;
       const bool is_v = head >= ra.Hq + ra.Hkv;
       if (is_v) {
@@ -336,6 +348,12 @@ __global__ __launch_bounds__(256 * MH, MH == 1 ? 2 : 1) void gemm_stream(const b
         if constexpr (EPI == 1) {
 #pragma unroll
           for (int i = 0; i < 4; ++i) v[i] += (float)pre_rr[a][j][i];
+        }
+        if constexpr (EPI == 0) {
+          if (ne.y32) {
+            *reinterpret_cast<f32x4*>(ne.y32 + (size_t)m * N + n) = v;
+            continue;
+          }
         }
         bf16x4 o;
 #pragma unroll

@@ -17,6 +17,8 @@ struct NormEpi {
   unsigned long long* ss_out = nullptr;     // [M] fixed point (common.h SS_FIX), zeroed by the caller
   const unsigned long long* ss_in = nullptr;
   float inv_h = 0.f, eps = 0.f;
+  // EPI 0 of the weight-streaming kernels: fp32 rows here instead of bf16 ones to Y
+  float* y32 = nullptr;
   // gated activation of EPI 2 (common.h gated_act): g sigmoid(g (act_c0 + act_c1 g^2)) u;
   // (1, 0) is SwiGLU, the pair below the tanh form of gelu
   float act_c0 = 1.f, act_c1 = 0.f;
@@ -41,10 +43,10 @@ void launch_silu_mul(const void* x, void* y, int T, int F, hipStream_t s);
 void launch_embedding(const int* ids, const void* table, void* out, int T, int H, hipStream_t s);
 void launch_rope_kv(const void* qkv, const int* pos, const int* slots, const void* cos_sin,
                     void* q_out, void* k_cache, void* v_cache, int T, int Hq, int Hkv, int D,
-                    int BS, hipStream_t s);
+                    int BS, hipStream_t s, const float* bias = nullptr);
 void launch_add_inplace(void* y, const void* x, size_t n, hipStream_t s);
 
-// any head sizes, q / k / v biases (fp32 or null), bf16 or f32; nonzero: head sizes not multiples of 8
+// any head sizes, q / k / v biases (fp32 or null), bf16 or f32; nonzero: head sizes not multiples of 16
 int launch_rope_kv_any(const void* qkv, const float* bias, const int* pos, const int* slots,
                        const void* cos_sin, void* q_out, void* k_cache, void* v_cache, int T, int Hq,
                        int Hkv, int DK, int DV, int BS, bool f32, hipStream_t s);
@@ -86,8 +88,11 @@ struct MaskedAttnArgs {
   float* split_o;
   float* split_ml;
   int rows;
+  int* tickets;              // set by the launcher
 };
 int launch_attn_masked(const MaskedAttnArgs& a, int nwork, int form, int nz, hipStream_t s);
+constexpr int ATTN_SPLIT_TICKETS = 1 << 16;
+int* attn_split_counters();  // this device's tickets, zero between launches (attention.hip)
 int launch_attn_row(const MaskedAttnArgs& a, int T, bool f32, hipStream_t s);
 
 // QKV projection + RoPE + paged K/V write fused in the GEMM epilogue (K1+K4+K10)
@@ -123,6 +128,7 @@ struct RopeArgs {
   void* k_cache;           // [nb, Hkv, BS, D]
   void* v_cache;
   int Hq, Hkv, BS;
+  const float* bias = nullptr;   // q / k / v projection biases [(Hq + 2 Hkv) D], added before the rotation
 };
 // fused when the AGPR GEMM serves the shape (D = 128), else GEMM into qkv + rope_kv
 void launch_qkv_rope(const void* X, const void* W, void* qkv, int M, int N, int K, int D,

@@ -32,35 +32,44 @@ DEV void store4(T* p, const f32x4& v) {
   *reinterpret_cast<typename Vec4<T>::type*>(p) = o;
 }
 
+template <int NT>
 DEV float block_sum(float v, float* red) {
   v = wave_sum(v);
-  __syncthreads();                                   // red is free again
   if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = v;
   __syncthreads();
-  return red[0] + red[1] + red[2] + red[3];
+  float t = 0.f;
+#pragma unroll
+  for (int w = 0; w < NT / 64; ++w) t += red[w];
+  return t;
 }
 
-// One 256-thread block per row, 4 floats per thread and step, the row in
-// registers between the passes:
+// One block per row (1024 threads for few rows: shorter chains; 256 otherwise),
+// 4 floats per thread and step, the row and the norm weights in registers
+// between the passes:
 //   y given:      x += y / rms(y) * w_post          (written back)
 //   w_pre given:  out = x / rms(x) * w_pre,  else out = x   (as T, row stride ld)
 // Rows are Hp wide (columns >= H are zero and stay zero), means are over H.
-template <class T, int VMAX>
-__global__ __launch_bounds__(256) void residual_norm_kernel(
+template <class T, int VMAX, int NT>
+__global__ __launch_bounds__(NT) void residual_norm_kernel(
     float* __restrict__ x, const T* __restrict__ y, const float* __restrict__ w_post,
     const float* __restrict__ w_pre, T* __restrict__ out, int ld, int H, int Hp, float eps) {
-  __shared__ float red[4];
+  __shared__ float red[2][NT / 64];
   const int row = blockIdx.x, nvec = Hp >> 2;
   float* xr = x + (size_t)row * Hp;
   const float inv_h = 1.f / (float)H;
-  f32x4 xv[VMAX], yv[VMAX];
+  constexpr bool EARLY = VMAX <= 2;                  // weights fit the registers too
+  f32x4 xv[VMAX], yv[VMAX], wa[EARLY ? VMAX : 1], wb[EARLY ? VMAX : 1];
 #pragma unroll
   for (int i = 0; i < VMAX; ++i) {
-    const int c = threadIdx.x + i * 256;
+    const int c = threadIdx.x + i * NT;
     xv[i] = yv[i] = f32x4{0.f, 0.f, 0.f, 0.f};
     if (c < nvec) {
       xv[i] = *reinterpret_cast<const f32x4*>(xr + 4 * c);
       if (y) yv[i] = load4(y + (size_t)row * Hp + 4 * c);
+      if constexpr (EARLY) {
+        if (y) wa[i] = *reinterpret_cast<const f32x4*>(w_post + 4 * c);
+        if (w_pre) wb[i] = *reinterpret_cast<const f32x4*>(w_pre + 4 * c);
+      }
     }
   }
   if (y) {
@@ -69,12 +78,12 @@ __global__ __launch_bounds__(256) void residual_norm_kernel(
     for (int i = 0; i < VMAX; ++i)
 #pragma unroll
       for (int j = 0; j < 4; ++j) ss += yv[i][j] * yv[i][j];
-    const float inv = 1.f / sqrtf(block_sum(ss, red) * inv_h + eps);
+    const float inv = 1.f / sqrtf(block_sum<NT>(ss, red[0]) * inv_h + eps);
 #pragma unroll
     for (int i = 0; i < VMAX; ++i) {
-      const int c = threadIdx.x + i * 256;
+      const int c = threadIdx.x + i * NT;
       if (c < nvec) {
-        const f32x4 w = *reinterpret_cast<const f32x4*>(w_post + 4 * c);
+        const f32x4 w = EARLY ? wa[EARLY ? i : 0] : *reinterpret_cast<const f32x4*>(w_post + 4 * c);
 #pragma unroll
         for (int j = 0; j < 4; ++j) xv[i][j] += yv[i][j] * inv * w[j];
         *reinterpret_cast<f32x4*>(xr + 4 * c) = xv[i];
@@ -89,16 +98,16 @@ __global__ __launch_bounds__(256) void residual_norm_kernel(
     for (int i = 0; i < VMAX; ++i)
 #pragma unroll
       for (int j = 0; j < 4; ++j) ss += xv[i][j] * xv[i][j];
-    inv = 1.f / sqrtf(block_sum(ss, red) * inv_h + eps);
+    inv = 1.f / sqrtf(block_sum<NT>(ss, red[1]) * inv_h + eps);
   }
   T* orow = out + (size_t)row * ld;
 #pragma unroll
   for (int i = 0; i < VMAX; ++i) {
-    const int c = threadIdx.x + i * 256;
+    const int c = threadIdx.x + i * NT;
     if (c < nvec) {
       f32x4 o = xv[i];
       if (w_pre) {
-        const f32x4 w = *reinterpret_cast<const f32x4*>(w_pre + 4 * c);
+        const f32x4 w = EARLY ? wb[EARLY ? i : 0] : *reinterpret_cast<const f32x4*>(w_pre + 4 * c);
 #pragma unroll
         for (int j = 0; j < 4; ++j) o[j] = o[j] * inv * w[j];
       }
@@ -110,14 +119,21 @@ __global__ __launch_bounds__(256) void residual_norm_kernel(
 template <class T>
 void residual_norm_dispatch(float* x, const T* y, const float* w_post, const float* w_pre, T* out,
                             int ld, int rows, int H, int Hp, float eps, hipStream_t s) {
+#define RN_CASE(V, NT) \
+  residual_norm_kernel<T, V, NT><<<rows, NT, 0, s>>>(x, y, w_post, w_pre, out, ld, H, Hp, eps)
+  if (rows <= 512 && Hp > 1024) {
+    const int v = (Hp / 4 + 1023) / 1024;
+    if (v <= 1) RN_CASE(1, 1024);
+    else if (v <= 2) RN_CASE(2, 1024);
+    else RN_CASE(4, 1024);
+    return;
+  }
   const int v = (Hp / 4 + 255) / 256;
-#define RN_CASE(V) \
-  residual_norm_kernel<T, V><<<rows, 256, 0, s>>>(x, y, w_post, w_pre, out, ld, H, Hp, eps)
-  if (v <= 1) RN_CASE(1);
-  else if (v <= 2) RN_CASE(2);
-  else if (v <= 4) RN_CASE(4);
-  else if (v <= 8) RN_CASE(8);
-  else RN_CASE(16);
+  if (v <= 1) RN_CASE(1, 256);
+  else if (v <= 2) RN_CASE(2, 256);
+  else if (v <= 4) RN_CASE(4, 256);
+  else if (v <= 8) RN_CASE(8, 256);
+  else RN_CASE(16, 256);
 #undef RN_CASE
 }
 

@@ -312,9 +312,16 @@ def qkv_rope(h, wqkv, pos, slots, cos_sin, q_out, k_cache, v_cache, Hq, Hkv, D, 
 
 def qkv_rope_bias(h, wqkv, bias, pos, slots, cos_sin, q_out, k_cache, v_cache):
     """``qkv_rope`` with projection biases (fp32 [N]) and key / value heads of
-    any sizes (multiples of 8): sizes come from q_out [T, Hq, DK] and the
-    caches.  Pairs that do not rotate hold (1, 0) in ``cos_sin``."""
+    any sizes (multiples of 16): sizes come from q_out [T, Hq, DK] and the
+    caches.  Pairs that do not rotate hold (1, 0) in ``cos_sin``.  d = 128
+    runs the projection's fused epilogue, other sizes GEMM + rope_kv_any."""
     if h.is_cuda:
+        Hq, DK, Hkv = q_out.shape[1], q_out.shape[2], k_cache.shape[1]
+        if h.dtype == torch.bfloat16 and DK == v_cache.shape[3] == 128:
+            qkv = h.new_empty(h.shape[0], wqkv.shape[0])     # scratch of the unfused shapes
+            lib().qkv_rope(h, wqkv, qkv, pos, slots, cos_sin, q_out, k_cache, v_cache, Hq, Hkv, DK,
+                           None, 0.0, bias)
+            return q_out
         qkv = gemm(h, wqkv)
         lib().rope_kv_any(qkv, bias, pos, slots, cos_sin, q_out, k_cache, v_cache)
         return q_out
@@ -609,8 +616,10 @@ def masked_attention(q, k_cache, v_cache, meta, scale, group: int, soft_cap: flo
             for nw, ws, wq in meta.work_lists():
                 nz, so, sm = 1, None, None
                 if nw == 1 and int(meta.kv_splits) > 1:
-                    # a block's 4 waves share the keys already
-                    nz = max(1, int(meta.kv_splits) // _MASKED_SPLIT_DIV)
+                    # a block's 4 waves share the keys already; the partials are
+                    # addressed with 31 bits
+                    nz = max(1, min(int(meta.kv_splits) // _MASKED_SPLIT_DIV,
+                                    (1 << 31) // max(1, 4 * out.numel()) - 1))
                 if nz > 1:
                     so = torch.empty(nz, *out.shape, device=q.device, dtype=torch.float32)
                     sm = torch.empty(nz, q.shape[0], q.shape[1], 2, device=q.device, dtype=torch.float32)

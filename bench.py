@@ -78,11 +78,23 @@ def parse_args(argv=None):
     ap.add_argument("--overlap", type=float, default=0.0,
                     help="submit the next batch once this fraction of the current one is still "
                          "running (0: closed batches)")
+    ap.add_argument("--compare", choices=["dozazen"],
+                    help="instead of the headline workload: prefill and decode throughput of this "
+                         "design's layers beside Llama's at equal sizes (utils/layerbench.py)")
+    ap.add_argument("--compare-sizes", help="comma-separated sizes of --compare")
+    ap.add_argument("--compare-phases", help="comma-separated phases of --compare")
+    ap.add_argument("--compare-only", help="run one side of --compare (profiling)")
     return ap.parse_args(argv)
 
 
 def main():
     args = parse_args()
+    if args.compare:
+        from mcp_amd.utils import layerbench
+        split = lambda v: v.split(",") if v else None
+        layerbench.run(args.compare, split(args.compare_sizes), split(args.compare_phases),
+                       split(args.compare_only))
+        return
     from mcp_amd.parallel.launch import check_devices, self_launch
     rc = self_launch(args.gpus)          # parent of N ranks: never touches the GPU
     if rc is not None:
