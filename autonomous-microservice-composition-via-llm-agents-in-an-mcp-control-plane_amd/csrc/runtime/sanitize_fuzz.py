@@ -89,8 +89,10 @@ def random_step(cascade):
         nblk += len(blocks)
         toks = [rng.randrange(128256) for _ in range(take + rng.randint(0, 3))]
         sample = rng.random() < 0.6
+        if rng.random() < 0.2:                         # chosen rows instead of the last one
+            sample = [rng.randrange(take) for _ in range(rng.randint(0, 4))]
         entries.append((toks, take, start, blocks, 128 if cascade and s < 5 else 0, sample))
-        if sample:
+        for _ in range(len(sample) if isinstance(sample, list) else int(sample)):
             allowed.append([rng.randrange(128256) for _ in range(rng.randint(1, 40))])
             ctr.append(rng.randrange(1 << 31))
     copies = [(rng.randrange(4096), rng.randrange(4096)) for _ in range(rng.randint(0, 5))]
@@ -111,6 +113,8 @@ h, l = rt.pack_step([], BS, 4, [(1, 2)])            # copy-only step
 assert int(sum(l)) == h.size
 expect(ValueError, rt.pack_step, [([1, 2], 3, 0, [0], 0, False)], BS, 4)          # take > len(tokens)
 expect(ValueError, rt.pack_step, [([1, 2], 0, 0, [0], 0, False)], BS, 4)          # empty span
+expect(ValueError, rt.pack_step, [([1, 2], 2, 0, [0], 0, [0, 2])], BS, 4)         # row past the span
+expect(ValueError, rt.pack_step, [([1, 2], 2, 0, [0], 0, [-1])], BS, 4)
 expect(ValueError, rt.pack_step, [([1] * 70, 70, 0, [0], 0, False)], BS, 4)       # too few blocks
 expect(ValueError, rt.pack_step, [([1], 1, 0, [0], 0, True)], BS, 4, None, None, 0, [], [])
 expect(ValueError, rt.pack_step, [([1], 1, 0, [0], 0, True)], BS, 4, None, None, 0, [[1]], [])

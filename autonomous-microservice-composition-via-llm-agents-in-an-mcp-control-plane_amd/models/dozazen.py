@@ -125,7 +125,8 @@ def config_from_json(c: dict, name: str = "dozazen", max_pos: int = MAX_POS) -> 
         m, mlp = ly["mixer"], ly.get("mlp")
         if mlp is not None and mlp["kind"] != "dense":
             raise NotImplementedError(f"layer {i}: feed-forward kind {mlp['kind']!r}")
-        r, sc = m["rot"], m["rot"].get("scaling")
+        r = m.get("rot") or {"dims": 0, "base": 1.0}
+        sc = r.get("scaling")
         if m["heads"] % m["kv_heads"] or r["dims"] % 2 or r["dims"] > m["dim"]:
             raise ValueError(f"layer {i}: heads {m['heads']} / {m['kv_heads']}, rotated dimensions "
                              f"{r['dims']} of {m['dim']}")
@@ -218,8 +219,8 @@ def half_rotation_order(dim: int, rot_dims: int, padded: int) -> torch.Tensor:
     that do not rotate to the rows left over."""
     at = torch.full((padded,), -1, dtype=torch.long)
     half = rot_dims // 2
-    at[:half] = torch.arange(0, rot_dims, 2)
-    at[padded // 2:padded // 2 + half] = torch.arange(1, rot_dims, 2)
+    at[:half] = 2 * torch.arange(half)
+    at[padded // 2:padded // 2 + half] = 2 * torch.arange(half) + 1
     free = (at < 0).nonzero().flatten()
     at[free[:dim - rot_dims]] = torch.arange(rot_dims, dim)
     return at
@@ -345,7 +346,8 @@ class DozazenModel:
     def _table(self, rot: Rotary, padded: int) -> torch.Tensor:
         cs = torch.zeros(self.cfg.max_pos, padded // 2, 2)
         cs[..., 0] = 1.0
-        cs[:, :rot.dims // 2] = ref.rope_cos_sin(self.cfg.max_pos, rot.dims, rot.base, None, rot.scaling)
+        if rot.dims:
+            cs[:, :rot.dims // 2] = ref.rope_cos_sin(self.cfg.max_pos, rot.dims, rot.base, None, rot.scaling)
         return cs.to(self.device)
 
     @classmethod
