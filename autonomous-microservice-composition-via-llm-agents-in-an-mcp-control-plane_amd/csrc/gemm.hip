@@ -718,6 +718,9 @@ void launch_gemm_tn_f32out(const void* X, const void* W, float* Y, int M, int N,
       return;
     if (launch_gemm_skinny(X, W, nullptr, nullptr, M, N, K, 0, s) == 0) return;
   }
+  if (M > GEMM_STREAM_MAX_M && gemm_select(M, N, K) == 1 &&
+      launch_gemm_tn_256d_f32(X, W, Y, M, N, K, s) == 0)
+    return;
   const int nm = (M + BM - 1) / BM, nn = (N + BN - 1) / BN;
   gemm_tn_128<0, float><<<dim3(nm * nn), 256, 0, s>>>((const bf16*)X, (const bf16*)W, Y,
                                                       nullptr, M, N, K, NormEpi{});

@@ -395,6 +395,19 @@ __global__ __launch_bounds__(256, 1) void gemm_tn_256d(const bf16* __restrict__ 
       store_wide_slab<EPI, MTW>(acc, rsY, R, M, ldy, m0 + wm * WROWS, col0, fr, fq, rsc, ne, slab);
     else
       store_wide<EPI, MTW>(acc, rsY, R, M, ldy, m0 + wm * WROWS, col0, fr, fq, rsc, ne);
+  } else if (EPI == 0 && ne.y32 != nullptr) {
+    // ---- fp32 rows (products that enter an fp32 stream): 16 B per lane, 64
+    //      contiguous bytes of a row per instruction, straight from the
+    //      accumulators
+#pragma unroll
+    for (int mt = 0; mt < MTW; ++mt) {
+      const int m = m0 + wm * WROWS + mt * 16 + fr;
+      float* yr = ne.y32 + (size_t)m * N + n0 + wn * 128 + fq * 4;
+      if (m < M) {
+#pragma unroll
+        for (int nt_ = 0; nt_ < 8; ++nt_) *reinterpret_cast<f32x4*>(yr + nt_ * 16) = acc[mt][nt_];
+      }
+    }
   } else {
     // ---- staged epilogue.  The direct one below stores 8 B per lane in
     //      32-B row pieces (the MFMA layout: lane = 4 columns of one row); at
@@ -756,6 +769,30 @@ static int launch_256d_impl(const void* X, const void* W, void* Y, const void* R
     case 192: return launch_height<192>(X, W, Y, R, M, N, K, epi, grid, group, ra, s);
     case 160: return launch_height<160>(X, W, Y, R, M, N, K, epi, grid, group, ra, s);
     case 128: return launch_height<128>(X, W, Y, R, M, N, K, epi, grid, group, ra, s);
+    default: return 4;
+  }
+}
+
+// fp32 output (norm_epi().y32), data-parallel tiles at the selector's height
+int launch_gemm_tn_256d_f32(const void* X, const void* W, float* Y, int M, int N, int K, hipStream_t s) {
+  if (const int rc = gemm256d_ok(M, N, K)) return rc;
+  const int bm = gemm256d_height(M, N, K), group = gemm256d_group(M, N, K);
+  const dim3 grid(((M + bm - 1) / bm) * ((N + BN - 1) / BN));
+  NormEpi ne;
+  ne.y32 = Y;
+  const RopeArgs ra{};
+  auto x = (const bf16*)X;
+  auto w = (const bf16*)W;
+  switch (bm) {
+#define F32_CASE(H)                                                                             \
+  case H: gemm_tn_256d<0, H><<<grid, 256, 0, s>>>(x, w, nullptr, nullptr, M, N, K, group, ra, ne, \
+                                                  nullptr, nullptr); return 0
+    F32_CASE(256);
+    F32_CASE(224);
+    F32_CASE(192);
+    F32_CASE(160);
+    F32_CASE(128);
+#undef F32_CASE
     default: return 4;
   }
 }

@@ -17,7 +17,7 @@ struct NormEpi {
   unsigned long long* ss_out = nullptr;     // [M] fixed point (common.h SS_FIX), zeroed by the caller
   const unsigned long long* ss_in = nullptr;
   float inv_h = 0.f, eps = 0.f;
-  // EPI 0 of the weight-streaming kernels: fp32 rows here instead of bf16 ones to Y
+  // EPI 0 of the weight-streaming and AGPR kernels: fp32 rows here instead of bf16 ones to Y
   float* y32 = nullptr;
   // gated activation of EPI 2 (common.h gated_act): g sigmoid(g (act_c0 + act_c1 g^2)) u;
   // (1, 0) is SwiGLU, the pair below the tanh form of gelu
@@ -183,6 +183,7 @@ int gemm256d_code_height(int code);     // plan code 1..5 -> AGPR tile height (0
 // probe 0 production, 1 MFMA only, 2 + ds_read + barriers, 3 + LDS-DMA (no stores)
 int launch_gemm_probe(const void* X, const void* W, void* Y, int M, int N, int K, int epi,
                       int probe, hipStream_t s);
+int launch_gemm_tn_256d_f32(const void* X, const void* W, float* Y, int M, int N, int K, hipStream_t s);
 // K-half split form (gemm256d.hip SPLIT 2): two workgroups per tile
 void gemm_pf_force(int p);                           // W L2 fills in the split form: -1 env, 0 / 1
 int launch_gemm_tn_256d_split2(const void* X, const void* W, void* Y, const void* R, int M, int N,

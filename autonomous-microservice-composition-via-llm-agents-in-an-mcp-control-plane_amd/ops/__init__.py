@@ -595,8 +595,6 @@ def paged_attention(q, k_cache, v_cache, meta, scale, out=None):
 
 
 MASKED_MAX_HEAD = 256           # largest head of the MFMA forms (csrc/attention_masked.hip)
-# scheduler split counts are for one wave per split: blocks of 4 waves take fewer
-_MASKED_SPLIT_DIV = int(os.environ.get("MCP_MASKED_SPLIT_DIV", "2"))
 
 
 def masked_attention(q, k_cache, v_cache, meta, scale, group: int, soft_cap: float = 0.0,
@@ -616,10 +614,8 @@ def masked_attention(q, k_cache, v_cache, meta, scale, group: int, soft_cap: flo
             for nw, ws, wq in meta.work_lists():
                 nz, so, sm = 1, None, None
                 if nw == 1 and int(meta.kv_splits) > 1:
-                    # a block's 4 waves share the keys already; the partials are
-                    # addressed with 31 bits
-                    nz = max(1, min(int(meta.kv_splits) // _MASKED_SPLIT_DIV,
-                                    (1 << 31) // max(1, 4 * out.numel()) - 1))
+                    # (the partials are addressed with 31 bits)
+                    nz = max(1, min(int(meta.kv_splits), (1 << 31) // max(1, 4 * out.numel()) - 1))
                 if nz > 1:
                     so = torch.empty(nz, *out.shape, device=q.device, dtype=torch.float32)
                     sm = torch.empty(nz, q.shape[0], q.shape[1], 2, device=q.device, dtype=torch.float32)

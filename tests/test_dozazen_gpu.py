@@ -75,7 +75,7 @@ def test_gemm_f32_is_exact_and_row_independent(M, N, K):
     assert torch.equal(ops.gemm(X[-1:].contiguous(), W), got[-1:])
 
 
-@pytest.mark.parametrize("M", [1, 3, 16, 40, 64, 100, 128, 200, 700])
+@pytest.mark.parametrize("M", [1, 3, 16, 40, 64, 100, 128, 200, 700, 2600])
 @pytest.mark.parametrize("N,K", [(64, 128), (192, 384), (452, 192), (4096, 8192)])
 def test_gemm_f32out(M, N, K):
     X, W = _rnd(M, K, seed=1, dtype=torch.bfloat16), _rnd(N, K, seed=2, dtype=torch.bfloat16)
