@@ -16,6 +16,7 @@ from __future__ import annotations
 
 import argparse
 import concurrent.futures as cf
+import contextlib
 import os
 import shutil
 import subprocess
@@ -92,10 +93,11 @@ def build(force: bool = False, jobs: int = 8, verbose: bool = False) -> Path:
     with cf.ThreadPoolExecutor(max_workers=max(1, jobs)) as ex:
         list(ex.map(lambda c: _run(c, verbose), jobs_list))
     if force or jobs_list or not KERNELS_SO.exists():
-        _run([hipcc, f"--offload-arch={ARCH}", "-shared", "-fPIC", *map(str, objs), "-o",
-              str(KERNELS_SO), f"-L{tlib}", "-ltorch", "-ltorch_cpu", "-lc10", "-lc10_hip",
-              "-ltorch_hip", "-ltorch_python", "-L/opt/rocm/lib", "-lrccl", f"-Wl,-rpath,{tlib}",
-              "-Wl,-rpath,/opt/rocm/lib"], verbose)
+        with _replacing(KERNELS_SO) as out:
+            _run([hipcc, f"--offload-arch={ARCH}", "-shared", "-fPIC", *map(str, objs), "-o",
+                  str(out), f"-L{tlib}", "-ltorch", "-ltorch_cpu", "-lc10", "-lc10_hip",
+                  "-ltorch_hip", "-ltorch_python", "-L/opt/rocm/lib", "-lrccl", f"-Wl,-rpath,{tlib}",
+                  "-Wl,-rpath,/opt/rocm/lib"], verbose)
     _check_stubs(KERNELS_SO)
     build_runtime(force, verbose)
     return KERNELS_SO
@@ -123,9 +125,32 @@ def build_runtime(force: bool = False, verbose: bool = False) -> Path | None:
     deps = srcs + list(rdir.glob("*.h"))
     if force or _newer(RUNTIME_SO, deps):
         cxx = shutil.which("g++") or "g++"
-        _run([cxx, "-O3", "-std=c++17", "-fPIC", "-shared", "-DMODULE_NAME=_runtime",
-              *[f"-I{p}" for p in _py_includes()], *map(str, srcs), "-o", str(RUNTIME_SO)], verbose)
+        with _replacing(RUNTIME_SO) as out:
+            _run([cxx, "-O3", "-std=c++17", "-fPIC", "-shared", "-DMODULE_NAME=_runtime",
+                  *[f"-I{p}" for p in _py_includes()], *map(str, srcs), "-o", str(out)], verbose)
     return RUNTIME_SO
+
+
+@contextlib.contextmanager
+def _replacing(so: Path):
+    """Link into a temporary name and move it over ``so``: a process that has
+    the old library loaded keeps its mapping."""
+    tmp = so.with_name(f"{so.name}.tmp{os.getpid()}")
+    try:
+        yield tmp
+        os.replace(tmp, so)
+    finally:
+        tmp.unlink(missing_ok=True)
+
+
+def ensure(jobs: int = 8) -> Path:
+    """Build unless both libraries are there and newer than every source (the
+    object files need not be)."""
+    srcs = [*HERE.glob("*.hip"), *HERE.glob("*.h"), HERE / "bindings.cpp"]
+    rt = list((HERE / "runtime").glob("*.cpp"))
+    if _newer(KERNELS_SO, srcs) or _newer(RUNTIME_SO, rt):
+        return build(jobs=jobs)
+    return KERNELS_SO
 
 
 if __name__ == "__main__":

@@ -77,16 +77,13 @@ def main(argv=None) -> int:
     ap.add_argument("--max-tokens", type=int, required=True,
                     help="most tokens live requests hold at a time (the cache pool)")
     a = ap.parse_args(argv)
-    from ..models.registry import load_model
+    from ..models.registry import FLOAT32_FAMILIES, architecture_of, load_model
+    if a.dtype == "float32" and architecture_of(a.model) not in FLOAT32_FAMILIES:
+        print(f"{architecture_of(a.model)} has no 32-bit mode", file=sys.stderr)
+        return 3
     if not torch.cuda.is_available():
         raise RuntimeError("no GPU: the kernels run on gfx950")
-    try:
-        model = load_model(a.model, "cuda:0", dtype=getattr(torch, a.dtype), max_pos=a.max_tokens + 64)
-    except NotImplementedError as e:
-        if a.dtype == "float32":
-            print(e, file=sys.stderr)
-            return 3
-        raise
+    model = load_model(a.model, "cuda:0", dtype=getattr(torch, a.dtype), max_pos=a.max_tokens + 64)
     run = Replay(model, a.max_tokens, model.cfg.vocab_size)
     for line in sys.stdin:
         if not line.strip():

@@ -15,6 +15,7 @@ import torch
 from . import dozazen, llama
 
 _FAMILIES = {"llama": llama.CONFIGS, "dozazen": dozazen.CONFIGS}
+FLOAT32_FAMILIES = ("dozazen",)            # families with a 32-bit mode on the GPU
 
 
 def architecture_of(path) -> str:
@@ -40,7 +41,7 @@ def load_model(path, device, tp_rank: int = 0, tp: int = 1, tp_group=None, dtype
         if tp > 1:
             raise NotImplementedError("dozazen runs on one GPU per replica (tp = 1)")
         return dozazen.load(path, device, dtype=dtype, max_pos=max_pos)
-    if dtype != torch.bfloat16 and torch.device(device).type == "cuda":
+    if dtype != torch.bfloat16 and fam not in FLOAT32_FAMILIES:
         raise NotImplementedError(f"{fam} runs in bfloat16")
     from .weights import llama_from_checkpoint
     return llama_from_checkpoint(path, device, tp_rank, tp, tp_group)

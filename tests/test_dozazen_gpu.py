@@ -34,7 +34,7 @@ def _close(got, want, tol):
 
 # ------------------------------------------------------------------- kernels
 @pytest.mark.parametrize("dtype", [torch.bfloat16, torch.float32])
-@pytest.mark.parametrize("rows,H,Hp", [(1, 100, 128), (3, 192, 192), (700, 200, 256), (1, 4096, 4096),
+@pytest.mark.parametrize("rows,H,Hp", [(1, 100, 128), (3, 320, 320), (700, 200, 256), (1, 4096, 4096),
                                        (5, 5000, 5056), (600, 8192, 8192), (2, 16384, 16384)])
 def test_residual_norm(rows, H, Hp, dtype):
     def padded(t):
@@ -59,15 +59,15 @@ def test_residual_norm(rows, H, Hp, dtype):
 
 @pytest.mark.parametrize("dtype", [torch.bfloat16, torch.float32])
 def test_embedding_scaled(dtype):
-    table = _rnd(50, 192, dtype=dtype)
+    table = _rnd(50, 320, dtype=dtype)
     ids = torch.tensor([3, 49, 0, 3], dtype=torch.int32, device=DEV)
-    lo = torch.zeros(4, 384, device=DEV, dtype=dtype)
-    x = ops.embedding_scaled(ids, table, 12.5, lo[:, 192:])
-    want = table[ids.long()].float() * 12.5
-    assert torch.equal(x, want) and torch.equal(lo[:, 192:], want.to(dtype)) and not lo[:, :192].any()
+    lo = torch.zeros(4, 640, device=DEV, dtype=dtype)
+    x = ops.embedding_scaled(ids, table, 7.5, lo[:, 320:])
+    want = table[ids.long()].float() * 7.5
+    assert torch.equal(x, want) and torch.equal(lo[:, 320:], want.to(dtype)) and not lo[:, :320].any()
 
 
-@pytest.mark.parametrize("M,N,K", [(1, 4, 64), (7, 100, 128), (65, 448, 192), (300, 260, 1024)])
+@pytest.mark.parametrize("M,N,K", [(1, 4, 64), (7, 100, 128), (65, 452, 320), (300, 260, 1024)])
 def test_gemm_f32_is_exact_and_row_independent(M, N, K):
     X, W = _rnd(M, K, seed=1), _rnd(N, K, seed=2)
     got = ops.gemm(X, W)
@@ -76,14 +76,14 @@ def test_gemm_f32_is_exact_and_row_independent(M, N, K):
 
 
 @pytest.mark.parametrize("M", [1, 3, 16, 40, 64, 100, 128, 200, 700, 2600])
-@pytest.mark.parametrize("N,K", [(64, 128), (192, 384), (452, 192), (4096, 8192)])
+@pytest.mark.parametrize("N,K", [(64, 128), (320, 640), (452, 320), (4096, 8192)])
 def test_gemm_f32out(M, N, K):
     X, W = _rnd(M, K, seed=1, dtype=torch.bfloat16), _rnd(N, K, seed=2, dtype=torch.bfloat16)
     _close(ops.gemm_f32out(X, W), X.float() @ W.float().t(), 2e-5)
 
 
 @pytest.mark.parametrize("M", [1, 4, 12, 33, 64, 100, 150, 200, 300, 520, 1100, 2600])
-@pytest.mark.parametrize("F,K", [(64, 64), (320, 192), (14336, 4096)])
+@pytest.mark.parametrize("F,K", [(64, 64), (192, 320), (14336, 4096)])
 def test_gelu_gate_in_every_gemm_path(M, F, K):
     """The tanh form of gelu in the gated GEMM epilogue of every kernel the row
     count can pick; also that silu is what it was."""
@@ -99,7 +99,7 @@ def test_gelu_gate_in_every_gemm_path(M, F, K):
 
 @pytest.mark.parametrize("dtype", [torch.bfloat16, torch.float32])
 @pytest.mark.parametrize("M", [1, 20, 60, 100, 130, 300, 700, 2600])
-@pytest.mark.parametrize("Hq,Hkv,DK,DV,K", [(4, 1, 64, 64, 192), (6, 2, 128, 64, 64), (4, 2, 128, 128, 256),
+@pytest.mark.parametrize("Hq,Hkv,DK,DV,K", [(6, 3, 64, 64, 320), (6, 2, 128, 64, 64), (4, 2, 128, 128, 256),
                                             (32, 8, 128, 128, 4096)])
 def test_qkv_rope_bias(M, Hq, Hkv, DK, DV, K, dtype):
     if dtype == torch.float32 and K == 4096 and M > 300:

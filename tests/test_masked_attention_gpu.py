@@ -64,7 +64,7 @@ MIXED = [(0, 70), (63, 1), (64, 1), (190, 3), (0, 1), (129, 40), (255, 2)]
 
 
 @pytest.mark.parametrize("dtype", [torch.bfloat16, torch.float32])
-@pytest.mark.parametrize("Hq,Hkv,DK,DV", [(4, 1, 64, 64), (8, 2, 128, 128), (6, 2, 128, 64), (5, 5, 64, 128),
+@pytest.mark.parametrize("Hq,Hkv,DK,DV", [(6, 2, 64, 64), (8, 2, 128, 128), (6, 2, 128, 64), (5, 5, 64, 128),
                                           (40, 2, 64, 64), (7, 1, 192, 128), (4, 2, 256, 256), (4, 4, 64, 192)])
 def test_head_shapes(Hq, Hkv, DK, DV, dtype):
     _check(MIXED, Hq, Hkv, DK, DV, 30.0, 50, True, dtype)
@@ -92,7 +92,7 @@ def test_chunk_edges_stand_out(chunk):
         for new in (1, 2, 5, pos + 1):
             if new > pos + 1:
                 continue
-            q, kc, vc, step = _case([(pos + 1 - new, new)], 4, 1, 64, 64, torch.bfloat16, seed=pos)
+            q, kc, vc, step = _case([(pos + 1 - new, new)], 2, 1, 64, 64, torch.bfloat16, seed=pos)
             first = pos // chunk * chunk
             bt = step.block_table[0]
             u = torch.randn(64, generator=torch.Generator().manual_seed(pos))
@@ -110,7 +110,7 @@ def test_chunk_edges_stand_out(chunk):
 
 def test_sink_without_keys_in_reach_of_zero():
     """Scores far below the sink's 0: the sink takes nearly all the weight."""
-    q, kc, vc, step = _case([(30, 2)], 4, 1, 64, 64, torch.bfloat16)
+    q, kc, vc, step = _case([(30, 2)], 2, 1, 64, 64, torch.bfloat16)
     q[:] = 1.0
     kc[:] = torch.where(kc.isnan(), kc, torch.full_like(kc, -1.0))     # score -8 before the cap
     vc[:] = torch.where(vc.isnan(), vc, torch.ones_like(vc))
