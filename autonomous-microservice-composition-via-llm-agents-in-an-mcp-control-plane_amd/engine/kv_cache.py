@@ -13,7 +13,8 @@ A model whose cached layers differ in head count or head size, whose keys and
 values differ, or that runs a layer more than once (each run caches its own keys)
 gives one (kv_heads, key_dim, value_dim) per cached layer instead
 (``KVCache.from_specs``): same blocks and block ids, one stacked tensor per
-distinct (kv_heads, dim).
+distinct (kv_heads, dim).  Latent attention caches one row per token that holds
+both (value_dim 0).
 """
 from __future__ import annotations
 
@@ -94,18 +95,22 @@ class KVCache:
 
     @classmethod
     def from_specs(cls, specs, num_blocks: int, device, dtype=torch.bfloat16) -> "KVCache":
-        """``specs``: (kv_heads, key_dim, value_dim) of every cached layer."""
+        """``specs``: (kv_heads, key_dim, value_dim) of every cached layer; value_dim
+        0: the values are part of the keys, the layer has no value tensor."""
         self = cls.__new__(cls)
         self.layers, self.num_blocks, self.data = len(specs), num_blocks, None
         place, count = [], {}
         for h, dk, dv in specs:
             for d in (dk, dv):
+                if d == 0:
+                    place.append(None)
+                    continue
                 place.append(((h, d), count.get((h, d), 0)))
                 count[(h, d)] = count.get((h, d), 0) + 1
         stack = {(h, d): torch.zeros(n, 1, num_blocks, h, BLOCK_SIZE, d, device=device, dtype=dtype)
                  for (h, d), n in count.items()}
         self.stacks = list(stack.values())
-        at = [stack[k][i, 0] for k, i in place]
+        at = [None if p is None else stack[p[0]][p[1], 0] for p in place]
         self._layer = list(zip(at[0::2], at[1::2]))
         self.allocator = make_allocator(num_blocks)
         return self

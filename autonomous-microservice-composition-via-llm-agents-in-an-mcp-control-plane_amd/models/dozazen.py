@@ -17,7 +17,7 @@ One ragged, paged step (n = rms norm with its own weight, c(z; k) = k tanh(z / k
 What this module adds to the shared machinery is the mapping onto it:
 
 * every size is padded to what the MFMA kernels tile by (width and feed-forward
-  to 64, head sizes to ``HEAD_SIZES``) with zero rows / columns, which is exact;
+  to 64, head sizes to ``packing.HEAD_SIZES``) with zero rows / columns, which is exact;
 * neighbouring-pair rotation becomes the kernels' half rotation by permuting the
   rows of Wq / Wk (the same permutation on both leaves q . k unchanged); pairs
   that do not rotate (partial rotation, padding) hold (1, 0) in the table;
@@ -39,16 +39,8 @@ import torch
 from .. import ops
 from ..ops import reference as ref
 from .llama import padded_group
-
-HEAD_SIZES = (64, 128, 192, 256)
-MAX_POS = 131072          # positions of the rotation tables when nothing else bounds them
-
-
-@dataclasses.dataclass(frozen=True)
-class Rotary:
-    dims: int
-    base: float
-    scaling: Optional[Tuple[float, float, float, float]] = None   # factor, low, high, original
+from .packing import MAX_POS, Rotary, head_size, rope_table
+from .packing import leading as _leading, pad as _pad, pick_rows as _pick_rows, up as _up
 
 
 @dataclasses.dataclass(frozen=True)
@@ -203,16 +195,6 @@ class DozazenWeights:
     lm_head: torch.Tensor                  # [V padded to 4, Wp]
 
 
-def _up(n: int, m: int) -> int:
-    return -(-n // m) * m
-
-
-def head_size(d: int) -> int:
-    """The head size ``d`` runs at: the next of ``HEAD_SIZES`` (larger heads,
-    outside the MFMA forms, at the next multiple of 64)."""
-    return next((h for h in HEAD_SIZES if h >= d), _up(d, 64))
-
-
 def half_rotation_order(dim: int, rot_dims: int, padded: int) -> torch.Tensor:
     """Row of the checkpoint's head that goes to each row of the padded head
     (-1: a zero row): pair (2i, 2i + 1) to (i, i + padded / 2), the dimensions
@@ -224,21 +206,6 @@ def half_rotation_order(dim: int, rot_dims: int, padded: int) -> torch.Tensor:
     free = (at < 0).nonzero().flatten()
     at[free[:dim - rot_dims]] = torch.arange(rot_dims, dim)
     return at
-
-
-def _pick_rows(w: torch.Tensor, heads: int, dim: int, order: torch.Tensor) -> torch.Tensor:
-    """[heads * dim, ...] -> [heads * len(order), ...] rows by ``order`` per head."""
-    w = w.reshape(heads, dim, *w.shape[1:])
-    out = w.new_zeros(heads, len(order), *w.shape[2:])
-    on = order >= 0
-    out[:, on] = w[:, order[on]]
-    return out.reshape(heads * len(order), *w.shape[2:])
-
-
-def _pad(w: torch.Tensor, *shape: int) -> torch.Tensor:
-    out = w.new_zeros(*shape)
-    out[tuple(slice(0, n) for n in w.shape)] = w
-    return out
 
 
 def pack_weights(cfg: DozazenConfig, get, device, dtype=torch.bfloat16) -> DozazenWeights:
@@ -257,8 +224,7 @@ def pack_weights(cfg: DozazenConfig, get, device, dtype=torch.bfloat16) -> Dozaz
         m, p = s.mixer, f"l{i}."
         DK, DV = head_size(m.dim), head_size(m.vdim)
         qk = half_rotation_order(m.dim, m.rot.dims, DK)
-        vo = torch.full((DV,), -1, dtype=torch.long)
-        vo[:m.vdim] = torch.arange(m.vdim)
+        vo = _leading(m.vdim, DV)
         parts = ((m.heads, m.dim, qk, "q"), (m.kv_heads, m.dim, qk, "k"), (m.kv_heads, m.vdim, vo, "v"))
         wqkv = torch.cat([_pick_rows(get(f"{p}mix.{n}"), h, d, o) for h, d, o, n in parts])
         bqkv = torch.cat([_pick_rows(get(f"{p}mix.{n}.b").float(), h, d, o) for h, d, o, n in parts])
@@ -344,11 +310,7 @@ class DozazenModel:
         self.logit_scale, self.logit_cap = cfg.logit_scale, cfg.logit_cap
 
     def _table(self, rot: Rotary, padded: int) -> torch.Tensor:
-        cs = torch.zeros(self.cfg.max_pos, padded // 2, 2)
-        cs[..., 0] = 1.0
-        if rot.dims:
-            cs[:, :rot.dims // 2] = ref.rope_cos_sin(self.cfg.max_pos, rot.dims, rot.base, None, rot.scaling)
-        return cs.to(self.device)
+        return rope_table(rot, self.cfg.max_pos, padded // 2, self.device)
 
     @classmethod
     def random(cls, name, device, seed: int = 0, dtype=torch.bfloat16):
@@ -431,9 +393,5 @@ def load(path, device, dtype=torch.bfloat16, max_pos: Optional[int] = None) -> D
 
 def save(cfg: DozazenConfig, get, path) -> None:
     """Checkpoint directory from tensors in the checkpoint layout (``get(name)``)."""
-    from safetensors.torch import save_file
-    path = Path(path)
-    path.mkdir(parents=True, exist_ok=True)
-    save_file({n: get(n).to(torch.bfloat16).cpu().contiguous() for n in tensor_shapes(cfg)},
-              str(path / "model.safetensors"))
-    (path / "config.json").write_text(json.dumps(config_to_json(cfg), indent=1))
+    from .weights import save_tensors
+    save_tensors(path, tensor_shapes(cfg), get, config_to_json(cfg))

@@ -12,10 +12,12 @@ from typing import Optional
 
 import torch
 
-from . import dozazen, llama
+from . import dozazen, llama, topelorn
 
-_FAMILIES = {"llama": llama.CONFIGS, "dozazen": dozazen.CONFIGS}
-FLOAT32_FAMILIES = ("dozazen",)            # families with a 32-bit mode on the GPU
+_FAMILIES = {"llama": llama.CONFIGS, "dozazen": dozazen.CONFIGS, "topelorn": topelorn.CONFIGS}
+# families on one GPU per replica, with a 32-bit mode on the GPU
+_ONE_GPU = {"dozazen": (dozazen.load, dozazen.DozazenModel), "topelorn": (topelorn.load, topelorn.TopelornModel)}
+FLOAT32_FAMILIES = tuple(_ONE_GPU)
 
 
 def architecture_of(path) -> str:
@@ -37,10 +39,10 @@ def load_model(path, device, tp_rank: int = 0, tp: int = 1, tp_group=None, dtype
     """The model over a checkpoint directory.  ``dtype`` float32 needs a family
     with a 32-bit mode; ``max_pos`` bounds the position tables."""
     fam = architecture_of(path)
-    if fam == "dozazen":
+    if fam in _ONE_GPU:
         if tp > 1:
-            raise NotImplementedError("dozazen runs on one GPU per replica (tp = 1)")
-        return dozazen.load(path, device, dtype=dtype, max_pos=max_pos)
+            raise NotImplementedError(f"{fam} runs on one GPU per replica (tp = 1)")
+        return _ONE_GPU[fam][0](path, device, dtype=dtype, max_pos=max_pos)
     if dtype != torch.bfloat16 and fam not in FLOAT32_FAMILIES:
         raise NotImplementedError(f"{fam} runs in bfloat16")
     from .weights import llama_from_checkpoint
@@ -57,7 +59,8 @@ def get_config(name: str):
 
 def random_model(name: str, device, seed: int = 0):
     """A named configuration with random-init weights, one GPU."""
-    if name in dozazen.CONFIGS:
-        return dozazen.DozazenModel.random(name, device, seed=seed)
+    for fam, (_, model) in _ONE_GPU.items():
+        if name in _FAMILIES[fam]:
+            return model.random(name, device, seed=seed)
     get_config(name)
     return llama.LlamaModel.random(name, device, seed=seed)

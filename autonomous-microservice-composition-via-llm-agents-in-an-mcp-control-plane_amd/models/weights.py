@@ -195,6 +195,15 @@ def save_llama_safetensors(cfg: LlamaConfig, w: LlamaWeights, path, shard_layers
            if cfg.rope_scaling else {})}, indent=1))
 
 
+def save_tensors(path, names, get, config: dict) -> None:
+    """Checkpoint directory of the tensors ``get(name)`` (bf16) and ``config``."""
+    from safetensors.torch import save_file
+    path = Path(path)
+    path.mkdir(parents=True, exist_ok=True)
+    save_file({n: get(n).to(torch.bfloat16).cpu().contiguous() for n in names}, str(path / "model.safetensors"))
+    (path / "config.json").write_text(json.dumps(config, indent=1))
+
+
 def llama_from_checkpoint(path, device, tp_rank: int = 0, tp: int = 1, tp_group=None):
     """LlamaModel over an HF safetensors checkpoint directory."""
     from .llama import LlamaModel

@@ -173,10 +173,10 @@ def gemm(X, W, R=None, out=None, algo: int = -1, ss_out=None):
         if _TRACE is not None:
             _trace(X, W, "gemm" if R is None else "gemm+res")
         out = X.new_empty(*X.shape[:-1], W.shape[0]) if out is None else out
-        if X.dtype == torch.float32:              # the 32-bit mode: plain products only
-            if R is not None or ss_out is not None:
-                raise NotImplementedError("float32 gemm: no residual epilogue")
-            lib().gemm_f32(X, W, out)
+        if X.dtype == torch.float32:              # the 32-bit mode
+            if ss_out is not None:
+                raise NotImplementedError("float32 gemm: no norm statistics")
+            lib().gemm_f32(X, W, out, R)
         else:
             lib().gemm(X, W, out, R, algo, ss_out)
         return out
@@ -211,14 +211,17 @@ def embedding_scaled(ids, table, scale: float, lo=None):
     return x
 
 
-def residual_norm(x, H: int, eps: float, y=None, w_post=None, w_pre=None, out=None):
+def residual_norm(x, H: int, eps: float, y=None, w_post=None, w_pre=None, out=None,
+                  center: bool = False):
     """One pass over the fp32 residual ``x`` [T, Hp] (in place; means over the
-    first ``H`` columns, the rest are zero): x += rms(y) * w_post when ``y`` is
-    given, then ``out`` = rms(x) * w_pre, or x itself without ``w_pre``."""
+    first ``H`` columns, the rest are zero): x += rms(y) * w_post (y as it is
+    without ``w_post``) when ``y`` is given, then ``out`` = rms(x) * w_pre, or x
+    itself without ``w_pre``.  ``center``: the second norm is a layer norm (the
+    mean is taken off first)."""
     if x.is_cuda:
-        lib().residual_norm(x, y, w_post, w_pre, out, int(H), float(eps))
+        lib().residual_norm(x, y, w_post, w_pre, out, int(H), float(eps), bool(center))
         return out
-    return ref.residual_norm(x, H, eps, y, w_post, w_pre, out)
+    return ref.residual_norm(x, H, eps, y, w_post, w_pre, out, center)
 
 
 def logit_finish(z, scale: float = 1.0, cap: float = 0.0):
@@ -594,38 +597,95 @@ def paged_attention(q, k_cache, v_cache, meta, scale, out=None):
     return r if out is None else out.copy_(r)
 
 
+def qk_norm_kv(z, slots, wq, wk, dim: int, eps: float, q_out, k_cache, v_cache, v_first=None,
+               lam: float = 0.0):
+    """q_out, K/V cache <- the projected rows ``z`` [T, >= (Hq + Hkv) DK + Hkv DV]:
+    an RMS norm of every q and k head (mean over the first ``dim`` elements,
+    weights fp32 [DK]) and v, or (1 - lam) v + lam v_first with ``v_first``
+    [T, Hkv DV] (a row-strided view is fine).  Columns after v are not read."""
+    if z.is_cuda:
+        lib().qk_norm_kv(z, slots, wq, wk, int(dim), float(eps), q_out, k_cache, v_cache, v_first,
+                         float(lam))
+    else:
+        ref.qk_norm_kv(z, slots, wq, wk, dim, eps, q_out, k_cache, v_cache, v_first, lam)
+    return q_out
+
+
+def latent_qkv(z, pos, slots, cos_sin, w_c, eps: float, heads: int, dim: int, rot: int, rank: int,
+               rank_true: int, q_out, k_cache):
+    """Latent attention's rows around the absorbed query: ``z`` [T, >= heads
+    (dim + rot) + rank + rot] holds per head [unrotated | rotated], then the
+    latent and the shared rotated key.  Writes the key row [rms(latent) * w_c |
+    rotated key | 0] to the cache and [rotated query | 0] to q_out[..., rank:];
+    q_out[..., :rank] is ``gemm_heads``'s.  cos_sin [P, n, 2] rotates the first
+    2 n of the ``rot`` elements as halves."""
+    if z.is_cuda:
+        lib().latent_qkv(z, pos, slots, cos_sin, w_c, float(eps), int(heads), int(dim), int(rot),
+                         int(rank), int(rank_true), q_out, k_cache)
+    else:
+        ref.latent_qkv(z, pos, slots, cos_sin, w_c, eps, heads, dim, rot, rank, rank_true, q_out, k_cache)
+    return q_out
+
+
+def gemm_heads(X, W, out):
+    """One product per head: out[t, h] = X[t, h] @ W[h]^T, X [T, H, K] and out
+    [T, H, N] strided views (inner stride 1), W [H, N, K].  K % 32 == 0, N % 16 == 0."""
+    if X.is_cuda:
+        lib().gemm_heads(X, W, out)
+        return out
+    return ref.gemm_heads(X, W, out)
+
+
 MASKED_MAX_HEAD = 256           # largest head of the MFMA forms (csrc/attention_masked.hip)
+# (key, value) sizes of the MFMA form whose values are the first columns of the
+# keys (csrc/attention_latent.hip)
+LATENT_SIZES = ((64, 64), (128, 64), (128, 128), (192, 128), (192, 192), (256, 192), (256, 256),
+                (320, 256), (448, 384), (576, 512))
 
 
 def masked_attention(q, k_cache, v_cache, meta, scale, group: int, soft_cap: float = 0.0,
-                     chunk: int = 0, sink: bool = False):
-    """Paged causal attention, q [T, Hq, DK] -> [T, Hq, DV], with the score
-    soft cap (s <- cap tanh(s / cap); 0 = none), the chunked mask (keys of the
-    query's own ``chunk``-token stretch of the sequence; 0 = all earlier keys)
-    and the softmax sink (one added to the denominator).  ``group``: the GQA
-    group the step's work lists were cut for (16 / group tokens per 1-wave
-    item); the heads' own group may be another."""
+                     chunk: int = 0, sink=False, window: int = 0, keep_first: int = 0, slopes=None,
+                     gate=None, v_dim: Optional[int] = None, max_splits: int = 1 << 30):
+    """Paged causal attention, q [T, Hq, DK] -> [T, Hq, DV].
+
+    ``soft_cap``: s <- cap tanh(s / cap); 0 = none.  ``chunk``: only keys of the
+    query's own ``chunk``-token stretch of the sequence; 0 = all earlier keys.
+    ``window``: only the last ``window`` keys, the query's own included, and the
+    first ``keep_first`` of the sequence; 0 = all.  ``slopes`` (fp32 [Hq]): s -=
+    slope * distance (not with a cap or chunk).  ``sink``: True adds one to the
+    softmax denominator, fp32 [Hq] adds exp(sink).  ``gate`` ([T, Hq], row-strided
+    view of q's type): the output times sigmoid(gate).  ``v_cache`` None: the
+    values are the first ``v_dim`` columns of the keys (latent attention).
+    ``group``: the GQA group the step's work lists were cut for (16 / group
+    tokens per 1-wave item); the heads' own group may be another.
+    ``max_splits`` bounds the scheduler's key splits for this layer."""
     if q.is_cuda:
-        out = torch.empty(q.shape[0], q.shape[1], v_cache.shape[3], device=q.device, dtype=q.dtype)
+        shared = v_cache is None
+        DV = v_dim if shared else v_cache.shape[3]
+        out = torch.empty(q.shape[0], q.shape[1], DV, device=q.device, dtype=q.dtype)
         L = lib()
+        sinks = sink if isinstance(sink, torch.Tensor) else None
         a = (q, k_cache, v_cache, out, meta.q_start, meta.q_len, meta.ctx_len, meta.block_table)
-        k = (float(scale), float(soft_cap), int(chunk), bool(sink))
-        if q.dtype == torch.bfloat16 and max(q.shape[2], v_cache.shape[3]) <= MASKED_MAX_HEAD:
+        k = (float(scale), float(soft_cap), int(chunk), sinks is not None or bool(sink), int(window),
+             int(keep_first), slopes, sinks, gate)
+        if q.dtype == torch.bfloat16 and ((q.shape[2], DV) in LATENT_SIZES if shared else
+                                          max(q.shape[2], DV) <= MASKED_MAX_HEAD):
             for nw, ws, wq in meta.work_lists():
                 nz, so, sm = 1, None, None
                 if nw == 1 and int(meta.kv_splits) > 1:
                     # (the partials are addressed with 31 bits)
-                    nz = max(1, min(int(meta.kv_splits), (1 << 31) // max(1, 4 * out.numel()) - 1))
+                    nz = max(1, min(int(meta.kv_splits), max_splits, (1 << 31) // max(1, 4 * out.numel()) - 1))
                 if nz > 1:
                     so = torch.empty(nz, *out.shape, device=q.device, dtype=torch.float32)
                     sm = torch.empty(nz, q.shape[0], q.shape[1], 2, device=q.device, dtype=torch.float32)
                 if not L.attention_masked(*a, ws, wq, nw, nw * (16 // group), *k, nz, so, sm):
-                    raise ValueError(f"masked attention: head sizes {q.shape[2]} / {v_cache.shape[3]}")
+                    raise ValueError(f"masked attention: head sizes {q.shape[2]} / {DV}")
             return out
         L.attention_row(*a, *k)
         return out
     return ref.masked_attention(q, k_cache, v_cache, meta.q_start, meta.q_len, meta.ctx_len,
-                                meta.block_table, scale, soft_cap, chunk, sink)
+                                meta.block_table, scale, soft_cap, chunk, sink, window, keep_first, slopes,
+                                gate, v_dim)
 
 
 def sample_dense(logits, allow_ptr, allow_ids, ctr, temperature, seed):

@@ -163,14 +163,16 @@ def soft_cap(z, cap: float):
     return cap * torch.tanh(z / cap) if cap > 0 else z
 
 
-def residual_norm(x, H, eps, y=None, w_post=None, w_pre=None, out=None):
-    def norm(v, w):
+def residual_norm(x, H, eps, y=None, w_post=None, w_pre=None, out=None, center=False):
+    def norm(v, w, center):
         v = v.float()
+        if center:
+            v = v - v[:, :H].mean(-1, keepdim=True)
         return v / torch.sqrt((v[:, :H] ** 2).mean(-1, keepdim=True) + eps) * w
     if y is not None:
-        x += norm(y, w_post)
+        x += y.float() if w_post is None else norm(y, w_post, False)
     if out is not None:
-        out.copy_(x if w_pre is None else norm(x, w_pre))
+        out.copy_(x if w_pre is None else norm(x, w_pre, center))
     return out
 
 
@@ -189,10 +191,70 @@ def rope_kv_any(qkv, pos, slots, cos_sin, q_out, k_cache, v_cache):
     v_cache[b, :, o] = v[on]
 
 
-def masked_attention(q, k_cache, v_cache, q_start, q_len, ctx_len, block_table, scale,
-                     cap=0.0, chunk=0, sink=False):
-    T, Hq, DK = q.shape
+def _cache_rows(slots, block: int):
+    """(tokens with a slot, their blocks, their places in the block)."""
+    on = slots >= 0
+    return on, (slots[on] // block).long(), (slots[on] % block).long()
+
+
+def head_rms(x, w, dim, eps):
+    """RMS norm of the first ``dim`` elements of every head, x [T, H, D]."""
+    x = x.float()
+    return x / torch.sqrt((x[..., :dim] ** 2).mean(-1, keepdim=True) + eps) * w
+
+
+def qk_norm_kv(z, slots, wq, wk, dim, eps, q_out, k_cache, v_cache, v_first=None, lam=0.0):
+    T, Hq, DK = q_out.shape
     Hkv, BS, DV = k_cache.shape[1], k_cache.shape[2], v_cache.shape[3]
+    q, k, v, _ = torch.split(z, [Hq * DK, Hkv * DK, Hkv * DV, z.shape[1] - (Hq + Hkv) * DK - Hkv * DV], dim=-1)
+    q_out.copy_(head_rms(q.reshape(T, Hq, DK), wq, dim, eps))
+    k = head_rms(k.reshape(T, Hkv, DK), wk, dim, eps)
+    v = v.float()
+    if v_first is not None:
+        v = (1 - lam) * v + lam * v_first.float()
+    on, b, o = _cache_rows(slots, BS)
+    k_cache[b, :, o] = k[on].to(k_cache.dtype)
+    v_cache[b, :, o] = v.reshape(T, Hkv, DV)[on].to(v_cache.dtype)
+
+
+def _rotate_halves(x, cs):
+    """x [T, ..., R]; dimension i turns with i + n for the table's n pairs."""
+    n = cs.shape[1]
+    cs = cs.view(cs.shape[0], *([1] * (x.dim() - 2)), n, 2)
+    u, v, rest = x[..., :n], x[..., n:2 * n], x[..., 2 * n:]
+    c, s = cs[..., 0], cs[..., 1]
+    return torch.cat([u * c - v * s, v * c + u * s, rest], -1)
+
+
+def latent_qkv(z, pos, slots, cos_sin, w_c, eps, heads, dim, rot, rank, rank_true, q_out, k_cache):
+    T, _, DK = q_out.shape
+    cs = cos_sin[pos.long()]
+    pre = heads * (dim + rot)
+    q = z[:, :pre].float().view(T, heads, dim + rot)
+    q_out[..., rank:] = 0
+    q_out[..., rank:rank + rot] = _rotate_halves(q[..., dim:], cs).to(q_out.dtype)
+    row = torch.zeros(T, DK)
+    row[:, :rank] = head_rms(z[:, pre:pre + rank], w_c, rank_true, eps)
+    row[:, rank:rank + rot] = _rotate_halves(z[:, pre + rank:pre + rank + rot].float(), cs)
+    on, b, o = _cache_rows(slots, k_cache.shape[2])
+    k_cache[b, 0, o] = row[on].to(k_cache.dtype)
+
+
+def gemm_heads(X, W, out):
+    return out.copy_(torch.einsum("thk,hnk->thn", X.float(), W.float()))
+
+
+def masked_attention(q, k_cache, v_cache, q_start, q_len, ctx_len, block_table, scale,
+                     cap=0.0, chunk=0, sink=False, window=0, keep_first=0, slopes=None, gate=None,
+                     v_dim=None):
+    """``sink``: a bool (a key of score 0), or [Hq] scores."""
+    T, Hq, DK = q.shape
+    Hkv, BS = k_cache.shape[1], k_cache.shape[2]
+    if v_cache is None:
+        v_cache = k_cache[..., :v_dim]
+    DV = v_cache.shape[3]
+    if isinstance(sink, bool):
+        sink = torch.zeros(Hq) if sink else None
     out = q.new_zeros(T, Hq, DV)
     for s in range(q_start.numel()):
         qs, ql, cl = int(q_start[s]), int(q_len[s]), int(ctx_len[s])
@@ -205,16 +267,25 @@ def masked_attention(q, k_cache, v_cache, q_start, q_len, ctx_len, block_table, 
         S = soft_cap(Q @ K.unsqueeze(1).transpose(2, 3) * scale, cap)
         i = torch.arange(cl - ql, cl).unsqueeze(1)
         j = torch.arange(cl).unsqueeze(0)
+        if slopes is not None:
+            S = S - slopes.view(Hkv, Hq // Hkv, 1, 1) * (i - j)
         ok = j <= i
         if chunk:
             ok = ok & (j // chunk == i // chunk)
+        if window:
+            ok = ok & ((i - j < window) | (j < keep_first))
         S = S.masked_fill(~ok, float("-inf"))
         m = S.amax(-1, keepdim=True)
-        if sink:
-            m = m.clamp(min=0)
+        if sink is not None:
+            sk = sink.view(Hkv, Hq // Hkv, 1, 1).expand_as(m)
+            m = torch.maximum(m, sk)
         P = torch.exp(S - m)
-        den = P.sum(-1, keepdim=True) + (torch.exp(-m) if sink else 0)
+        den = P.sum(-1, keepdim=True)
+        if sink is not None:
+            den = den + torch.exp(sk - m)
         out[qs:qs + ql] = (P / den @ V.unsqueeze(1)).permute(2, 0, 1, 3).reshape(ql, Hq, DV).to(q.dtype)
+    if gate is not None:
+        out.copy_(out * torch.sigmoid(gate.float()).unsqueeze(-1))
     return out
 
 
