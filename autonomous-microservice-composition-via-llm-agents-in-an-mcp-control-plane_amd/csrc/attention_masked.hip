@@ -1,8 +1,11 @@
 // Paged attention with a mask and a softmax of a model's own choosing: logit
 // soft-capping (s <- cap tanh(s / cap)), chunked causal masks (a query sees the
-// keys of its own chunk of the sequence only), a sink of score 0 in the softmax
-// denominator, key and value heads of different sizes, any GQA group.  The
-// plain causal softmax kernels for d = 128 are in attention.hip.
+// keys of its own chunk of the sequence only), sliding windows that keep the
+// first keys, scores that fall with the distance, a sink in the softmax
+// denominator (of score 0 or learned), a gate on every head's output, key and
+// value heads of different sizes, any GQA group.  The plain causal softmax
+// kernels for d = 128 are in attention.hip, values that are part of the keys in
+// attention_latent.hip.
 //
 // Layouts: q [T, Hq, DK], k cache [num_blocks, Hkv, 64, DK], v cache
 // [num_blocks, Hkv, 64, DV], out [T, Hq, DV].
@@ -20,130 +23,19 @@
 // query row), then O^T += V^T P^T with P^T straight from the S^T accumulators and
 // V^T from transposed LDS reads, as attention.hip does.
 //
-// Softmax.  The sink is a key of score 0 without a value: a running sum that
-// starts at m = 0, l = 1.  A soft cap bounds every score by +-cap, so while
+// Softmax.  The sink is a key of fixed score without a value: a running sum that
+// starts at m = its score, l = 1.  A soft cap bounds every score by +-cap, so while
 // e^cap is far inside fp32 (cap <= NOMAX_CAP) the weights e^s need no running
 // maximum at all: no row reductions and no rescaling inside the key loop, and
 // partial sums over keys (waves, splits) simply add.
-#include "common.h"
-#include "kernels.h"
+#include "attention_masked.h"
 
 namespace {
-
-constexpr int KT = 64;                        // keys per cache block
-
-typedef __attribute__((ext_vector_type(4))) short s16x4;
-constexpr float LOG2E = 1.4426950408889634f;
-constexpr float NOMAX_CAP = 60.f;             // e^60 x 1e6 keys is far below fp32's range
-
-enum { PLAIN = 0, CAPPED = 1, CAPPED_NOMAX = 2 };   // score forms
-
-DEV bf16x4 tr_read(const bf16* p) {
-  s16x4 v = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) s16x4*)(p));
-  return __builtin_bit_cast(bf16x4, v);
-}
-
-// Score constants (log2 units): PLAIN s = acc a; CAPPED s = C tanh(acc scale / cap)
-// = C - 2 C / (1 + 2^(acc a)), a = 2 log2(e) scale / cap, C = cap log2(e)
-struct ScoreConst {
-  float a, c;
-};
-template <int MODE>
-DEV ScoreConst score_const(const MaskedAttnArgs& p) {
-  if constexpr (MODE == PLAIN) return {p.scale * LOG2E, 0.f};
-  return {2.f * LOG2E * p.scale / p.cap, p.cap * LOG2E};
-}
-template <int MODE>
-DEV float score(float acc, const ScoreConst& k) {
-  if constexpr (MODE == PLAIN) return acc * k.a;
-  return fmaf(-2.f * k.c, __builtin_amdgcn_rcpf(1.f + fexp2(acc * k.a)), k.c);
-}
-
-// running softmax state of one query row (the lane's)
-struct Run {
-  float m, l;                                 // maximum (log2 units; 0 in CAPPED_NOMAX), this lane's sum
-};
-
-// One 64-key tile of the lane's row (keys 16 nt + 4 fq + r): scores -> weights
-// (bf16 MFMA fragments, key order as in the accumulators).  MASKED: keys outside
-// [lo, hi] (tile-relative) drop out.  Returns the factor O is to be rescaled by.
-template <int MODE, bool MASKED>
-DEV float tile_weights(f32x4 (&sacc)[4], bf16x8 (&pf)[2], Run& st, const ScoreConst& k, int lo, int hi,
-                       int fq) {
-  float alpha = 1.f;
-  float tmax = -INFINITY;
-#pragma unroll
-  for (int nt = 0; nt < 4; ++nt)
-#pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      float v = score<MODE>(sacc[nt][r], k);
-      if constexpr (MASKED) {
-        const int key = nt * 16 + fq * 4 + r;
-        v = (key >= lo && key <= hi) ? v : -INFINITY;
-      }
-      sacc[nt][r] = v;
-      if constexpr (MODE != CAPPED_NOMAX) tmax = fmaxf(tmax, v);
-    }
-  float mu = 0.f;
-  if constexpr (MODE != CAPPED_NOMAX) {
-    tmax = fmaxf(tmax, __shfl_xor(tmax, 16, 64));
-    tmax = fmaxf(tmax, __shfl_xor(tmax, 32, 64));
-    const float m_new = fmaxf(st.m, tmax);
-    mu = m_new == -INFINITY ? 0.f : m_new;    // every key masked so far
-    alpha = fexp2(st.m - mu);
-    st.m = m_new;
-  }
-  float sum = 0.f;
-#pragma unroll
-  for (int nt = 0; nt < 4; ++nt)
-#pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const float p = fexp2(sacc[nt][r] - mu);
-      sum += p;
-      pf[nt >> 1][(nt & 1) * 4 + r] = (bf16)p;
-    }
-  st.l = st.l * alpha + sum;
-  return alpha;
-}
-
-// O^T += V^T P^T over one tile; Vl: [64][DV] with 16-B chunk swizzle ^= row & 7
-template <int DV>
-DEV void tile_pv(const bf16* Vl, const bf16x8 (&pf)[2], f32x4 (&o)[DV / 16], int lane) {
-  const int fq = lane >> 4, tq = (lane & 15) >> 2, tp = lane & 3;
-#pragma unroll
-  for (int dt = 0; dt < DV / 16; ++dt) {
-    const int chunk = dt * 2 + (tp >> 1), half = (tp & 1) * 4;
-#pragma unroll
-    for (int k2 = 0; k2 < 2; ++k2) {
-      const int key0 = k2 * 32 + fq * 4 + tq;
-      const int key1 = key0 + 16;
-      const bf16x4 v0 = tr_read(Vl + key0 * DV + ((chunk ^ (key0 & 7)) << 3) + half);
-      const bf16x4 v1 = tr_read(Vl + key1 * DV + ((chunk ^ (key1 & 7)) << 3) + half);
-      const bf16x8 vf = bf16x8{v0[0], v0[1], v0[2], v0[3], v1[0], v1[1], v1[2], v1[3]};
-      o[dt] = mfma16x16x32(vf, pf[k2], o[dt]);
-    }
-  }
-}
-
-// LDS-DMA of pieces [p0, p1) (1 KiB each) of a [64][D] block, swizzled
-template <int D, int P0, int P1>
-DEV void stage_rows(const bf16* src, bf16* dst, int first, int lane) {
-  constexpr int NC = D / 8;                   // 16-B chunks per row
-#pragma unroll
-  for (int i = P0; i < P1; ++i) {
-    const int p = first + i;
-    const int c = p * 64 + lane;
-    const int row = c / NC, chunk = c % NC;
-    glds16(src + row * D + ((chunk ^ (row & 7)) << 3), dst + p * 512);
-  }
-}
-
-DEV int chunk_start(int pos, int chunk) { return chunk > 0 ? pos / chunk * chunk : 0; }
 
 // ---- row form: one wave per (token, query head).  Lanes take keys for the
 // scores and value columns for the sum; everything is fp32.  The 32-bit mode
 // runs on it, and head sizes the MFMA forms do not cover.
-constexpr int ROW_MAX_DV = 512;
+constexpr int ROW_MAX_DV = 1024;
 
 template <class T>
 __global__ __launch_bounds__(64) void attn_row_kernel(const MaskedAttnArgs a) {
@@ -167,24 +59,30 @@ __global__ __launch_bounds__(64) void attn_row_kernel(const MaskedAttnArgs a) {
   for (int d = lane; d < a.DK; d += 64) qs[d] = (float)qp[d];
   __syncthreads();
   const int qpos = a.ctx_len[s] - a.q_len[s] + (t - a.q_start[s]);
-  const int first = chunk_start(qpos, a.chunk);
+  const int first = first_key(a, qpos);
   const int* bt = a.block_table + (size_t)s * a.max_blocks;
-  float m_run = a.sink ? 0.f : -INFINITY, l = a.sink ? 1.f : 0.f;
+  const float slope = a.slopes ? a.slopes[head] : 0.f;
+  const T* vc = a.vc ? (const T*)a.vc : (const T*)a.kc;   // (values inside the keys)
+  const int ldv = a.vc ? a.DV : a.DK;
+  float m_run = !a.sink ? -INFINITY : a.sinks ? a.sinks[head] : 0.f, l = a.sink ? 1.f : 0.f;
   float o[ROW_MAX_DV / 64];
 #pragma unroll
   for (int i = 0; i < ROW_MAX_DV / 64; ++i) o[i] = 0.f;
-  for (int kt = first / KT; kt <= qpos / KT; ++kt) {
+  const TileWalk walk(a, first, qpos);
+  for (int i = 0; i < walk.n; ++i) {
+    const int kt = walk.tile(i);
     const size_t blk = (size_t)bt[kt] * a.Hkv + kvh;
     const T* kr = (const T*)a.kc + (blk * KT + lane) * a.DK;
     const int key = kt * KT + lane;
-    const bool on = key >= first && key <= qpos;
+    const bool on = key <= qpos && (key >= first || key < a.keep);
     float sc = 0.f;
     if (on) {
       for (int d = 0; d < a.DK; ++d) sc = fmaf(qs[d], (float)kr[d], sc);
       sc *= a.scale;
       if (a.cap > 0.f) sc = a.cap * tanhf(sc / a.cap);
+      sc -= slope * (float)(qpos - key);
     }
-    const float mt = wave_max(on ? sc : -INFINITY);
+    const float mt = wave_max(on ? sc : -INFINITY);     // (every tile of the walk has a visible key)
     const float m_new = fmaxf(m_run, mt);
     const float alpha = expf(m_run - m_new);
     const float p = on ? expf(sc - m_new) : 0.f;
@@ -193,19 +91,19 @@ __global__ __launch_bounds__(64) void attn_row_kernel(const MaskedAttnArgs a) {
     __syncthreads();
     ps[lane] = p;
     __syncthreads();
-    const int k0 = max(first - kt * KT, 0), k1 = min(qpos - kt * KT, KT - 1);
+    const int k0 = kt * KT < a.keep ? 0 : max(first - kt * KT, 0), k1 = min(qpos - kt * KT, KT - 1);
 #pragma unroll
     for (int i = 0; i < ROW_MAX_DV / 64; ++i) {
       const int d = i * 64 + lane;
       if (d < a.DV) {
         float acc = o[i] * alpha;
-        const T* vr = (const T*)a.vc + blk * KT * a.DV + d;
-        for (int k = k0; k <= k1; ++k) acc = fmaf(ps[k], (float)vr[(size_t)k * a.DV], acc);
+        const T* vr = vc + blk * KT * ldv + d;
+        for (int k = k0; k <= k1; ++k) acc = fmaf(ps[k], (float)vr[(size_t)k * ldv], acc);
         o[i] = acc;
       }
     }
   }
-  const float inv = 1.f / l;
+  const float inv = head_gate<T>(a, t, head) / l;
   T* op = (T*)a.out + ((size_t)t * a.Hq + head) * a.DV;
 #pragma unroll
   for (int i = 0; i < ROW_MAX_DV / 64; ++i) {
@@ -237,12 +135,12 @@ void attn_tile_kernel(const MaskedAttnArgs a) {
   const int tok = q0 + rr / G, head = kvh * G + rr % G;
   const int base = cl - ql;                              // position of the span's first token
   const int qpos = base + tok;
-  const int first = chunk_start(qpos, a.chunk);          // first key of this lane's row
+  const int first = first_key(a, qpos);          // first key of this lane's row
   // key tiles of the block, and of this wave's rows
-  const int b_lo = chunk_start(base + q0 + row0 / G, a.chunk), b_hi = base + q0 + (row0 + rows - 1) / G;
+  const int b_lo = first_key(a, base + q0 + row0 / G), b_hi = base + q0 + (row0 + rows - 1) / G;
   const int w0 = min(row0 + wave * 16, row0 + rows - 1), w1 = min(row0 + wave * 16 + 15, row0 + rows - 1);
   const int wp0 = base + q0 + w0 / G, wp1 = base + q0 + w1 / G;   // the wave's positions
-  const int w_lo = chunk_start(wp0, a.chunk), w_in = chunk_start(wp1, a.chunk);
+  const int w_lo = first_key(a, wp0), w_in = first_key(a, wp1);
   const bool w_on = wave * 16 < rows;
 
   bf16x8 qf[DK / 32];
@@ -251,25 +149,21 @@ void attn_tile_kernel(const MaskedAttnArgs a) {
 #pragma unroll
     for (int ks = 0; ks < DK / 32; ++ks) qf[ks] = *reinterpret_cast<const bf16x8*>(qp + 32 * ks);
   }
-  const ScoreConst kc = score_const<MODE>(a);
-  Run st;
-  st.m = MODE == CAPPED_NOMAX || a.sink ? 0.f : -INFINITY;
-  st.l = a.sink && fq == 0 ? 1.f : 0.f;
+  const ScoreConst kc = score_const<MODE>(a, head);
+  Run st = run_start<MODE>(a, head, a.sink, fq);
   f32x4 o[DV / 16];
 #pragma unroll
   for (int i = 0; i < DV / 16; ++i) o[i] = f32x4{0.f, 0.f, 0.f, 0.f};
 
   bf16* Kl = smem;
   bf16* Vl = smem + KT * DK;
-  const int kt0 = b_lo / KT, kt1 = b_hi / KT;
+  const TileWalk walk(a, b_lo, b_hi);
   const int* bt = a.block_table + (size_t)s * a.max_blocks;
-  int base_kt = kt0, bt_v = kt0 + lane <= kt1 ? bt[kt0 + lane] : 0;   // 64 table entries per load
-  for (int kt = kt0; kt <= kt1; ++kt) {
-    if (kt - base_kt >= 64) {
-      base_kt = kt;
-      bt_v = kt + lane <= kt1 ? bt[kt + lane] : 0;
-    }
-    const size_t blk = (size_t)__builtin_amdgcn_readlane(bt_v, kt - base_kt) * Hkv + kvh;
+  int bt_v = 0;                                          // 64 table entries per load
+  for (int i = 0; i < walk.n; ++i) {
+    if ((i & 63) == 0) bt_v = i + lane < walk.n ? bt[walk.tile(i + lane)] : 0;
+    const int kt = walk.tile(i);
+    const size_t blk = (size_t)__builtin_amdgcn_readlane(bt_v, i & 63) * Hkv + kvh;
     stage_rows<DK, 0, DK / 32>((const bf16*)a.kc + blk * (KT * DK), Kl, wave * (DK / 32), lane);
     stage_rows<DV, 0, DV / 32>((const bf16*)a.vc + blk * (KT * DV), Vl, wave * (DV / 32), lane);
     __syncthreads();                                     // drains the LDS-DMA
@@ -280,7 +174,7 @@ void attn_tile_kernel(const MaskedAttnArgs a) {
       __syncthreads();
     }
     const int k_lo = kt * KT, k_hi = k_lo + KT - 1;
-    if (w_on && k_lo <= wp1 && k_hi >= w_lo) {           // (wave-uniform) some row of the wave sees it
+    if (w_on && k_lo <= wp1 && (k_hi >= w_lo || k_lo < a.keep)) {   // (wave-uniform) some row of the wave sees it
       f32x4 sacc[4];
 #pragma unroll
       for (int nt = 0; nt < 4; ++nt) {
@@ -293,9 +187,10 @@ void attn_tile_kernel(const MaskedAttnArgs a) {
         }
       }
       bf16x8 pf[2];
-      const float alpha = (k_hi <= wp0 && k_lo >= w_in)
-                              ? tile_weights<MODE, false>(sacc, pf, st, kc, 0, 0, fq)
-                              : tile_weights<MODE, true>(sacc, pf, st, kc, first - k_lo, qpos - k_lo, fq);
+      const int lo = first - k_lo, hi = qpos - k_lo, keep = a.keep - k_lo;
+      const float alpha = (k_hi <= wp0 && (k_lo >= w_in || keep >= KT))
+                              ? tile_weights<MODE, false>(sacc, pf, st, kc, lo, hi, keep, fq)
+                              : tile_weights<MODE, true>(sacc, pf, st, kc, lo, hi, keep, fq);
       if constexpr (MODE != CAPPED_NOMAX) {
 #pragma unroll
         for (int dt = 0; dt < DV / 16; ++dt) o[dt] *= alpha;
@@ -307,7 +202,7 @@ void attn_tile_kernel(const MaskedAttnArgs a) {
   float l = st.l + __shfl_xor(st.l, 16, 64);
   l += __shfl_xor(l, 32, 64);
   if (!valid) return;
-  const float inv = l > 0.f ? 1.f / l : 0.f;
+  const float inv = l > 0.f ? head_gate<bf16>(a, qs + tok, head) / l : 0.f;
   bf16* op = (bf16*)a.out + ((size_t)(qs + tok) * a.Hq + head) * DV + 4 * fq;
 #pragma unroll
   for (int dt = 0; dt < DV / 16; ++dt) {
@@ -343,9 +238,9 @@ void attn_split_kernel(const MaskedAttnArgs a) {
   const int rr = row0 + (valid ? fr : 0);
   const int tok = q0 + rr / G, head = kvh * G + rr % G;
   const int base = cl - ql, qpos = base + tok;
-  const int first = chunk_start(qpos, a.chunk);
+  const int first = first_key(a, qpos);
   const int p0 = base + q0 + row0 / G, p1 = base + q0 + (row0 + rows - 1) / G;
-  const int lo = chunk_start(p0, a.chunk), in = chunk_start(p1, a.chunk);
+  const int lo = first_key(a, p0), in = first_key(a, p1);
 
   bf16x8 qf[DK / 32];
   {
@@ -353,25 +248,24 @@ void attn_split_kernel(const MaskedAttnArgs a) {
 #pragma unroll
     for (int ks = 0; ks < DK / 32; ++ks) qf[ks] = *reinterpret_cast<const bf16x8*>(qp + 32 * ks);
   }
-  const ScoreConst kc = score_const<MODE>(a);
-  const bool sink = a.sink && z == 0 && wave == 0;
-  Run st;
-  st.m = MODE == CAPPED_NOMAX || sink ? 0.f : -INFINITY;
-  st.l = sink && fq == 0 ? 1.f : 0.f;
+  const ScoreConst kc = score_const<MODE>(a, head);
+  Run st = run_start<MODE>(a, head, a.sink && z == 0 && wave == 0, fq);
   f32x4 o[DV / 16];
 #pragma unroll
   for (int i = 0; i < DV / 16; ++i) o[i] = f32x4{0.f, 0.f, 0.f, 0.f};
 
   bf16* Vl = smem + wave * (KT * DV);
-  const int kt0 = lo / KT, kt1 = p1 / KT, step = NWV * nz;
+  const TileWalk walk(a, lo, p1);
+  const int step = NWV * nz;
   const int* bt = a.block_table + (size_t)s * a.max_blocks;
-  int kt = kt0 + z * NWV + wave, left = 0, bt_v = 0;
-  for (; kt <= kt1; kt += step, --left) {
+  int left = 0, bt_v = 0;
+  for (int it = z * NWV + wave; it < walk.n; it += step, --left) {
     if (left == 0) {                                     // the wave's next 64 table entries
-      const int i = kt + lane * step;
-      bt_v = i <= kt1 ? bt[i] : 0;
+      const int i = it + lane * step;
+      bt_v = i < walk.n ? bt[walk.tile(i)] : 0;
       left = 64;
     }
+    const int kt = walk.tile(it);
     const size_t blk = (size_t)__builtin_amdgcn_readlane(bt_v, 64 - left) * Hkv + kvh;
     const bf16* kp = (const bf16*)a.kc + blk * (KT * DK) + fr * DK + 8 * fq;
     bf16x8 kf[4][DK / 32];
@@ -390,9 +284,10 @@ void attn_split_kernel(const MaskedAttnArgs a) {
     }
     const int k_lo = kt * KT, k_hi = k_lo + KT - 1;
     bf16x8 pf[2];
-    const float alpha = (k_hi <= p0 && k_lo >= in)
-                            ? tile_weights<MODE, false>(sacc, pf, st, kc, 0, 0, fq)
-                            : tile_weights<MODE, true>(sacc, pf, st, kc, first - k_lo, qpos - k_lo, fq);
+    const int wlo = first - k_lo, whi = qpos - k_lo, keep = a.keep - k_lo;
+    const float alpha = (k_hi <= p0 && (k_lo >= in || keep >= KT))
+                            ? tile_weights<MODE, false>(sacc, pf, st, kc, wlo, whi, keep, fq)
+                            : tile_weights<MODE, true>(sacc, pf, st, kc, wlo, whi, keep, fq);
     if constexpr (MODE != CAPPED_NOMAX) {
 #pragma unroll
       for (int dt = 0; dt < DV / 16; ++dt) o[dt] *= alpha;
@@ -442,7 +337,9 @@ void attn_split_kernel(const MaskedAttnArgs a) {
                                               c0 + 64 * i) * wgt[w];
   }
   bf16* op = (bf16*)a.out + orow * DV + c0;
+  const float gate = head_gate<bf16>(a, orow / a.Hq, (int)(orow % a.Hq));
   auto put = [&](float inv) {
+    inv *= gate;
 #pragma unroll
     for (int i = 0; i < DV / 64; ++i) {
       bf16x4 b;
@@ -520,7 +417,8 @@ void launch_mode(const MaskedAttnArgs& a, int nwork, int form, int nz, hipStream
 
 template <int DK, int DV>
 void launch_dims(const MaskedAttnArgs& a, int nwork, int form, int nz, hipStream_t s) {
-  if (a.cap <= 0.f) launch_mode<DK, DV, PLAIN>(a, nwork, form, nz, s);
+  if (a.slopes) launch_mode<DK, DV, BIASED>(a, nwork, form, nz, s);
+  else if (a.cap <= 0.f) launch_mode<DK, DV, PLAIN>(a, nwork, form, nz, s);
   else if (a.cap <= NOMAX_CAP) launch_mode<DK, DV, CAPPED_NOMAX>(a, nwork, form, nz, s);
   else launch_mode<DK, DV, CAPPED>(a, nwork, form, nz, s);
 }
@@ -543,7 +441,7 @@ int launch_dk(const MaskedAttnArgs& a, int nwork, int form, int nz, hipStream_t 
 int launch_attn_masked(const MaskedAttnArgs& args, int nwork, int form, int nz, hipStream_t s) {
   MaskedAttnArgs a = args;
   if (nwork <= 0) return 0;
-  if (form != 1 && form != 4) return 1;
+  if ((form != 1 && form != 4) || (a.slopes && a.cap > 0.f)) return 1;
   if (nz < 1 || (form == 4 && nz != 1) || (nz > 1 && (!a.split_o || !a.split_ml))) return 2;
   if (nz > 1) {
     // tickets: one per item, key head and row group (the split-KV tickets of attention.hip)

@@ -746,7 +746,7 @@ void sample_dense(const at::Tensor& logits, const at::Tensor& allow_ptr, const a
 // is fine), w_post / w_pre [Hp] f32 or none
 void residual_norm(at::Tensor& x, const c10::optional<at::Tensor>& y,
                    const c10::optional<at::Tensor>& w_post, const c10::optional<at::Tensor>& w_pre,
-                   const c10::optional<at::Tensor>& out, int64_t H, double eps) {
+                   const c10::optional<at::Tensor>& out, int64_t H, double eps, bool center) {
   CHECK_F32_TENSOR(x);
   const int Hp = x.size(-1), rows = x.numel() / Hp;
   bool f32 = false;
@@ -754,7 +754,7 @@ void residual_norm(at::Tensor& x, const c10::optional<at::Tensor>& y,
   if (y.has_value()) {
     CHECK_TENSOR((*y));
     f32 = low_is_f32(*y);
-    TORCH_CHECK(y->numel() == x.numel() && w_post.has_value(), "residual_norm: y [T, Hp] with w_post");
+    TORCH_CHECK(y->numel() == x.numel(), "residual_norm: y [T, Hp]");
   }
   for (const auto* w : {&w_post, &w_pre})
     if (w->has_value()) { CHECK_F32_TENSOR((**w)); TORCH_CHECK((*w)->numel() == Hp, "norm weight [Hp]"); }
@@ -771,7 +771,7 @@ void residual_norm(at::Tensor& x, const c10::optional<at::Tensor>& y,
                                    w_post.has_value() ? w_post->data_ptr<float>() : nullptr,
                                    w_pre.has_value() ? w_pre->data_ptr<float>() : nullptr,
                                    out.has_value() ? out->data_ptr() : nullptr, ld, rows, (int)H, Hp,
-                                   (float)eps, f32, stream()) == 0,
+                                   (float)eps, center, f32, stream()) == 0,
               "residual_norm: unsupported width ", Hp);
   check_launch("residual_norm");
 }
@@ -800,11 +800,14 @@ void logit_finish(at::Tensor& z, double scale, double cap) {
   check_launch("logit_finish");
 }
 
-void gemm_f32(const at::Tensor& X, const at::Tensor& W, at::Tensor& Y) {
+void gemm_f32(const at::Tensor& X, const at::Tensor& W, at::Tensor& Y,
+              const c10::optional<at::Tensor>& R) {
   CHECK_F32_TENSOR(X); CHECK_F32_TENSOR(W); CHECK_F32_TENSOR(Y);
   const int K = X.size(-1), M = X.numel() / K, N = W.size(0);
   TORCH_CHECK(W.dim() == 2 && W.size(1) == K && Y.numel() == (int64_t)M * N, "gemm_f32 shapes");
-  TORCH_CHECK(launch_gemm_f32(X.data_ptr<float>(), W.data_ptr<float>(), Y.data_ptr<float>(), M, N, K,
+  if (R.has_value()) { CHECK_F32_TENSOR((*R)); TORCH_CHECK(R->numel() == Y.numel(), "gemm_f32: R shape"); }
+  TORCH_CHECK(launch_gemm_f32(X.data_ptr<float>(), W.data_ptr<float>(),
+                              R.has_value() ? R->data_ptr<float>() : nullptr, Y.data_ptr<float>(), M, N, K,
                               stream()) == 0, "gemm_f32: K % 16 == 0, N % 4 == 0");
   check_launch("gemm_f32");
 }
@@ -841,34 +844,153 @@ void rope_kv_any(const at::Tensor& qkv, const c10::optional<at::Tensor>& bias, c
   check_launch("rope_kv_any");
 }
 
-MaskedAttnArgs masked_args(const at::Tensor& q, const at::Tensor& k_cache, const at::Tensor& v_cache,
-                           at::Tensor& out, const at::Tensor& q_start, const at::Tensor& q_len,
-                           const at::Tensor& ctx_len, const at::Tensor& block_table, double scale,
-                           double cap, int64_t chunk, bool sink) {
-  CHECK_TENSOR(q); CHECK_TENSOR(k_cache); CHECK_TENSOR(v_cache); CHECK_TENSOR(out);
+// a [T, C] view with rows of its own stride, inner stride 1
+void check_rows(const at::Tensor& t, int64_t T, at::ScalarType type, const char* what) {
+  CHECK_DEV(t);
+  TORCH_CHECK(t.dim() == 2 && t.size(0) == T && t.stride(1) == 1 && t.scalar_type() == type, what,
+              ": rows [T, C] of one type, inner stride 1");
+}
+
+void qk_norm_kv(const at::Tensor& z, const at::Tensor& slots, const at::Tensor& wq, const at::Tensor& wk,
+                int64_t dim, double eps, at::Tensor& q_out, at::Tensor& k_cache, at::Tensor& v_cache,
+                const c10::optional<at::Tensor>& v_first, double lam) {
+  const int T = slots.numel();
+  check_rows(z, T, q_out.scalar_type(), "qk_norm_kv: z");
+  CHECK_I32_TENSOR(slots); CHECK_F32_TENSOR(wq); CHECK_F32_TENSOR(wk);
+  CHECK_TENSOR(q_out); CHECK_TENSOR(k_cache); CHECK_TENSOR(v_cache);
+  const bool f32 = low_is_f32(q_out);
+  for (const auto* t : {&k_cache, &v_cache})
+    TORCH_CHECK(t->scalar_type() == q_out.scalar_type(), "qk_norm_kv: one type");
+  TORCH_CHECK(q_out.dim() == 3 && q_out.size(0) == T && k_cache.dim() == 4 && v_cache.dim() == 4, "qk_norm_kv dims");
+  const int Hq = q_out.size(1), DK = q_out.size(2), Hkv = k_cache.size(1), BS = k_cache.size(2),
+            DV = v_cache.size(3);
+  TORCH_CHECK(k_cache.size(3) == DK && v_cache.size(0) == k_cache.size(0) && v_cache.size(1) == Hkv &&
+                  v_cache.size(2) == BS, "qk_norm_kv: caches [nb, Hkv, BS, D]");
+  TORCH_CHECK(z.size(1) >= (int64_t)(Hq + Hkv) * DK + (int64_t)Hkv * DV, "qk_norm_kv: z [T, >= q | k | v]");
+  TORCH_CHECK(wq.numel() == DK && wk.numel() == DK && dim > 0 && dim <= DK, "qk_norm_kv: weights [DK]");
+  int ldv = 0;
+  if (v_first.has_value()) {
+    check_rows(*v_first, T, q_out.scalar_type(), "qk_norm_kv: v_first");
+    TORCH_CHECK(v_first->size(1) == (int64_t)Hkv * DV, "qk_norm_kv: v_first [T, Hkv DV]");
+    ldv = v_first->stride(0);
+  }
+  TORCH_CHECK(launch_qk_norm_kv(z.data_ptr(), z.stride(0), slots.data_ptr<int>(), wq.data_ptr<float>(),
+                                wk.data_ptr<float>(), (int)dim, (float)eps, q_out.data_ptr(),
+                                k_cache.data_ptr(), v_cache.data_ptr(),
+                                v_first.has_value() ? v_first->data_ptr() : nullptr, ldv, (float)lam, T, Hq,
+                                Hkv, DK, DV, BS, f32, stream()) == 0, "qk_norm_kv: head sizes or strides");
+  check_launch("qk_norm_kv");
+}
+
+void latent_qkv(const at::Tensor& z, const at::Tensor& pos, const at::Tensor& slots, const at::Tensor& cos_sin,
+                const at::Tensor& w_c, double eps, int64_t heads, int64_t dim, int64_t rot, int64_t rank,
+                int64_t rank_true, at::Tensor& q_out, at::Tensor& k_cache) {
+  const int T = slots.numel();
+  check_rows(z, T, q_out.scalar_type(), "latent_qkv: z");
+  CHECK_I32_TENSOR(pos); CHECK_I32_TENSOR(slots); CHECK_F32_TENSOR(cos_sin); CHECK_F32_TENSOR(w_c);
+  CHECK_TENSOR(q_out); CHECK_TENSOR(k_cache);
+  TORCH_CHECK(k_cache.scalar_type() == q_out.scalar_type(), "latent_qkv: one type");
+  TORCH_CHECK(q_out.dim() == 3 && q_out.size(0) == T && q_out.size(1) == heads && pos.numel() == T &&
+                  k_cache.dim() == 4 && k_cache.size(1) == 1 && k_cache.size(3) == q_out.size(2),
+              "latent_qkv: q_out [T, heads, DK], cache [nb, 1, BS, DK]");
+  TORCH_CHECK(z.size(1) >= heads * (dim + rot) + rank + rot && w_c.numel() == rank && rank_true > 0 &&
+                  rank_true <= rank, "latent_qkv: z [T, >= heads (dim + rot) + rank + rot], w_c [rank]");
+  TORCH_CHECK(cos_sin.dim() == 3 && cos_sin.size(2) == 2, "cos_sin [P, pairs, 2]");
+  LatentRowArgs a{};
+  a.z = z.data_ptr();
+  a.ldz = z.stride(0);
+  a.pos = pos.data_ptr<int>();
+  a.slots = slots.data_ptr<int>();
+  a.cos_sin = cos_sin.data_ptr<float>();
+  a.pairs = cos_sin.size(1);
+  a.w_c = w_c.data_ptr<float>();
+  a.eps = (float)eps;
+  a.heads = heads;
+  a.dim = dim;
+  a.rot = rot;
+  a.rank = rank;
+  a.rank_true = rank_true;
+  a.q_out = q_out.data_ptr();
+  a.k_cache = k_cache.data_ptr();
+  a.DK = q_out.size(2);
+  a.BS = k_cache.size(2);
+  a.T = T;
+  TORCH_CHECK(launch_latent_rows(a, low_is_f32(q_out), stream()) == 0, "latent_qkv: sizes");
+  check_launch("latent_qkv");
+}
+
+void gemm_heads(const at::Tensor& X, const at::Tensor& W, at::Tensor& out) {
+  CHECK_DEV(X); CHECK_TENSOR(W); CHECK_DEV(out);
+  const bool f32 = low_is_f32(W);
+  TORCH_CHECK(X.scalar_type() == W.scalar_type() && out.scalar_type() == W.scalar_type(), "gemm_heads: one type");
+  TORCH_CHECK(X.dim() == 3 && W.dim() == 3 && out.dim() == 3 && X.stride(2) == 1 && out.stride(2) == 1,
+              "gemm_heads: X [T, H, K], W [H, N, K], out [T, H, N], inner stride 1");
+  HeadGemmArgs a{};
+  a.T = X.size(0);
+  a.H = W.size(0);
+  a.N = W.size(1);
+  a.K = W.size(2);
+  TORCH_CHECK(X.size(1) == a.H && X.size(2) == a.K && out.size(0) == a.T && out.size(1) == a.H &&
+                  out.size(2) == a.N, "gemm_heads shapes");
+  a.X = X.data_ptr();
+  a.W = W.data_ptr();
+  a.out = out.data_ptr();
+  a.xt = X.stride(0);
+  a.xh = X.stride(1);
+  a.ot = out.stride(0);
+  a.oh = out.stride(1);
+  TORCH_CHECK(((uintptr_t)a.X | (uintptr_t)a.out) % 16 == 0, "gemm_heads: 16-byte aligned views");
+  TORCH_CHECK(launch_gemm_heads(a, f32, stream()) == 0, "gemm_heads: K % 32, N % 16, strides % 8");
+  check_launch("gemm_heads");
+}
+
+MaskedAttnArgs masked_args(const at::Tensor& q, const at::Tensor& k_cache,
+                           const c10::optional<at::Tensor>& v_cache, at::Tensor& out,
+                           const at::Tensor& q_start, const at::Tensor& q_len, const at::Tensor& ctx_len,
+                           const at::Tensor& block_table, double scale, double cap, int64_t chunk, bool sink,
+                           int64_t window, int64_t keep, const c10::optional<at::Tensor>& slopes,
+                           const c10::optional<at::Tensor>& sinks, const c10::optional<at::Tensor>& gate) {
+  CHECK_TENSOR(q); CHECK_TENSOR(k_cache); CHECK_TENSOR(out);
   CHECK_I32_TENSOR(q_start); CHECK_I32_TENSOR(q_len); CHECK_I32_TENSOR(ctx_len);
   CHECK_I32_TENSOR(block_table);
-  for (const auto* t : {&k_cache, &v_cache, (const at::Tensor*)&out})
+  for (const auto* t : {&k_cache, (const at::Tensor*)&out})
     TORCH_CHECK(t->scalar_type() == q.scalar_type(), "masked attention: one type");
-  TORCH_CHECK(q.dim() == 3 && k_cache.dim() == 4 && v_cache.dim() == 4 && out.dim() == 3 &&
-                  block_table.dim() == 2, "masked attention dims");
+  TORCH_CHECK(q.dim() == 3 && k_cache.dim() == 4 && out.dim() == 3 && block_table.dim() == 2,
+              "masked attention dims");
   MaskedAttnArgs a{};
   a.Hq = q.size(1);
   a.DK = q.size(2);
   a.Hkv = k_cache.size(1);
-  a.DV = v_cache.size(3);
+  a.DV = out.size(2);
   a.S = q_len.numel();
   a.max_blocks = block_table.size(1);
-  TORCH_CHECK(a.Hq % a.Hkv == 0 && k_cache.size(2) == 64 && v_cache.size(2) == 64 &&
-                  k_cache.size(3) == a.DK && v_cache.size(1) == a.Hkv && v_cache.size(0) == k_cache.size(0),
+  TORCH_CHECK(a.Hq % a.Hkv == 0 && k_cache.size(2) == 64 && k_cache.size(3) == a.DK,
               "masked attention: caches [nb, Hkv, 64, D]");
-  TORCH_CHECK(out.size(0) == q.size(0) && out.size(1) == a.Hq && out.size(2) == a.DV, "out [T, Hq, DV]");
+  if (v_cache.has_value()) {
+    CHECK_TENSOR((*v_cache));
+    TORCH_CHECK(v_cache->scalar_type() == q.scalar_type() && v_cache->dim() == 4 && v_cache->size(2) == 64 &&
+                    v_cache->size(1) == a.Hkv && v_cache->size(0) == k_cache.size(0) && v_cache->size(3) == a.DV,
+                "masked attention: value cache [nb, Hkv, 64, DV]");
+    a.vc = v_cache->data_ptr();
+  } else {
+    TORCH_CHECK(a.DV <= a.DK, "masked attention: values inside the keys");
+  }
+  TORCH_CHECK(out.size(0) == q.size(0) && out.size(1) == a.Hq, "out [T, Hq, DV]");
   TORCH_CHECK(q_start.numel() == a.S && ctx_len.numel() == a.S && block_table.size(0) == a.S,
               "masked attention: per-sequence arrays");
-  TORCH_CHECK(chunk >= 0 && cap >= 0, "masked attention: chunk, cap >= 0");
+  TORCH_CHECK(chunk >= 0 && cap >= 0 && window >= 0 && keep >= 0 && !(chunk > 0 && window > 0),
+              "masked attention: chunk, cap, window, keep >= 0, one of chunk and window");
+  for (const auto* t : {&slopes, &sinks})
+    if (t->has_value()) { CHECK_F32_TENSOR((**t)); TORCH_CHECK((*t)->numel() == a.Hq, "slopes, sinks [Hq]"); }
+  TORCH_CHECK(!(slopes.has_value() && cap > 0), "masked attention: slopes or a soft cap");
+  if (gate.has_value()) {
+    check_rows(*gate, q.size(0), q.scalar_type(), "masked attention: gate");
+    TORCH_CHECK(gate->size(1) == a.Hq, "gate [T, Hq]");
+    a.gate = gate->data_ptr();
+    a.gate_ld = gate->stride(0);
+  }
   a.q = q.data_ptr();
   a.kc = k_cache.data_ptr();
-  a.vc = v_cache.data_ptr();
   a.out = out.data_ptr();
   a.q_start = q_start.data_ptr<int>();
   a.q_len = q_len.data_ptr<int>();
@@ -878,20 +1000,26 @@ MaskedAttnArgs masked_args(const at::Tensor& q, const at::Tensor& k_cache, const
   a.cap = (float)cap;
   a.chunk = (int)chunk;
   a.sink = sink;
+  a.window = (int)window;
+  a.keep = window > 0 ? (int)keep : 0;
+  a.slopes = slopes.has_value() ? slopes->data_ptr<float>() : nullptr;
+  a.sinks = sinks.has_value() ? sinks->data_ptr<float>() : nullptr;
   return a;
 }
 
-// one work list of the MFMA forms (form 4 / 1, attention_masked.hip); false: head
-// sizes outside them, nothing launched
-bool attention_masked(const at::Tensor& q, const at::Tensor& k_cache, const at::Tensor& v_cache,
+// one work list of the MFMA forms (form 4 / 1, attention_masked.hip; without a
+// value cache attention_latent.hip); false: head sizes outside them, nothing launched
+bool attention_masked(const at::Tensor& q, const at::Tensor& k_cache, const c10::optional<at::Tensor>& v_cache,
                       at::Tensor& out, const at::Tensor& q_start, const at::Tensor& q_len,
                       const at::Tensor& ctx_len, const at::Tensor& block_table,
                       const at::Tensor& work_seq, const at::Tensor& work_q0, int64_t form,
                       int64_t item_tokens, double scale, double cap, int64_t chunk, bool sink,
+                      int64_t window, int64_t keep, const c10::optional<at::Tensor>& slopes,
+                      const c10::optional<at::Tensor>& sinks, const c10::optional<at::Tensor>& gate,
                       int64_t nz, const c10::optional<at::Tensor>& split_o,
                       const c10::optional<at::Tensor>& split_ml) {
   MaskedAttnArgs a = masked_args(q, k_cache, v_cache, out, q_start, q_len, ctx_len, block_table,
-                                 scale, cap, chunk, sink);
+                                 scale, cap, chunk, sink, window, keep, slopes, sinks, gate);
   CHECK_BF16(q); CHECK_I32_TENSOR(work_seq); CHECK_I32_TENSOR(work_q0);
   TORCH_CHECK(work_seq.numel() == work_q0.numel() && item_tokens > 0, "attention_masked: work list");
   a.work_seq = work_seq.data_ptr<int>();
@@ -906,20 +1034,23 @@ bool attention_masked(const at::Tensor& q, const at::Tensor& k_cache, const at::
     a.split_o = split_o->data_ptr<float>();
     a.split_ml = split_ml->data_ptr<float>();
   }
-  const int rc = launch_attn_masked(a, work_seq.numel(), (int)form, (int)nz, stream());
+  const int rc = v_cache.has_value() ? launch_attn_masked(a, work_seq.numel(), (int)form, (int)nz, stream())
+                                     : launch_attn_latent(a, work_seq.numel(), (int)nz, stream());
   if (rc == 3) return false;
   TORCH_CHECK(rc == 0, "attention_masked: code ", rc);
   check_launch("attention_masked");
   return true;
 }
 
-void attention_row(const at::Tensor& q, const at::Tensor& k_cache, const at::Tensor& v_cache,
+void attention_row(const at::Tensor& q, const at::Tensor& k_cache, const c10::optional<at::Tensor>& v_cache,
                    at::Tensor& out, const at::Tensor& q_start, const at::Tensor& q_len,
                    const at::Tensor& ctx_len, const at::Tensor& block_table, double scale, double cap,
-                   int64_t chunk, bool sink) {
+                   int64_t chunk, bool sink, int64_t window, int64_t keep,
+                   const c10::optional<at::Tensor>& slopes, const c10::optional<at::Tensor>& sinks,
+                   const c10::optional<at::Tensor>& gate) {
   const MaskedAttnArgs a = masked_args(q, k_cache, v_cache, out, q_start, q_len, ctx_len, block_table,
-                                       scale, cap, chunk, sink);
-  TORCH_CHECK(launch_attn_row(a, q.size(0), low_is_f32(q), stream()) == 0, "attention_row: value heads <= 512");
+                                       scale, cap, chunk, sink, window, keep, slopes, sinks, gate);
+  TORCH_CHECK(launch_attn_row(a, q.size(0), low_is_f32(q), stream()) == 0, "attention_row: value heads <= 1024");
   check_launch("attention_row");
 }
 
@@ -1170,14 +1301,18 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("residual_norm", &residual_norm);
   m.def("embedding_scaled", &embedding_scaled);
   m.def("logit_finish", &logit_finish);
-  m.def("gemm_f32", &gemm_f32);
+  m.def("gemm_f32", &gemm_f32, py::arg("X"), py::arg("W"), py::arg("Y"), py::arg("R") = py::none());
+  m.def("qk_norm_kv", &qk_norm_kv);
+  m.def("latent_qkv", &latent_qkv);
+  m.def("gemm_heads", &gemm_heads);
   m.def("gated_act_f32", &gated_act_f32);
   m.def("rope_kv_any", &rope_kv_any);
   m.def("attention_row", &attention_row);
   m.def("attention_masked", &attention_masked, py::arg("q"), py::arg("k_cache"), py::arg("v_cache"),
         py::arg("out"), py::arg("q_start"), py::arg("q_len"), py::arg("ctx_len"), py::arg("block_table"),
         py::arg("work_seq"), py::arg("work_q0"), py::arg("form"), py::arg("item_tokens"),
-        py::arg("scale"), py::arg("cap"), py::arg("chunk"), py::arg("sink"), py::arg("nz") = 1,
+        py::arg("scale"), py::arg("cap"), py::arg("chunk"), py::arg("sink"), py::arg("window"),
+        py::arg("keep"), py::arg("slopes"), py::arg("sinks"), py::arg("gate"), py::arg("nz") = 1,
         py::arg("split_o") = py::none(), py::arg("split_ml") = py::none());
   m.def("branch_select", &branch_select);
   m.def("add_inplace", &add_inplace);

@@ -1,4 +1,4 @@
-// True 32-bit TN GEMM, Y[M, N] = X[M, K] W[N, K]^T, for the 32-bit mode of the
+// True 32-bit TN GEMM, Y[M, N] = X[M, K] W[N, K]^T (+ R), for the 32-bit mode of the
 // models that have one.  64 x 64 tiles, 16-wide k-steps through LDS, 4 x 4
 // outputs per thread with plain fp32 FMAs.  Every output is one sum in k order,
 // so a row's result does not depend on the other rows of the call.
@@ -10,7 +10,7 @@ constexpr int FT = 64, FK = 16;
 
 __global__ __launch_bounds__(256) void gemm_f32_kernel(const float* __restrict__ X,
                                                        const float* __restrict__ W,
-                                                       float* __restrict__ Y, int M, int N, int K) {
+                                                       const float* __restrict__ R, float* __restrict__ Y, int M, int N, int K) {
   __shared__ float xs[FK][FT + 4], ws[FK][FT + 4];
   const int m0 = blockIdx.y * FT, n0 = blockIdx.x * FT;
   const int tr = threadIdx.x >> 4, tc = threadIdx.x & 15;
@@ -41,8 +41,11 @@ __global__ __launch_bounds__(256) void gemm_f32_kernel(const float* __restrict__
 #pragma unroll
   for (int i = 0; i < 4; ++i) {
     const int m = m0 + tr * 4 + i, n = n0 + tc * 4;
-    if (m < M && n < N)
-      *reinterpret_cast<f32x4*>(Y + (size_t)m * N + n) = f32x4{acc[i][0], acc[i][1], acc[i][2], acc[i][3]};
+    if (m < M && n < N) {
+      f32x4 v = f32x4{acc[i][0], acc[i][1], acc[i][2], acc[i][3]};
+      if (R) v += *reinterpret_cast<const f32x4*>(R + (size_t)m * N + n);
+      *reinterpret_cast<f32x4*>(Y + (size_t)m * N + n) = v;
+    }
   }
 }
 
@@ -67,10 +70,11 @@ __global__ __launch_bounds__(256) void gated_act_f32_kernel(const float* __restr
 }
 }  // namespace
 
-int launch_gemm_f32(const float* X, const float* W, float* Y, int M, int N, int K, hipStream_t s) {
+int launch_gemm_f32(const float* X, const float* W, const float* R, float* Y, int M, int N, int K,
+                    hipStream_t s) {
   if (K % FK || N % 4) return 1;
   if (M <= 0 || N <= 0) return 0;
-  gemm_f32_kernel<<<dim3((N + FT - 1) / FT, (M + FT - 1) / FT), 256, 0, s>>>(X, W, Y, M, N, K);
+  gemm_f32_kernel<<<dim3((N + FT - 1) / FT, (M + FT - 1) / FT), 256, 0, s>>>(X, W, R, Y, M, N, K);
   return 0;
 }
 

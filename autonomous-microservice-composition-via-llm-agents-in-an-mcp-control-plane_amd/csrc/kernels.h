@@ -51,21 +51,55 @@ int launch_rope_kv_any(const void* qkv, const float* bias, const int* pos, const
                        const void* cos_sin, void* q_out, void* k_cache, void* v_cache, int T, int Hq,
                        int Hkv, int DK, int DV, int BS, bool f32, hipStream_t s);
 
-// residual.hip: fp32 residual stream, norms on both sides of a sublayer
+// head_rows.hip: projected rows -> queries and cache.  Per-head rms norms of q and
+// k and mixed values; latent attention's row and rotated parts.
+int launch_qk_norm_kv(const void* z, int ldz, const int* slots, const float* wq, const float* wk,
+                      int dim, float eps, void* q_out, void* k_cache, void* v_cache,
+                      const void* v_first, int ldv, float lam, int T, int Hq, int Hkv, int DK,
+                      int DV, int BS, bool f32, hipStream_t s);
+struct LatentRowArgs {
+  const void* z;             // [T, ldz]: heads x [dim | rot], latent [rank], rotated key [rot], ...
+  int ldz;
+  const int* pos;
+  const int* slots;
+  const float* cos_sin;      // [P, pairs, 2]
+  int pairs;
+  const float* w_c;          // [rank]
+  float eps;
+  int heads, dim, rot, rank, rank_true;
+  void* q_out;               // [T, heads, DK], columns from rank on are written
+  void* k_cache;             // [nb, 1, BS, DK]
+  int DK, BS, T;
+};
+int launch_latent_rows(const LatentRowArgs& a, bool f32, hipStream_t s);
+
+// gemm_heads.hip: one product per head, out[t, h, n] = sum_k X[t, h, k] W[h, n, k];
+// strides in elements, inner stride 1
+struct HeadGemmArgs {
+  const void* X;
+  const void* W;
+  void* out;
+  long long xt, xh, ot, oh;  // token and head strides of X and out
+  int T, H, N, K;
+};
+int launch_gemm_heads(const HeadGemmArgs& a, bool f32, hipStream_t s);
+
+// residual.hip: fp32 residual stream, norms around the sublayers
 constexpr int RESIDUAL_MAX_WIDTH = 16384;
 int launch_residual_norm(float* x, const void* y, const float* w_post, const float* w_pre,
-                         void* out, int ld, int rows, int H, int Hp, float eps, bool f32,
-                         hipStream_t s);
+                         void* out, int ld, int rows, int H, int Hp, float eps, bool center,
+                         bool f32, hipStream_t s);
 void launch_embedding_scaled(const int* ids, const void* table, float scale, float* x, void* lo,
                              int ld, int T, int Hp, bool f32, hipStream_t s);
 void launch_logit_finish(float* z, size_t n, float scale, float cap, hipStream_t s);
 
 // gemm_f32.hip: the 32-bit mode's products
 enum GatedAct { ACT_SILU = 0, ACT_GELU_TANH = 1 };
-int launch_gemm_f32(const float* X, const float* W, float* Y, int M, int N, int K, hipStream_t s);
+int launch_gemm_f32(const float* X, const float* W, const float* R, float* Y, int M, int N, int K,
+                    hipStream_t s);
 void launch_gated_act_f32(const float* z, float* y, int M, int F, int act, hipStream_t s);
 
-// attention_masked.hip
+// attention_masked.hip, attention_latent.hip
 struct MaskedAttnArgs {
   const void* q;
   const void* kc;
@@ -80,6 +114,11 @@ struct MaskedAttnArgs {
   float scale, cap;          // cap 0: no soft cap
   int chunk;                 // 0: plain causal
   int sink;
+  int window, keep;          // window > 0: the last ``window`` keys and the first ``keep``
+  const float* slopes;       // [Hq] or null: s -= slope (query position - key position)
+  const float* sinks;        // [Hq] or null: the sinks' scores (null: 0)
+  const void* gate;          // [T, Hq] rows of gate_ld in q's type, or null: out *= sigmoid(gate)
+  int gate_ld;
   // work-list forms: items of item_tokens tokens
   const int* work_seq;
   const int* work_q0;
@@ -91,8 +130,11 @@ struct MaskedAttnArgs {
   int* tickets;              // set by the launcher
 };
 int launch_attn_masked(const MaskedAttnArgs& a, int nwork, int form, int nz, hipStream_t s);
+// values are the first DV columns of the keys (vc is not read); either work list
+int launch_attn_latent(const MaskedAttnArgs& a, int nwork, int nz, hipStream_t s);
 constexpr int ATTN_SPLIT_TICKETS = 1 << 16;
 int* attn_split_counters();  // this device's tickets, zero between launches (attention.hip)
+// vc null: values are the first DV columns of the keys
 int launch_attn_row(const MaskedAttnArgs& a, int T, bool f32, hipStream_t s);
 
 // QKV projection + RoPE + paged K/V write fused in the GEMM epilogue (K1+K4+K10)

@@ -1,7 +1,6 @@
-// Row kernels of decoders whose residual stream is fp32 and whose sublayers are
-// normed on both sides (x += norm_post(f(norm_pre(x)))): the scaled embedding,
-// the post-norm + residual add + next pre-norm in one pass, and the capped
-// logits.  T is the activation type of the projections (bf16, or float in the
+// Row kernels of decoders whose residual stream is fp32: the scaled embedding,
+// the residual add (post-normed or plain) + next pre-norm (rms or layer norm) in
+// one pass, and the capped logits.  T is the activation type of the projections (bf16, or float in the
 // 32-bit mode); the residual, the norms and the logits are always fp32.
 #include "common.h"
 #include "kernels.h"
@@ -46,14 +45,15 @@ DEV float block_sum(float v, float* red) {
 // One block per row (1024 threads for few rows: shorter chains; 256 otherwise),
 // 4 floats per thread and step, the row and the norm weights in registers
 // between the passes:
-//   y given:      x += y / rms(y) * w_post          (written back)
+//   y given:      x += y / rms(y) * w_post, or x += y   (written back)
 //   w_pre given:  out = x / rms(x) * w_pre,  else out = x   (as T, row stride ld)
+//   CENTER:       the row's mean comes off x before that norm (layer norm)
 // Rows are Hp wide (columns >= H are zero and stay zero), means are over H.
-template <class T, int VMAX, int NT>
+template <class T, int VMAX, int NT, bool CENTER>
 __global__ __launch_bounds__(NT) void residual_norm_kernel(
     float* __restrict__ x, const T* __restrict__ y, const float* __restrict__ w_post,
     const float* __restrict__ w_pre, T* __restrict__ out, int ld, int H, int Hp, float eps) {
-  __shared__ float red[2][NT / 64];
+  __shared__ float red[3][NT / 64];
   const int row = blockIdx.x, nvec = Hp >> 2;
   float* xr = x + (size_t)row * Hp;
   const float inv_h = 1.f / (float)H;
@@ -67,12 +67,21 @@ __global__ __launch_bounds__(NT) void residual_norm_kernel(
       xv[i] = *reinterpret_cast<const f32x4*>(xr + 4 * c);
       if (y) yv[i] = load4(y + (size_t)row * Hp + 4 * c);
       if constexpr (EARLY) {
-        if (y) wa[i] = *reinterpret_cast<const f32x4*>(w_post + 4 * c);
+        if (w_post) wa[i] = *reinterpret_cast<const f32x4*>(w_post + 4 * c);
         if (w_pre) wb[i] = *reinterpret_cast<const f32x4*>(w_pre + 4 * c);
       }
     }
   }
-  if (y) {
+  if (y && !w_post) {
+#pragma unroll
+    for (int i = 0; i < VMAX; ++i) {
+      const int c = threadIdx.x + i * NT;
+      if (c < nvec) {
+        xv[i] += yv[i];
+        *reinterpret_cast<f32x4*>(xr + 4 * c) = xv[i];
+      }
+    }
+  } else if (y) {
     float ss = 0.f;
 #pragma unroll
     for (int i = 0; i < VMAX; ++i)
@@ -94,6 +103,19 @@ __global__ __launch_bounds__(NT) void residual_norm_kernel(
   float inv = 1.f;
   if (w_pre) {
     float ss = 0.f;
+    if constexpr (CENTER) {
+      float sum = 0.f;
+#pragma unroll
+      for (int i = 0; i < VMAX; ++i)
+#pragma unroll
+        for (int j = 0; j < 4; ++j) sum += xv[i][j];
+      const float mean = block_sum<NT>(sum, red[2]) * inv_h;
+#pragma unroll
+      for (int i = 0; i < VMAX; ++i)
+#pragma unroll
+        for (int j = 0; j < 4; ++j)                    // (columns from H on stay zero)
+          xv[i][j] = 4 * ((int)threadIdx.x + i * NT) + j < H ? xv[i][j] - mean : 0.f;
+    }
 #pragma unroll
     for (int i = 0; i < VMAX; ++i)
 #pragma unroll
@@ -118,9 +140,10 @@ __global__ __launch_bounds__(NT) void residual_norm_kernel(
 
 template <class T>
 void residual_norm_dispatch(float* x, const T* y, const float* w_post, const float* w_pre, T* out,
-                            int ld, int rows, int H, int Hp, float eps, hipStream_t s) {
-#define RN_CASE(V, NT) \
-  residual_norm_kernel<T, V, NT><<<rows, NT, 0, s>>>(x, y, w_post, w_pre, out, ld, H, Hp, eps)
+                            int ld, int rows, int H, int Hp, float eps, bool center, hipStream_t s) {
+#define RN_CASE(V, NT)                                                                                     \
+  (center ? residual_norm_kernel<T, V, NT, true><<<rows, NT, 0, s>>>(x, y, w_post, w_pre, out, ld, H, Hp, eps) \
+          : residual_norm_kernel<T, V, NT, false><<<rows, NT, 0, s>>>(x, y, w_post, w_pre, out, ld, H, Hp, eps))
   if (rows <= 512 && Hp > 1024) {
     const int v = (Hp / 4 + 1023) / 1024;
     if (v <= 1) RN_CASE(1, 1024);
@@ -167,14 +190,14 @@ __global__ __launch_bounds__(256) void logit_finish_kernel(float* __restrict__ z
 }  // namespace
 
 int launch_residual_norm(float* x, const void* y, const float* w_post, const float* w_pre,
-                         void* out, int ld, int rows, int H, int Hp, float eps, bool f32,
-                         hipStream_t s) {
+                         void* out, int ld, int rows, int H, int Hp, float eps, bool center,
+                         bool f32, hipStream_t s) {
   if (rows <= 0) return 0;
-  if (Hp % 4 || Hp > RESIDUAL_MAX_WIDTH || H > Hp || (y && !w_post)) return 1;
+  if (Hp % 4 || Hp > RESIDUAL_MAX_WIDTH || H > Hp || (w_post && !y)) return 1;
   if (f32)
-    residual_norm_dispatch<float>(x, (const float*)y, w_post, w_pre, (float*)out, ld, rows, H, Hp, eps, s);
+    residual_norm_dispatch<float>(x, (const float*)y, w_post, w_pre, (float*)out, ld, rows, H, Hp, eps, center, s);
   else
-    residual_norm_dispatch<bf16>(x, (const bf16*)y, w_post, w_pre, (bf16*)out, ld, rows, H, Hp, eps, s);
+    residual_norm_dispatch<bf16>(x, (const bf16*)y, w_post, w_pre, (bf16*)out, ld, rows, H, Hp, eps, center, s);
   return 0;
 }
 

@@ -1,6 +1,6 @@
 """Prefill and decode throughput of one design's layers beside another's.
 
-``bench.py --compare dozazen`` runs it: a few decoder layers with the sizes of a
+``bench.py --compare dozazen`` (or ``topelorn``) runs it: a few decoder layers with the sizes of a
 real model, random weights, on the engine's own step descriptors and paged cache
 - a prompt step eagerly, decode steps as the replayed hipGraph they are when
 served - for the design and for Llama at equal sizes, the two alternating.  One
@@ -26,7 +26,7 @@ PHASES = {"prefill_1x4096": (1, 0, 4096), "prefill_4x1024": (4, 0, 1024), "decod
 
 
 def _models(size: str, device, which):
-    from ..models import dozazen, llama
+    from ..models import dozazen, llama, topelorn
     W, H, G, D, F = SIZES[size]
     out = {}
     if "llama" in which:
@@ -38,6 +38,10 @@ def _models(size: str, device, which):
         cfg = dozazen.uniform_config(f"dozazen-{size}", LAYERS - 1, W, H, G, D, F, VOCAB, 8192,
                                      loop=(1, 2, 2), max_pos=8192)
         out["dozazen"] = dozazen.DozazenModel.random(cfg, device, seed=1)
+    if "topelorn" in which:
+        # attention and latent layers in turn, windows no shorter than Llama's spans here
+        cfg = topelorn.alternating_config(f"topelorn-{size}", LAYERS, W, H, G, D, F, VOCAB, max_pos=8192)
+        out["topelorn"] = topelorn.TopelornModel.random(cfg, device, seed=1)
     return out
 
 

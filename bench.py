@@ -78,7 +78,7 @@ def parse_args(argv=None):
     ap.add_argument("--overlap", type=float, default=0.0,
                     help="submit the next batch once this fraction of the current one is still "
                          "running (0: closed batches)")
-    ap.add_argument("--compare", choices=["dozazen"],
+    ap.add_argument("--compare", choices=["dozazen", "topelorn"],
                     help="instead of the headline workload: prefill and decode throughput of this "
                          "design's layers beside Llama's at equal sizes (utils/layerbench.py)")
     ap.add_argument("--compare-sizes", help="comma-separated sizes of --compare")
