@@ -51,8 +51,8 @@ DEV Run run_start(const MaskedAttnArgs& p, int head, bool sink, int fq) {
 }
 
 // the output factor of a row
-template <class T>
-DEV float head_gate(const MaskedAttnArgs& p, size_t tok, int head) {
+template <class T, class Args>
+DEV float head_gate(const Args& p, size_t tok, int head) {
   if (!p.gate) return 1.f;
   const float z = (float)((const T*)p.gate)[tok * p.gate_ld + head];
   return 1.f / (1.f + expf(-z));
@@ -103,42 +103,79 @@ DEV float tile_weights(f32x4 (&sacc)[4], bf16x8 (&pf)[2], Run& st, const ScoreCo
   return alpha;
 }
 
-// O^T += V^T P^T over one tile; Vl: [64][LD] with 16-B chunk swizzle ^= row & 7
-template <int DV, int LD = DV>
+// Addresses of a lane's fragments in a [64][LD] tile whose 16-B chunks are swizzled
+// by row & 7.  The swizzle only touches the low three bits of a chunk, so a few bases
+// and constant offsets reach everything.
+template <int LD>
+struct KeyFrag {                              // rows of K as MFMA operands
+  const bf16* p[2];
+  DEV KeyFrag(const bf16* Kl, int row, int fq) {
+#pragma unroll
+    for (int j = 0; j < 2; ++j) p[j] = Kl + row * LD + (((j * 4 + fq) ^ (row & 7)) << 3);
+  }
+  // 32 columns ``ks`` of a row ``down`` (a multiple of 8) below
+  DEV bf16x8 at(int down, int ks) const {
+    return *reinterpret_cast<const bf16x8*>(p[ks & 1] + down * LD + (ks >> 1) * 64);
+  }
+};
+template <int LD, int NB = 4>
+struct ValFrag {                              // V^T through transposed reads
+  const bf16* p[NB];                          // 16-column tiles dt0 + 0 .. NB - 1 (mod 4)
+  DEV ValFrag(const bf16* Vl, int lane, int dt0 = 0) {
+    const int key = (lane >> 4) * 4 + ((lane & 15) >> 2), tp = lane & 3;
+#pragma unroll
+    for (int j = 0; j < NB; ++j)
+      p[j] = Vl + key * LD + (((((dt0 + j) & 3) * 2 + (tp >> 1)) ^ (key & 7)) << 3) + (tp & 1) * 4;
+  }
+  // keys 32 k2 + 4 fq .. + 3 and 16 further, base j, ``cols`` (a multiple of 64) columns on
+  DEV bf16x8 at(int j, int k2, int cols) const {
+    const bf16* q = p[j] + k2 * 32 * LD + cols;
+    const bf16x4 v0 = tr_read(q), v1 = tr_read(q + 16 * LD);
+    return bf16x8{v0[0], v0[1], v0[2], v0[3], v1[0], v1[1], v1[2], v1[3]};
+  }
+};
+
+// O^T += V^T P^T over one tile; Vl: [64][DV] with 16-B chunk swizzle ^= row & 7
+template <int DV>
 DEV void tile_pv(const bf16* Vl, const bf16x8 (&pf)[2], f32x4 (&o)[DV / 16], int lane) {
-  const int fq = lane >> 4, tq = (lane & 15) >> 2, tp = lane & 3;
+  const ValFrag<DV> vf(Vl, lane);
 #pragma unroll
-  for (int dt = 0; dt < DV / 16; ++dt) {
-    const int chunk = dt * 2 + (tp >> 1), half = (tp & 1) * 4;
+  for (int dt = 0; dt < DV / 16; ++dt)
 #pragma unroll
-    for (int k2 = 0; k2 < 2; ++k2) {
-      const int key0 = k2 * 32 + fq * 4 + tq;
-      const int key1 = key0 + 16;
-      const bf16x4 v0 = tr_read(Vl + key0 * LD + ((chunk ^ (key0 & 7)) << 3) + half);
-      const bf16x4 v1 = tr_read(Vl + key1 * LD + ((chunk ^ (key1 & 7)) << 3) + half);
-      const bf16x8 vf = bf16x8{v0[0], v0[1], v0[2], v0[3], v1[0], v1[1], v1[2], v1[3]};
-      o[dt] = mfma16x16x32(vf, pf[k2], o[dt]);
+    for (int k2 = 0; k2 < 2; ++k2) o[dt] = mfma16x16x32(vf.at(dt & 3, k2, (dt >> 2) * 64), pf[k2], o[dt]);
+}
+
+// LDS-DMA of pieces [first, first + P1) (1 KiB each) of a [64][D] block, swizzled;
+// D / 64 pieces are 8 rows, so their lane offsets repeat from there
+template <int D, int P0, int P1>
+DEV void stage_rows(const bf16* src, bf16* dst, int first, int lane) {
+  constexpr int NC = D / 8, M = D / 64;       // 16-B chunks per row, pieces per 8 rows
+  if constexpr (P1 % M == 0 && P0 == 0) {     // whole 8-row groups (``first`` is one, too)
+    const char* base = (const char*)(src + (first / M) * 8 * D);
+    unsigned off[M];
+#pragma unroll
+    for (int j = 0; j < M; ++j) {
+      const int c = j * 64 + lane, row = c / NC, chunk = c % NC;
+      off[j] = (row * D + ((chunk ^ (row & 7)) << 3)) * 2;
+    }
+#pragma unroll
+    for (int i = 0; i < P1; ++i)
+      glds16(base + (i / M) * 8 * D * 2 + off[i % M], dst + (first + i) * 512);
+  } else {
+#pragma unroll
+    for (int i = P0; i < P1; ++i) {
+      const int p = first + i;
+      const int c = p * 64 + lane;
+      const int row = c / NC, chunk = c % NC;
+      glds16(src + row * D + ((chunk ^ (row & 7)) << 3), dst + p * 512);
     }
   }
 }
 
-// LDS-DMA of pieces [p0, p1) (1 KiB each) of a [64][D] block, swizzled
-template <int D, int P0, int P1>
-DEV void stage_rows(const bf16* src, bf16* dst, int first, int lane) {
-  constexpr int NC = D / 8;                   // 16-B chunks per row
-#pragma unroll
-  for (int i = P0; i < P1; ++i) {
-    const int p = first + i;
-    const int c = p * 64 + lane;
-    const int row = c / NC, chunk = c % NC;
-    glds16(src + row * D + ((chunk ^ (row & 7)) << 3), dst + p * 512);
-  }
-}
-
 // first key a query at ``pos`` sees (apart from the kept first ones)
+DEV int window_start(int window, int pos) { return window > 0 ? max(pos - window + 1, 0) : 0; }
 DEV int first_key(const MaskedAttnArgs& p, int pos) {
-  if (p.chunk > 0) return pos / p.chunk * p.chunk;
-  return p.window > 0 ? max(pos - p.window + 1, 0) : 0;
+  return p.chunk > 0 ? pos / p.chunk * p.chunk : window_start(p.window, pos);
 }
 
 // key tiles of rows whose first keys start at ``lo`` and whose last position is

@@ -157,6 +157,7 @@ void attn_tile_kernel(const MaskedAttnArgs a) {
 
   bf16* Kl = smem;
   bf16* Vl = smem + KT * DK;
+  const KeyFrag<DK> kfrag(Kl, fr, fq);
   const TileWalk walk(a, b_lo, b_hi);
   const int* bt = a.block_table + (size_t)s * a.max_blocks;
   int bt_v = 0;                                          // 64 table entries per load
@@ -179,12 +180,8 @@ void attn_tile_kernel(const MaskedAttnArgs a) {
 #pragma unroll
       for (int nt = 0; nt < 4; ++nt) {
         sacc[nt] = f32x4{0.f, 0.f, 0.f, 0.f};
-        const int kr = nt * 16 + fr;
 #pragma unroll
-        for (int ks = 0; ks < DK / 32; ++ks) {
-          const bf16x8 kf = *reinterpret_cast<const bf16x8*>(Kl + kr * DK + (((ks * 4 + fq) ^ (kr & 7)) << 3));
-          sacc[nt] = mfma16x16x32(kf, qf[ks], sacc[nt]);
-        }
+        for (int ks = 0; ks < DK / 32; ++ks) sacc[nt] = mfma16x16x32(kfrag.at(nt * 16, ks), qf[ks], sacc[nt]);
       }
       bf16x8 pf[2];
       const int lo = first - k_lo, hi = qpos - k_lo, keep = a.keep - k_lo;

@@ -884,15 +884,18 @@ void qk_norm_kv(const at::Tensor& z, const at::Tensor& slots, const at::Tensor& 
 
 void latent_qkv(const at::Tensor& z, const at::Tensor& pos, const at::Tensor& slots, const at::Tensor& cos_sin,
                 const at::Tensor& w_c, double eps, int64_t heads, int64_t dim, int64_t rot, int64_t rank,
-                int64_t rank_true, at::Tensor& q_out, at::Tensor& k_cache) {
+                int64_t rank_true, const c10::optional<at::Tensor>& q_out, at::Tensor& k_cache) {
   const int T = slots.numel();
-  check_rows(z, T, q_out.scalar_type(), "latent_qkv: z");
+  check_rows(z, T, k_cache.scalar_type(), "latent_qkv: z");
   CHECK_I32_TENSOR(pos); CHECK_I32_TENSOR(slots); CHECK_F32_TENSOR(cos_sin); CHECK_F32_TENSOR(w_c);
-  CHECK_TENSOR(q_out); CHECK_TENSOR(k_cache);
-  TORCH_CHECK(k_cache.scalar_type() == q_out.scalar_type(), "latent_qkv: one type");
-  TORCH_CHECK(q_out.dim() == 3 && q_out.size(0) == T && q_out.size(1) == heads && pos.numel() == T &&
-                  k_cache.dim() == 4 && k_cache.size(1) == 1 && k_cache.size(3) == q_out.size(2),
-              "latent_qkv: q_out [T, heads, DK], cache [nb, 1, BS, DK]");
+  CHECK_TENSOR(k_cache);
+  TORCH_CHECK(pos.numel() == T && k_cache.dim() == 4 && k_cache.size(1) == 1, "latent_qkv: cache [nb, 1, BS, DK]");
+  if (q_out.has_value()) {
+    CHECK_TENSOR((*q_out));
+    TORCH_CHECK(k_cache.scalar_type() == q_out->scalar_type(), "latent_qkv: one type");
+    TORCH_CHECK(q_out->dim() == 3 && q_out->size(0) == T && q_out->size(1) == heads &&
+                    k_cache.size(3) == q_out->size(2), "latent_qkv: q_out [T, heads, DK]");
+  }
   TORCH_CHECK(z.size(1) >= heads * (dim + rot) + rank + rot && w_c.numel() == rank && rank_true > 0 &&
                   rank_true <= rank, "latent_qkv: z [T, >= heads (dim + rot) + rank + rot], w_c [rank]");
   TORCH_CHECK(cos_sin.dim() == 3 && cos_sin.size(2) == 2, "cos_sin [P, pairs, 2]");
@@ -910,13 +913,83 @@ void latent_qkv(const at::Tensor& z, const at::Tensor& pos, const at::Tensor& sl
   a.rot = rot;
   a.rank = rank;
   a.rank_true = rank_true;
-  a.q_out = q_out.data_ptr();
+  a.q_out = q_out.has_value() ? q_out->data_ptr() : nullptr;
   a.k_cache = k_cache.data_ptr();
-  a.DK = q_out.size(2);
+  a.DK = k_cache.size(3);
   a.BS = k_cache.size(2);
   a.T = T;
-  TORCH_CHECK(launch_latent_rows(a, low_is_f32(q_out), stream()) == 0, "latent_qkv: sizes");
+  TORCH_CHECK(launch_latent_rows(a, low_is_f32(k_cache), stream()) == 0, "latent_qkv: sizes");
   check_launch("latent_qkv");
+}
+
+void latent_gather(const at::Tensor& cache, const at::Tensor& pages, const at::Tensor& valid, int64_t rank,
+                   at::Tensor& out) {
+  CHECK_BF16_TENSOR(cache); CHECK_I32_TENSOR(pages); CHECK_I32_TENSOR(valid); CHECK_BF16_TENSOR(out);
+  const int n = pages.numel(), BS = cache.size(2), DK = cache.size(3);
+  TORCH_CHECK(cache.dim() == 4 && cache.size(1) == 1 && valid.numel() == n && out.dim() == 2 &&
+                  out.size(0) == (int64_t)n * BS, "latent_gather: out [pages * BS, C]");
+  TORCH_CHECK(launch_latent_gather(cache.data_ptr(), pages.data_ptr<int>(), valid.data_ptr<int>(), n, DK, BS,
+                                   (int)rank, out.data_ptr(), out.size(1), stream()) == 0, "latent_gather: sizes");
+  check_launch("latent_gather");
+}
+
+void latent_prefill(const at::Tensor& z, const at::Tensor& pos, const at::Tensor& cos_sin, int64_t heads,
+                    int64_t dim, int64_t rot, const at::Tensor& exp, const at::Tensor& key0,
+                    const at::Tensor& cache, int64_t rank, const at::Tensor& q_start, const at::Tensor& q_len,
+                    const at::Tensor& ctx_len, const at::Tensor& block_table, const at::Tensor& item_seq,
+                    const at::Tensor& item_q0, int64_t DK, double scale, int64_t window,
+                    const c10::optional<at::Tensor>& gate, at::Tensor& out) {
+  const int T = pos.numel();
+  check_rows(z, T, at::kBFloat16, "latent_prefill: z");
+  CHECK_I32_TENSOR(pos); CHECK_F32_TENSOR(cos_sin); CHECK_BF16_TENSOR(exp); CHECK_I32_TENSOR(key0);
+  CHECK_BF16_TENSOR(cache); CHECK_I32_TENSOR(q_start); CHECK_I32_TENSOR(q_len); CHECK_I32_TENSOR(ctx_len);
+  CHECK_I32_TENSOR(block_table); CHECK_I32_TENSOR(item_seq); CHECK_I32_TENSOR(item_q0); CHECK_BF16_TENSOR(out);
+  const int S = q_len.numel();
+  TORCH_CHECK(out.dim() == 3 && out.size(0) == T && out.size(1) == heads, "latent_prefill: out [T, heads, DV]");
+  TORCH_CHECK(z.size(1) >= heads * (dim + rot) && z.stride(0) % 8 == 0, "latent_prefill: z [T, >= heads (dim + rot)]");
+  TORCH_CHECK(exp.dim() == 2 && exp.size(1) == heads * (dim + out.size(2)), "latent_prefill: exp [keys, heads (dim + DV)]");
+  TORCH_CHECK(cache.dim() == 4 && cache.size(1) == 1 && cache.size(2) == 64 && rank + rot <= cache.size(3),
+              "latent_prefill: cache [nb, 1, 64, >= rank + rot]");
+  TORCH_CHECK(key0.numel() == S && q_start.numel() == S && ctx_len.numel() == S && block_table.dim() == 2 &&
+                  block_table.size(0) == S && item_seq.numel() == item_q0.numel(), "latent_prefill: per-sequence arrays");
+  TORCH_CHECK(cos_sin.dim() == 3 && cos_sin.size(2) == 2 && window >= 0, "cos_sin [P, pairs, 2]");
+  LatentPrefillArgs a{};
+  a.z = z.data_ptr();
+  a.ldz = z.stride(0);
+  a.pos = pos.data_ptr<int>();
+  a.cos_sin = cos_sin.data_ptr<float>();
+  a.pairs = cos_sin.size(1);
+  a.dim = dim;
+  a.rot = rot;
+  a.exp = exp.data_ptr();
+  a.lde = exp.size(1);
+  a.key0 = key0.data_ptr<int>();
+  a.cache = cache.data_ptr();
+  a.ldc = cache.size(3);
+  a.rank = rank;
+  a.q_start = q_start.data_ptr<int>();
+  a.q_len = q_len.data_ptr<int>();
+  a.ctx_len = ctx_len.data_ptr<int>();
+  a.block_table = block_table.data_ptr<int>();
+  a.max_blocks = block_table.size(1);
+  a.item_seq = item_seq.data_ptr<int>();
+  a.item_q0 = item_q0.data_ptr<int>();
+  a.items = item_seq.numel();
+  a.H = heads;
+  a.DK = DK;
+  a.DV = out.size(2);
+  a.scale = (float)scale;
+  a.window = window;
+  if (gate.has_value()) {
+    check_rows(*gate, T, at::kBFloat16, "latent_prefill: gate");
+    TORCH_CHECK(gate->size(1) == heads, "gate [T, heads]");
+    a.gate = gate->data_ptr();
+    a.gate_ld = gate->stride(0);
+  }
+  a.out = out.data_ptr();
+  const int rc = launch_attn_latent_prefill(a, stream());
+  TORCH_CHECK(rc == 0, "latent_prefill: sizes (code ", rc, ")");
+  check_launch("latent_prefill");
 }
 
 void gemm_heads(const at::Tensor& X, const at::Tensor& W, at::Tensor& out) {
@@ -1017,7 +1090,8 @@ bool attention_masked(const at::Tensor& q, const at::Tensor& k_cache, const c10:
                       int64_t window, int64_t keep, const c10::optional<at::Tensor>& slopes,
                       const c10::optional<at::Tensor>& sinks, const c10::optional<at::Tensor>& gate,
                       int64_t nz, const c10::optional<at::Tensor>& split_o,
-                      const c10::optional<at::Tensor>& split_ml) {
+                      const c10::optional<at::Tensor>& split_ml, int64_t skip_q) {
+  TORCH_CHECK(skip_q == 0 || !v_cache.has_value(), "attention_masked: skip_q is the latent form's");
   MaskedAttnArgs a = masked_args(q, k_cache, v_cache, out, q_start, q_len, ctx_len, block_table,
                                  scale, cap, chunk, sink, window, keep, slopes, sinks, gate);
   CHECK_BF16(q); CHECK_I32_TENSOR(work_seq); CHECK_I32_TENSOR(work_q0);
@@ -1026,6 +1100,7 @@ bool attention_masked(const at::Tensor& q, const at::Tensor& k_cache, const c10:
   a.work_q0 = work_q0.data_ptr<int>();
   a.item_tokens = (int)item_tokens;
   a.rows = (int)(q.size(0) * q.size(1));
+  a.skip_q = (int)skip_q;
   if (nz > 1) {
     TORCH_CHECK(split_o.has_value() && split_ml.has_value(), "attention_masked: split buffers");
     CHECK_F32_TENSOR((*split_o)); CHECK_F32_TENSOR((*split_ml));
@@ -1304,6 +1379,9 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("gemm_f32", &gemm_f32, py::arg("X"), py::arg("W"), py::arg("Y"), py::arg("R") = py::none());
   m.def("qk_norm_kv", &qk_norm_kv);
   m.def("latent_qkv", &latent_qkv);
+  m.def("latent_gather", &latent_gather);
+  m.def("latent_prefill", &latent_prefill);
+  m.attr("LATENT_ITEM") = LATENT_ITEM;
   m.def("gemm_heads", &gemm_heads);
   m.def("gated_act_f32", &gated_act_f32);
   m.def("rope_kv_any", &rope_kv_any);
@@ -1313,7 +1391,7 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
         py::arg("work_seq"), py::arg("work_q0"), py::arg("form"), py::arg("item_tokens"),
         py::arg("scale"), py::arg("cap"), py::arg("chunk"), py::arg("sink"), py::arg("window"),
         py::arg("keep"), py::arg("slopes"), py::arg("sinks"), py::arg("gate"), py::arg("nz") = 1,
-        py::arg("split_o") = py::none(), py::arg("split_ml") = py::none());
+        py::arg("split_o") = py::none(), py::arg("split_ml") = py::none(), py::arg("skip_q") = 0);
   m.def("branch_select", &branch_select);
   m.def("add_inplace", &add_inplace);
   m.def("paged_attention_decode_oproj", &paged_attention_decode_oproj,

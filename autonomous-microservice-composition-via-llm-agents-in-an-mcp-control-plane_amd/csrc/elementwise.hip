@@ -1,6 +1,7 @@
 // Memory-bound kernels of the Llama-3 forward (SURVEY §2.6 K3, K4+K10, K7, K8).
 // All loads/stores are 16 B per lane (bf16x8), cdna_hip_programming.md Guideline 13.
 #include "common.h"
+#include "rows.h"
 #include "kernels.h"
 
 // ---------------------------------------------------------------- K3 RMSNorm
@@ -288,31 +289,6 @@ void launch_copy_blocks(void* data, const int* src, const int* dst, int npairs, 
 // (dimension j with j + DK / 2; cos_sin [max_pos, DK / 2] float2 holds the
 // identity for pairs that do not rotate), values pass.  One thread per 16
 // elements: 8 + 8 of a q / k head, 2 x 8 of a v head.
-DEV void load8(const bf16* p, float (&v)[8]) {
-  const bf16x8 x = *reinterpret_cast<const bf16x8*>(p);
-#pragma unroll
-  for (int j = 0; j < 8; ++j) v[j] = (float)x[j];
-}
-DEV void load8(const float* p, float (&v)[8]) {
-#pragma unroll
-  for (int h = 0; h < 2; ++h) {
-    const f32x4 x = reinterpret_cast<const f32x4*>(p)[h];
-#pragma unroll
-    for (int j = 0; j < 4; ++j) v[4 * h + j] = x[j];
-  }
-}
-DEV void store8(bf16* p, const float (&v)[8]) {
-  bf16x8 x;
-#pragma unroll
-  for (int j = 0; j < 8; ++j) x[j] = (bf16)v[j];
-  *reinterpret_cast<bf16x8*>(p) = x;
-}
-DEV void store8(float* p, const float (&v)[8]) {
-#pragma unroll
-  for (int h = 0; h < 2; ++h)
-    reinterpret_cast<f32x4*>(p)[h] = f32x4{v[4 * h], v[4 * h + 1], v[4 * h + 2], v[4 * h + 3]};
-}
-
 template <class T>
 __global__ __launch_bounds__(256) void rope_kv_any_kernel(
     const T* __restrict__ qkv, const float* __restrict__ bias, const int* __restrict__ pos,

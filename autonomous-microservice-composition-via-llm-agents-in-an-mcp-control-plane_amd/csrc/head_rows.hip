@@ -1,35 +1,10 @@
 // Projected rows -> queries and paged cache, for attention whose heads are normed
 // after the projection and for latent attention.  T is bf16, or float in the
 // 32-bit mode; norms, rotation and value mixing are fp32.
-#include "common.h"
+#include "rows.h"
 #include "kernels.h"
 
 namespace {
-
-DEV void load8(const bf16* p, float (&v)[8]) {
-  const bf16x8 x = *reinterpret_cast<const bf16x8*>(p);
-#pragma unroll
-  for (int j = 0; j < 8; ++j) v[j] = (float)x[j];
-}
-DEV void load8(const float* p, float (&v)[8]) {
-#pragma unroll
-  for (int h = 0; h < 2; ++h) {
-    const f32x4 x = reinterpret_cast<const f32x4*>(p)[h];
-#pragma unroll
-    for (int j = 0; j < 4; ++j) v[4 * h + j] = x[j];
-  }
-}
-DEV void store8(bf16* p, const float (&v)[8]) {
-  bf16x8 x;
-#pragma unroll
-  for (int j = 0; j < 8; ++j) x[j] = (bf16)v[j];
-  *reinterpret_cast<bf16x8*>(p) = x;
-}
-DEV void store8(float* p, const float (&v)[8]) {
-#pragma unroll
-  for (int h = 0; h < 2; ++h)
-    reinterpret_cast<f32x4*>(p)[h] = f32x4{v[4 * h], v[4 * h + 1], v[4 * h + 2], v[4 * h + 3]};
-}
 
 // ---- rms norm of every q / k head, value mixing, cache write.  LG lanes per
 // (token, head), 8 elements a lane and step, at most NCH steps.
@@ -117,42 +92,13 @@ int qk_norm_kv_dispatch(const T* z, int ldz, const int* slots, const float* wq, 
 // 0] and the queries' rotated parts.  One block per token; wave 0 takes the row,
 // the others the heads.
 template <class T>
-DEV float rotated(const T* __restrict__ p, const float* __restrict__ cs, int pairs, int rot, int d) {
-  if (d < pairs) return (float)p[d] * cs[2 * d] - (float)p[d + pairs] * cs[2 * d + 1];
-  if (d < 2 * pairs) {
-    const int e = d - pairs;
-    return (float)p[d] * cs[2 * e] + (float)p[e] * cs[2 * e + 1];
-  }
-  return d < rot ? (float)p[d] : 0.f;
-}
-// 8 elements from d on; halves that are multiples of 8 go by vectors
-template <class T>
-DEV void rotated8(const T* __restrict__ p, const float* __restrict__ cs, int pairs, int rot, int d,
-                  float (&v)[8]) {
-  if (pairs % 8 || d >= 2 * pairs) {
-#pragma unroll
-    for (int j = 0; j < 8; ++j) v[j] = rotated(p, cs, pairs, rot, d + j);
-    return;
-  }
-  const bool second = d >= pairs;
-  const int e = second ? d - pairs : d;
-  float a[8], b[8];
-  load8(p + e, a);
-  load8(p + e + pairs, b);
-#pragma unroll
-  for (int j = 0; j < 8; ++j) {
-    const float c = cs[2 * (e + j)], s = cs[2 * (e + j) + 1];
-    v[j] = second ? b[j] * c + a[j] * s : a[j] * c - b[j] * s;
-  }
-}
-
-template <class T>
 __global__ __launch_bounds__(256) void latent_rows_kernel(const LatentRowArgs a) {
   const int t = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const T* z = (const T*)a.z + (size_t)t * a.ldz;
   const float* cs = a.cos_sin + (size_t)a.pos[t] * a.pairs * 2;
   const int qs = a.dim + a.rot, tail = (a.DK - a.rank) / 8;
   if (wave) {
+    if (!a.q_out) return;
     for (int i = threadIdx.x - 64; i < a.heads * tail; i += 192) {
       const int h = i / tail, d = (i % tail) * 8;
       float v[8];
@@ -188,7 +134,30 @@ __global__ __launch_bounds__(256) void latent_rows_kernel(const LatentRowArgs a)
   }
 }
 
+// the latents of cached pages as plain rows: out [pages * BS, ldo], columns from
+// ``rank`` on and rows from a page's ``valid`` on zero
+__global__ __launch_bounds__(256) void latent_gather_kernel(const bf16* __restrict__ cache,
+                                                            const int* __restrict__ pages,
+                                                            const int* __restrict__ valid, int DK, int BS,
+                                                            int rank, bf16* __restrict__ out, int ldo) {
+  const int nc = ldo / 8, page = pages[blockIdx.x], n = valid[blockIdx.x];
+  for (int i = threadIdx.x; i < BS * nc; i += 256) {
+    const int r = i / nc, c = (i % nc) * 8;
+    bf16x8 v = {};
+    if (r < n && c < rank) v = *reinterpret_cast<const bf16x8*>(cache + ((size_t)page * BS + r) * DK + c);
+    *reinterpret_cast<bf16x8*>(out + ((size_t)blockIdx.x * BS + r) * ldo + c) = v;
+  }
+}
+
 }  // namespace
+
+int launch_latent_gather(const void* cache, const int* pages, const int* valid, int n, int DK, int BS,
+                         int rank, void* out, int ldo, hipStream_t s) {
+  if (n <= 0) return 0;
+  if (DK % 8 || rank % 8 || ldo % 8 || rank > DK || rank > ldo) return 1;
+  latent_gather_kernel<<<n, 256, 0, s>>>((const bf16*)cache, pages, valid, DK, BS, rank, (bf16*)out, ldo);
+  return 0;
+}
 
 int launch_qk_norm_kv(const void* z, int ldz, const int* slots, const float* wq, const float* wk,
                       int dim, float eps, void* q_out, void* k_cache, void* v_cache,

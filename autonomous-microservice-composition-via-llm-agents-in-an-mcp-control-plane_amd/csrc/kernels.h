@@ -67,11 +67,13 @@ struct LatentRowArgs {
   const float* w_c;          // [rank]
   float eps;
   int heads, dim, rot, rank, rank_true;
-  void* q_out;               // [T, heads, DK], columns from rank on are written
+  void* q_out;               // [T, heads, DK], columns from rank on are written; null: none
   void* k_cache;             // [nb, 1, BS, DK]
   int DK, BS, T;
 };
 int launch_latent_rows(const LatentRowArgs& a, bool f32, hipStream_t s);
+int launch_latent_gather(const void* cache, const int* pages, const int* valid, int n, int DK, int BS,
+                         int rank, void* out, int ldo, hipStream_t s);
 
 // gemm_heads.hip: one product per head, out[t, h, n] = sum_k X[t, h, k] W[h, n, k];
 // strides in elements, inner stride 1
@@ -128,10 +130,40 @@ struct MaskedAttnArgs {
   float* split_ml;
   int rows;
   int* tickets;              // set by the launcher
+  int skip_q;                // > 0: sequences with this many new tokens are somebody else's (latent form)
 };
 int launch_attn_masked(const MaskedAttnArgs& a, int nwork, int form, int nz, hipStream_t s);
 // values are the first DV columns of the keys (vc is not read); either work list
 int launch_attn_latent(const MaskedAttnArgs& a, int nwork, int nz, hipStream_t s);
+// long prompt portions of latent attention: keys and values per head from expanded
+// rows [dim | DV] of every key, the rotated key part from the cache
+struct LatentPrefillArgs {
+  const void* z;             // [T, ldz] projections, per head [dim | rot] first
+  int ldz;
+  const int* pos;
+  const float* cos_sin;      // [P, pairs, 2]
+  int pairs, dim, rot;
+  const void* exp;           // [keys, lde]: per head [dim | DV]
+  long long lde;
+  const int* key0;           // [S] row of exp that holds the sequence's key 0
+  const void* cache;         // [nb, 1, 64, ldc], the rotated key part from column rank on
+  int ldc, rank;
+  const int* q_start;
+  const int* q_len;
+  const int* ctx_len;
+  const int* block_table;
+  int max_blocks;
+  const int* item_seq;       // items of LATENT_ITEM tokens
+  const int* item_q0;
+  int items, H, DK, DV;      // DK: key size the kernel runs at, >= dim + rot
+  float scale;
+  int window;
+  const void* gate;
+  int gate_ld;
+  void* out;                 // [T, H, DV]
+};
+constexpr int LATENT_ITEM = 128;
+int launch_attn_latent_prefill(const LatentPrefillArgs& a, hipStream_t s);
 constexpr int ATTN_SPLIT_TICKETS = 1 << 16;
 int* attn_split_counters();  // this device's tickets, zero between launches (attention.hip)
 // vc null: values are the first DV columns of the keys

@@ -47,6 +47,9 @@ class AttnMeta:
     # longest own key span of the step in 64-key tiles (keys after the cascade
     # prefix); 0 = unknown (hipGraph layouts)
     own_tiles: int = 0
+    # the step's host-side arrays (eagerly launched steps), for models that plan
+    # launches by span length (``long_spans``)
+    host: Optional["StepInputs"] = None
 
     def work_lists(self):
         return self.work
@@ -185,6 +188,7 @@ class StepInputs:
     allow_ptr: Optional[np.ndarray] = None  # [R+1] sampling: CSR of grammar-allowed tokens
     allow_ids: Optional[np.ndarray] = None  # [A]
     sample_ctr: Optional[np.ndarray] = None  # [R] RNG counters
+    plans: dict = dataclasses.field(default_factory=dict)   # by whoever plans launches from it
 
     @property
     def num_tokens(self) -> int:
@@ -201,6 +205,50 @@ class DeviceStep:
     allow_ptr: Optional[torch.Tensor] = None
     allow_ids: Optional[torch.Tensor] = None
     sample_ctr: Optional[torch.Tensor] = None
+
+
+@dataclasses.dataclass
+class SpanPlan:
+    """The long query spans of a step and the pages their keys are in."""
+    pages: torch.Tensor        # [P] int32 physical blocks, sequence by sequence
+    valid: torch.Tensor        # [P] keys of the sequence in each
+    key0: torch.Tensor         # [S] row of a sequence's key 0 among the P * 64 gathered keys
+    item_seq: torch.Tensor     # work items, the ones with most keys first
+    item_q0: torch.Tensor
+    rest: Optional[tuple]      # [first, last) token around all other spans; None: there are none
+
+
+def long_spans(step: StepInputs, min_tokens: int, window: int, item_tokens: int, device) -> Optional[SpanPlan]:
+    """``SpanPlan`` of the spans of ``min_tokens`` or more, whose queries see
+    ``window`` keys (0: all); None without any."""
+    ql, cl = step.q_len, step.ctx_len
+    long = np.nonzero(ql >= min_tokens)[0]
+    if not len(long):
+        return None
+    key0 = np.zeros(len(ql), np.int32)
+    pages, valid, items, at = [], [], [], 0
+    for s in long.tolist():
+        n, ctx = int(ql[s]), int(cl[s])
+        start = ctx - n
+        k0 = max(start - window + 1, 0) // BLOCK_SIZE if window else 0
+        k1 = -(-ctx // BLOCK_SIZE)
+        pages.append(step.block_table[s, k0:k1])
+        valid.append(np.minimum(ctx - np.arange(k0, k1) * BLOCK_SIZE, BLOCK_SIZE))
+        key0[s] = (at - k0) * BLOCK_SIZE
+        at += k1 - k0
+        for q0 in range(0, n, item_tokens):
+            last = start + min(q0 + item_tokens, n) - 1
+            items.append((last // BLOCK_SIZE - (max(start + q0 - window + 1, 0) // BLOCK_SIZE if window else 0), s, q0))
+    items.sort(key=lambda t: -t[0])
+    other = np.nonzero((ql > 0) & (ql < min_tokens))[0]
+    rest = None
+    if len(other):
+        first = step.q_start[other]
+        rest = int(first.min()), int((first + ql[other]).max())
+    parts = [np.concatenate(pages), np.concatenate(valid), key0, np.asarray([i[1] for i in items]),
+             np.asarray([i[2] for i in items])]
+    dev = to_device(np.concatenate(parts).astype(np.int32), device)
+    return SpanPlan(*torch.split(dev, [len(p) for p in parts]), rest)
 
 
 def pack_host(step: StepInputs, group: int, copies=()):

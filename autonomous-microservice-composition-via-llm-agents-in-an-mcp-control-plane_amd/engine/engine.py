@@ -1355,7 +1355,9 @@ class LLMEngine:
             self.bcast.send(payload, layout)
         dstep, csrc, cdst = views(payload, layout)
         if pre is not None:
-            pre(dstep)
+            pre(dstep)                     # (the device arrays change: no host copy)
+        elif getattr(self.model, "uses_host_step", False):
+            dstep.attn.host = step_from_host(host, layout)
         if csrc.numel():
             self.kv.copy_blocks(csrc, cdst)
         if dstep.token_ids.numel() == 0:

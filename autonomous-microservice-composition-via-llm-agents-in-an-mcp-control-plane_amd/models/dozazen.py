@@ -17,7 +17,7 @@ One ragged, paged step (n = rms norm with its own weight, c(z; k) = k tanh(z / k
 What this module adds to the shared machinery is the mapping onto it:
 
 * every size is padded to what the MFMA kernels tile by (width and feed-forward
-  to 64, head sizes to ``packing.HEAD_SIZES``) with zero rows / columns, which is exact;
+  to 64, head sizes to ``ops.HEAD_SIZES``) with zero rows / columns, which is exact;
 * neighbouring-pair rotation becomes the kernels' half rotation by permuting the
   rows of Wq / Wk (the same permutation on both leaves q . k unchanged); pairs
   that do not rotate (partial rotation, padding) hold (1, 0) in the table;

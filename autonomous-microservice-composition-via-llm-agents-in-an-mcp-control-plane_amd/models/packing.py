@@ -8,9 +8,8 @@ from typing import Optional, Tuple
 
 import torch
 
-from ..ops import reference as ref
+from ..ops import HEAD_SIZES, reference as ref
 
-HEAD_SIZES = (64, 128, 192, 256)
 MAX_POS = 131072          # positions of the rotation tables when nothing else bounds them
 
 

@@ -23,9 +23,12 @@ How it maps onto the shared machinery:
 
 * all projections of h that feed the mixer, the head gates included, are ONE
   product (``w_in``); one kernel norms heads, mixes values and writes the cache;
-* latent layers run absorbed: (Wuk^T qn) . c and Wuv (sum p c), one product per
-  head on either side (``ops.gemm_heads``), so attention reads the cached rows
-  as they are, keys and values at once, one key head for all query heads;
+* latent layers cache [c | r] and nothing else.  Decoding and short portions run
+  absorbed: (Wuk^T qn) . c and Wuv (sum p c), one product per head on either side
+  (``ops.gemm_heads``), attention on the cached rows as they are, keys and values
+  at once, one key head for all query heads.  Long portions expand the latents of
+  the keys they see (one product) and run plain attention per head
+  (``ops.latent_prefill``): less arithmetic once enough queries share a key;
 * the feed-forward's down product takes the mixer's output as its residual, so a
   layer adds one vector to the stream, in the pass that also norms it for the
   next layer (``ops.residual_norm``);
@@ -43,6 +46,7 @@ from typing import Dict, List, Optional, Tuple, Union
 import torch
 
 from .. import ops
+from ..engine.batch import long_spans
 from ..ops import reference as ref
 from .llama import padded_group
 from .packing import MAX_POS, Rotary, head_size, leading, pad, pick_rows, rope_table, up
@@ -107,8 +111,12 @@ class LatentAttention:
 
     @property
     def vdim_p(self) -> int:
-        m = next(m for m in (16, 32, 64) if self.heads * m % 64 == 0)
-        return up(self.vdim, m)
+        return head_size(self.vdim)
+
+    @property
+    def expands(self) -> bool:
+        """Keys and values of a head fit the expanded form."""
+        return max(self.dim_p + self.rot_p, self.vdim_p) <= ops.MASKED_MAX_HEAD
 
     @property
     def kv_spec(self):
@@ -248,6 +256,7 @@ class TopelornLayer:
     c_norm: Optional[torch.Tensor] = None  # fp32 [latent]
     w_uk: Optional[torch.Tensor] = None    # [H, latent, dim]: the absorbed query's product
     w_uv: Optional[torch.Tensor] = None    # [H, value size, DV]
+    w_ukv: Optional[torch.Tensor] = None   # [H (dim + value size), latent to 64]: expands latents
 
 
 @dataclasses.dataclass
@@ -293,6 +302,10 @@ def pack_weights(cfg: TopelornConfig, get, device, dtype=torch.bfloat16) -> Tope
             kw = dict(c_norm=vec(p + "mix.dkv.norm", m.rank_p),
                       w_uk=put(pad(uk, m.heads, m.rank_p, m.dim_p)),
                       w_uv=put(pad(uv, m.heads, m.vdim_p, m.row[1])))
+            if m.expands and dtype == torch.bfloat16:
+                k64 = up(m.rank_p, 64)
+                ukv = torch.cat([pad(uk.transpose(1, 2), m.heads, m.dim_p, k64), pad(uv, m.heads, m.vdim_p, k64)], 1)
+                kw["w_ukv"] = put(ukv.reshape(-1, k64))
         else:
             qk, vo = leading(m.dim, m.dk), leading(m.vdim, m.dv)
             rows = [pick_rows(get(p + "mix.q"), m.heads, m.dim, qk),
@@ -365,6 +378,8 @@ class TopelornModel:
     tp = 1
     tp_rank = 0
     supports_cascade = False      # a shared prefix leaves the window as a request goes on
+    uses_host_step = True         # spans this long expand the latents they see
+    EXPAND_MIN, EXPAND_MAX_BYTES = 256, 4 << 30
     logit_scale, logit_cap = 1.0, 0.0
 
     def __init__(self, cfg: TopelornConfig, weights: TopelornWeights, device):
@@ -414,12 +429,12 @@ class TopelornModel:
             if tap is not None and i:
                 tap(i - 1, x[:, :W])
             z = ops.gemm(h, lw.w_in)
-            q, v = (self._latent_rows if s.latent else self._rows)(i, z, step, kv, v_first)
+            a, v = (self._latent if s.latent else self._attention)(
+                i, z, step, kv, v_first, last and rows.numel() == 0 and tap is None)
+            if a is None:
+                return h.new_empty(0, h.shape[1])      # every key is in the cache; nothing is read
             if i == self.first:
                 v_first = v
-            if last and rows.numel() == 0 and tap is None:
-                return h.new_empty(0, h.shape[1])      # every key is in the cache; nothing is read
-            a = self._attend(i, z, q, step, kv)
             if last and tap is None:                   # only the asked-for rows go on
                 ri = rows.long()
                 x, h, a = x.index_select(0, ri), h.index_select(0, ri), a.index_select(0, ri)
@@ -432,43 +447,66 @@ class TopelornModel:
             h = h.index_select(0, rows.long())
         return h
 
-    def _rows(self, i, z, step, kv, v_first):
-        """Attention layer: queries, and the projected values; keys and values
-        are in the cache."""
-        m, lw = self.cfg.layer_specs[i].mixer, self.w.layers[i]
+    def _gates(self, m, z):
+        return z[:, z.shape[1] - up(m.heads, 16):][:, :m.heads]
+
+    def _attention(self, i, z, step, kv, v_first, cache_only):
+        """([T, heads * value size] gated outputs, the projected values) of an
+        attention layer on its projected rows ``z``."""
+        m, lw, T = self.cfg.layer_specs[i].mixer, self.w.layers[i], z.shape[0]
         kc, vc = kv.layer(i)
-        q = torch.empty(z.shape[0], m.heads, m.dk, device=self.device, dtype=self.dtype)
-        at = (m.heads + m.kv_heads) * m.dk
+        q = torch.empty(T, m.heads, m.dk, device=self.device, dtype=self.dtype)
         ops.qk_norm_kv(z, step.slots, lw.q_norm, lw.k_norm, m.dim, self.cfg.eps, q, kc, vc,
                        v_first if m.v_mix else None, lw.lam)
-        return q, z[:, at:at + m.kv_heads * m.dv]
+        if cache_only:
+            return None, None
+        a = ops.masked_attention(q, kc, vc, step.attn, m.scale, self.cfg.group, sink=lw.sinks, window=m.window,
+                                 keep_first=m.keep_first, slopes=self.slopes[i], gate=self._gates(m, z),
+                                 max_splits=max(1, int(step.attn.kv_splits) * self.hkv // m.kv_heads))
+        at = (m.heads + m.kv_heads) * m.dk
+        return a.view(T, -1), z[:, at:at + m.kv_heads * m.dv]
 
-    def _latent_rows(self, i, z, step, kv, v_first):
-        """Latent layer: absorbed queries [Wuk^T q | rotated q]; the token's row
-        is in the cache."""
-        m, lw = self.cfg.layer_specs[i].mixer, self.w.layers[i]
+    def _latent(self, i, z, step, kv, v_first, cache_only):
+        """(gated outputs, None) of a latent layer."""
+        m, lw, T = self.cfg.layer_specs[i].mixer, self.w.layers[i], z.shape[0]
         kc, _ = kv.layer(i)
-        T, per = z.shape[0], m.dim_p + m.rot_p
-        q = torch.empty(T, m.heads, m.row[0], device=self.device, dtype=self.dtype)
+        plan = self._plan(i, step)
+        lo, hi = (0, T) if plan is None else plan.rest or (0, 0)      # tokens that run absorbed
+        q = torch.empty(T, m.heads, m.row[0], device=self.device, dtype=self.dtype) \
+            if hi > lo and not cache_only else None
         ops.latent_qkv(z, step.positions, step.slots, self.cos_sin[i], lw.c_norm, self.cfg.eps, m.heads,
                        m.dim_p, m.rot_p, m.rank_p, m.kv_rank, q, kc)
-        ops.gemm_heads(z[:, :m.heads * per].view(T, m.heads, per)[..., :m.dim_p], lw.w_uk, q[..., :m.rank_p])
-        return q, None
+        if cache_only:
+            return None, None
+        out = torch.empty(T, m.heads, m.vdim_p, device=self.device, dtype=self.dtype)
+        if q is not None:
+            per = m.dim_p + m.rot_p
+            qn = z[:, :m.heads * per].view(T, m.heads, per)[..., :m.dim_p]
+            ops.gemm_heads(qn[lo:hi], lw.w_uk, q[lo:hi, :, :m.rank_p])
+            a = ops.masked_attention(q, kc, None, step.attn, m.scale, self.cfg.group, window=m.window,
+                                     gate=self._gates(m, z), v_dim=m.row[1],
+                                     skip_q=0 if plan is None else self.EXPAND_MIN)
+            ops.gemm_heads(a[lo:hi], lw.w_uv, out[lo:hi])
+        if plan is not None:
+            c = torch.empty(plan.pages.numel() * kc.shape[2], lw.w_ukv.shape[1], device=self.device, dtype=self.dtype)
+            ops.latent_gather(kc, plan.pages, plan.valid, m.rank_p, c)
+            ops.latent_prefill(z, step.attn, plan, step.positions, self.cos_sin[i], m.heads, m.dim_p, m.rot_p,
+                               ops.gemm(c, lw.w_ukv), kc, m.rank_p, m.scale, m.window, self._gates(m, z), out)
+        return out.view(T, -1), None
 
-    def _attend(self, i, z, q, step, kv):
-        """[T, heads * value size] gated attention outputs."""
-        m, lw = self.cfg.layer_specs[i].mixer, self.w.layers[i]
-        kc, vc = kv.layer(i)
-        gates = z[:, z.shape[1] - up(m.heads, 16):][:, :m.heads]
-        splits = max(1, int(step.attn.kv_splits) * self.hkv // kc.shape[1])
-        latent = vc is None
-        a = ops.masked_attention(q, kc, vc, step.attn, m.scale, self.cfg.group, sink=False if latent else lw.sinks,
-                                 window=m.window, keep_first=m.keep_first, slopes=self.slopes[i], gate=gates,
-                                 v_dim=m.row[1] if latent else None, max_splits=splits)
-        if latent:
-            out = torch.empty(a.shape[0], m.heads, m.vdim_p, device=self.device, dtype=self.dtype)
-            a = ops.gemm_heads(a, lw.w_uv, out)
-        return a.view(a.shape[0], -1)
+    def _plan(self, i, step):
+        """The spans of the step whose keys layer ``i`` expands (one plan per
+        window, kept with the step)."""
+        m, meta = self.cfg.layer_specs[i].mixer, step.attn
+        if meta.host is None or self.w.layers[i].w_ukv is None or self.device.type != "cuda":
+            return None
+        plans = meta.host.plans
+        if m.window not in plans:
+            plans[m.window] = long_spans(meta.host, self.EXPAND_MIN, m.window, ops.LATENT_ITEM, self.device)
+        plan = plans[m.window]
+        if plan is None or plan.pages.numel() * 64 * self.w.layers[i].w_ukv.shape[0] * 2 > self.EXPAND_MAX_BYTES:
+            return None
+        return plan
 
     def logits(self, hidden: torch.Tensor) -> torch.Tensor:
         """[R, vocab] fp32 logits of ``forward``'s rows."""

@@ -616,8 +616,8 @@ def latent_qkv(z, pos, slots, cos_sin, w_c, eps: float, heads: int, dim: int, ro
     """Latent attention's rows around the absorbed query: ``z`` [T, >= heads
     (dim + rot) + rank + rot] holds per head [unrotated | rotated], then the
     latent and the shared rotated key.  Writes the key row [rms(latent) * w_c |
-    rotated key | 0] to the cache and [rotated query | 0] to q_out[..., rank:];
-    q_out[..., :rank] is ``gemm_heads``'s.  cos_sin [P, n, 2] rotates the first
+    rotated key | 0] to the cache and [rotated query | 0] to q_out[..., rank:]
+    (``q_out`` None: the cache only); q_out[..., :rank] is ``gemm_heads``'s.  cos_sin [P, n, 2] rotates the first
     2 n of the ``rot`` elements as halves."""
     if z.is_cuda:
         lib().latent_qkv(z, pos, slots, cos_sin, w_c, float(eps), int(heads), int(dim), int(rot),
@@ -625,6 +625,26 @@ def latent_qkv(z, pos, slots, cos_sin, w_c, eps: float, heads: int, dim: int, ro
     else:
         ref.latent_qkv(z, pos, slots, cos_sin, w_c, eps, heads, dim, rot, rank, rank_true, q_out, k_cache)
     return q_out
+
+
+def latent_gather(cache, pages, valid, rank: int, out):
+    """The latents (columns [:rank]) of cached pages as rows out [pages * 64, C];
+    other columns, and rows from a page's ``valid`` on, are zero."""
+    lib().latent_gather(cache, pages, valid, int(rank), out)
+    return out
+
+
+def latent_prefill(z, meta, plan, pos, cos_sin, heads: int, dim: int, rot: int, exp, cache, rank: int,
+                   scale: float, window: int, gate, out):
+    """Latent attention of a step's long spans (``plan``, engine.batch.long_spans)
+    on expanded keys and values: ``exp`` [keys, heads (dim + DV)] the projections
+    of the gathered latents, the rotated key part from the cache, queries from the
+    projected rows ``z`` (per head [dim | rot]).  Writes those spans' rows of
+    ``out`` [T, heads, DV]."""
+    lib().latent_prefill(z, pos, cos_sin, int(heads), int(dim), int(rot), exp, plan.key0, cache, int(rank),
+                         meta.q_start, meta.q_len, meta.ctx_len, meta.block_table, plan.item_seq, plan.item_q0,
+                         next(k for k in HEAD_SIZES if k >= dim + rot), float(scale), int(window), gate, out)
+    return out
 
 
 def gemm_heads(X, W, out):
@@ -636,16 +656,33 @@ def gemm_heads(X, W, out):
     return ref.gemm_heads(X, W, out)
 
 
-MASKED_MAX_HEAD = 256           # largest head of the MFMA forms (csrc/attention_masked.hip)
+HEAD_SIZES = (64, 128, 192, 256)                # head sizes of the MFMA forms (csrc/attention_masked.hip)
+MASKED_MAX_HEAD = HEAD_SIZES[-1]
+LATENT_ITEM = 128               # tokens per work item of latent_prefill (csrc/kernels.h)
 # (key, value) sizes of the MFMA form whose values are the first columns of the
 # keys (csrc/attention_latent.hip)
 LATENT_SIZES = ((64, 64), (128, 64), (128, 128), (192, 128), (192, 192), (256, 192), (256, 256),
                 (320, 256), (448, 384), (576, 512))
 
 
+def _latent_splits(meta, items: int, q, DV: int, window: int, keep_first: int) -> int:
+    """Key splits of an absorbed latent attention launch: one row group of 32
+    query heads per workgroup, about two workgroups per CU, a tile each at least.
+    A padded (hipGraph) work list has fewer items than entries; the scheduler's
+    split count says how few."""
+    tiles = meta.block_table.shape[1]
+    if window:
+        tiles = min(tiles, -(-window // 64) + 1 + -(-keep_first // 64))
+    want = 4 * int(meta.kv_splits) if meta.padded else \
+        2 * _num_cus(q.device) // max(1, items * -(-q.shape[1] // 32))
+    room = (256 << 20) // max(1, 4 * DV * q.shape[0] * q.shape[1])
+    return max(1, min(want, tiles, room))
+
+
 def masked_attention(q, k_cache, v_cache, meta, scale, group: int, soft_cap: float = 0.0,
                      chunk: int = 0, sink=False, window: int = 0, keep_first: int = 0, slopes=None,
-                     gate=None, v_dim: Optional[int] = None, max_splits: int = 1 << 30):
+                     gate=None, v_dim: Optional[int] = None, max_splits: int = 1 << 30,
+                     skip_q: int = 0):
     """Paged causal attention, q [T, Hq, DK] -> [T, Hq, DV].
 
     ``soft_cap``: s <- cap tanh(s / cap); 0 = none.  ``chunk``: only keys of the
@@ -658,7 +695,9 @@ def masked_attention(q, k_cache, v_cache, meta, scale, group: int, soft_cap: flo
     values are the first ``v_dim`` columns of the keys (latent attention).
     ``group``: the GQA group the step's work lists were cut for (16 / group
     tokens per 1-wave item); the heads' own group may be another.
-    ``max_splits`` bounds the scheduler's key splits for this layer."""
+    ``max_splits`` bounds the scheduler's key splits for this layer; latent
+    attention chooses its own while the scheduler splits.  ``skip_q`` (latent
+    attention): rows of spans of that many tokens are left alone."""
     if q.is_cuda:
         shared = v_cache is None
         DV = v_dim if shared else v_cache.shape[3]
@@ -672,13 +711,15 @@ def masked_attention(q, k_cache, v_cache, meta, scale, group: int, soft_cap: flo
                                           max(q.shape[2], DV) <= MASKED_MAX_HEAD):
             for nw, ws, wq in meta.work_lists():
                 nz, so, sm = 1, None, None
-                if nw == 1 and int(meta.kv_splits) > 1:
+                if shared and int(meta.kv_splits) > 1:
+                    nz = _latent_splits(meta, ws.numel(), q, DV, window, keep_first)
+                elif nw == 1 and int(meta.kv_splits) > 1:
                     # (the partials are addressed with 31 bits)
                     nz = max(1, min(int(meta.kv_splits), max_splits, (1 << 31) // max(1, 4 * out.numel()) - 1))
                 if nz > 1:
                     so = torch.empty(nz, *out.shape, device=q.device, dtype=torch.float32)
                     sm = torch.empty(nz, q.shape[0], q.shape[1], 2, device=q.device, dtype=torch.float32)
-                if not L.attention_masked(*a, ws, wq, nw, nw * (16 // group), *k, nz, so, sm):
+                if not L.attention_masked(*a, ws, wq, nw, nw * (16 // group), *k, nz, so, sm, skip_q):
                     raise ValueError(f"masked attention: head sizes {q.shape[2]} / {DV}")
             return out
         L.attention_row(*a, *k)

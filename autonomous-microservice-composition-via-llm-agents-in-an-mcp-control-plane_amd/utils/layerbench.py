@@ -46,7 +46,7 @@ def _models(size: str, device, which):
 
 
 def _step(model, seqs: int, ctx: int, new: int, device):
-    from ..engine.batch import BLOCK_SIZE, choose_kv_splits, pack_step, to_device, views
+    from ..engine.batch import BLOCK_SIZE, choose_kv_splits, pack_step, step_from_host, to_device, views
     from ..engine.kv_cache import KVCache
     need = -(-(ctx + new) // BLOCK_SIZE)
     kv = KVCache.for_model(model, seqs * need)
@@ -59,6 +59,8 @@ def _step(model, seqs: int, ctx: int, new: int, device):
     own = [ctx + new] * seqs
     ns = choose_kv_splits([new] * seqs, own, model.cfg.group, model.hkv, hq=model.hq)
     d = views(to_device(host, device), list(layout) + [ns, 0, -(-(ctx + new) // BLOCK_SIZE)])[0]
+    if getattr(model, "uses_host_step", False) and new > 1:
+        d.attn.host = step_from_host(host, layout)
     return d, kv
 
 
