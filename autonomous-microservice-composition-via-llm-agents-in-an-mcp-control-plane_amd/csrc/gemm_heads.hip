@@ -2,8 +2,8 @@
 // value projections of latent attention.  X and out are strided [T, H, .] views,
 // W [H, N, K].  MFMA accumulators hold out^T (A = W rows, B = X rows), so a lane
 // owns four neighbouring outputs of one token.  Three forms:
-//   few   up to 64 tokens (decode): a wave per 16 outputs of a head, operands
-//         straight from global memory;
+//   few   up to 64 tokens (decode): a block per 16 outputs of a head, the sum over
+//         k shared out to its 4 waves, operands straight from global memory;
 //   tile  128 tokens x 128 outputs per block, LDS-DMA staging, stores through
 //         LDS so that a token's outputs leave as whole lines;
 //   f32   the 32-bit mode, plain FMAs, one sum in k order per output.
@@ -15,10 +15,10 @@ namespace {
 // ------------------------------------------------------------------ few tokens
 template <int NT>
 __global__ __launch_bounds__(256) void heads_few_kernel(const HeadGemmArgs a) {
+  __shared__ f32x4 part[4][NT][64];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int fr = lane & 15, fq = lane >> 4;
-  const int h = blockIdx.y, n0 = (blockIdx.x * 4 + wave) * 16;
-  if (n0 >= a.N) return;
+  const int h = blockIdx.y, n0 = blockIdx.x * 16;
   const bf16* w = (const bf16*)a.W + ((size_t)h * a.N + n0 + fr) * a.K + 8 * fq;
   const bf16* x[NT];
 #pragma unroll
@@ -28,21 +28,22 @@ __global__ __launch_bounds__(256) void heads_few_kernel(const HeadGemmArgs a) {
 #pragma unroll
   for (int i = 0; i < NT; ++i) acc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll 4
-  for (int k = 0; k < a.K; k += 32) {
+  for (int k = wave * 32; k < a.K; k += 128) {
     const bf16x8 wf = *reinterpret_cast<const bf16x8*>(w + k);
 #pragma unroll
     for (int i = 0; i < NT; ++i)
       acc[i] = mfma16x16x32(wf, *reinterpret_cast<const bf16x8*>(x[i] + k), acc[i]);
   }
 #pragma unroll
-  for (int i = 0; i < NT; ++i) {
-    const int t = i * 16 + fr;
-    if (t >= a.T) continue;
-    bf16x4 o;
+  for (int i = 0; i < NT; ++i) part[wave][i][lane] = acc[i];
+  __syncthreads();
+  const int t = wave * 16 + fr;                         // wave i adds token tile i
+  if (wave >= NT || t >= a.T) return;
+  const f32x4 v = part[0][wave][lane] + part[1][wave][lane] + part[2][wave][lane] + part[3][wave][lane];
+  bf16x4 o;
 #pragma unroll
-    for (int r = 0; r < 4; ++r) o[r] = (bf16)acc[i][r];
-    *reinterpret_cast<bf16x4*>((bf16*)a.out + (size_t)t * a.ot + (size_t)h * a.oh + n0 + 4 * fq) = o;
-  }
+  for (int r = 0; r < 4; ++r) o[r] = (bf16)v[r];
+  *reinterpret_cast<bf16x4*>((bf16*)a.out + (size_t)t * a.ot + (size_t)h * a.oh + n0 + 4 * fq) = o;
 }
 
 // ------------------------------------------------------------------------ tile
@@ -174,7 +175,7 @@ int launch_gemm_heads(const HeadGemmArgs& a, bool f32, hipStream_t s) {
     return 0;
   }
   if (a.T <= 64) {
-    const dim3 grid((a.N + 63) / 64, a.H);
+    const dim3 grid(a.N / 16, a.H);
     if (a.T <= 16) heads_few_kernel<1><<<grid, 256, 0, s>>>(a);
     else if (a.T <= 32) heads_few_kernel<2><<<grid, 256, 0, s>>>(a);
     else heads_few_kernel<4><<<grid, 256, 0, s>>>(a);

@@ -435,7 +435,8 @@ class TopelornModel:
                 return h.new_empty(0, h.shape[1])      # every key is in the cache; nothing is read
             if i == self.first:
                 v_first = v
-            if last and tap is None:                   # only the asked-for rows go on
+            early = last and tap is None and rows.numel() < h.shape[0] and h.shape[0] > 64
+            if early:                                  # only the asked-for rows go on (few tokens: all do)
                 ri = rows.long()
                 x, h, a = x.index_select(0, ri), h.index_select(0, ri), a.index_select(0, ri)
             y = ops.gemm(a, lw.wo)
@@ -444,8 +445,7 @@ class TopelornModel:
         h = ops.residual_norm(x, W, eps, y, None, w.final_norm, torch.empty_like(h), center=True)
         if tap is not None:
             tap(cfg.layers - 1, x[:, :W])
-            h = h.index_select(0, rows.long())
-        return h
+        return h if early else h.index_select(0, rows.long())
 
     def _gates(self, m, z):
         return z[:, z.shape[1] - up(m.heads, 16):][:, :m.heads]
@@ -461,8 +461,7 @@ class TopelornModel:
         if cache_only:
             return None, None
         a = ops.masked_attention(q, kc, vc, step.attn, m.scale, self.cfg.group, sink=lw.sinks, window=m.window,
-                                 keep_first=m.keep_first, slopes=self.slopes[i], gate=self._gates(m, z),
-                                 max_splits=max(1, int(step.attn.kv_splits) * self.hkv // m.kv_heads))
+                                 keep_first=m.keep_first, slopes=self.slopes[i], gate=self._gates(m, z))
         at = (m.heads + m.kv_heads) * m.dk
         return a.view(T, -1), z[:, at:at + m.kv_heads * m.dv]
 

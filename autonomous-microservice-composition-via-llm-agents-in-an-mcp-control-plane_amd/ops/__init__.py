@@ -667,21 +667,21 @@ LATENT_SIZES = ((64, 64), (128, 64), (128, 128), (192, 128), (192, 192), (256, 1
 
 def _latent_splits(meta, items: int, q, DV: int, window: int, keep_first: int) -> int:
     """Key splits of an absorbed latent attention launch: one row group of 32
-    query heads per workgroup, about two workgroups per CU, a tile each at least.
-    A padded (hipGraph) work list has fewer items than entries; the scheduler's
-    split count says how few."""
+    query heads per workgroup, one workgroup per CU, two tiles each at least.  A padded
+    (hipGraph) work list has fewer items than entries; the scheduler's split count
+    says how few."""
     tiles = meta.block_table.shape[1]
     if window:
         tiles = min(tiles, -(-window // 64) + 1 + -(-keep_first // 64))
     want = 4 * int(meta.kv_splits) if meta.padded else \
-        2 * _num_cus(q.device) // max(1, items * -(-q.shape[1] // 32))
+        -(-_num_cus(q.device) // max(1, items * -(-q.shape[1] // 32)))
     room = (256 << 20) // max(1, 4 * DV * q.shape[0] * q.shape[1])
-    return max(1, min(want, tiles, room))
+    return max(1, min(want, -(-tiles // 2), room, 64))
 
 
 def masked_attention(q, k_cache, v_cache, meta, scale, group: int, soft_cap: float = 0.0,
                      chunk: int = 0, sink=False, window: int = 0, keep_first: int = 0, slopes=None,
-                     gate=None, v_dim: Optional[int] = None, max_splits: int = 1 << 30,
+                     gate=None, v_dim: Optional[int] = None,
                      skip_q: int = 0):
     """Paged causal attention, q [T, Hq, DK] -> [T, Hq, DV].
 
@@ -695,8 +695,8 @@ def masked_attention(q, k_cache, v_cache, meta, scale, group: int, soft_cap: flo
     values are the first ``v_dim`` columns of the keys (latent attention).
     ``group``: the GQA group the step's work lists were cut for (16 / group
     tokens per 1-wave item); the heads' own group may be another.
-    ``max_splits`` bounds the scheduler's key splits for this layer; latent
-    attention chooses its own while the scheduler splits.  ``skip_q`` (latent
+    While the scheduler splits keys, a layer whose heads or window give fewer
+    workgroups or tiles than it reckons with splits less.  ``skip_q`` (latent
     attention): rows of spans of that many tokens are left alone."""
     if q.is_cuda:
         shared = v_cache is None
@@ -714,8 +714,13 @@ def masked_attention(q, k_cache, v_cache, meta, scale, group: int, soft_cap: flo
                 if shared and int(meta.kv_splits) > 1:
                     nz = _latent_splits(meta, ws.numel(), q, DV, window, keep_first)
                 elif nw == 1 and int(meta.kv_splits) > 1:
-                    # (the partials are addressed with 31 bits)
-                    nz = max(1, min(int(meta.kv_splits), max_splits, (1 << 31) // max(1, 4 * out.numel()) - 1))
+                    # (the partials are addressed with 31 bits; 4 waves take a tile each)
+                    nz = min(int(meta.kv_splits), (1 << 31) // max(1, 4 * out.numel()) - 1)
+                    if not meta.padded:
+                        nz = min(nz, 2 * _num_cus(q.device) // max(1, ws.numel() * k_cache.shape[1]))
+                    if window:
+                        nz = min(nz, -(-(window + 63 + keep_first + 63) // 256))
+                    nz = max(1, nz)
                 if nz > 1:
                     so = torch.empty(nz, *out.shape, device=q.device, dtype=torch.float32)
                     sm = torch.empty(nz, q.shape[0], q.shape[1], 2, device=q.device, dtype=torch.float32)

@@ -227,12 +227,13 @@ def _rotate_halves(x, cs):
 
 
 def latent_qkv(z, pos, slots, cos_sin, w_c, eps, heads, dim, rot, rank, rank_true, q_out, k_cache):
-    T, _, DK = q_out.shape
+    T, DK = z.shape[0], k_cache.shape[3]
     cs = cos_sin[pos.long()]
     pre = heads * (dim + rot)
-    q = z[:, :pre].float().view(T, heads, dim + rot)
-    q_out[..., rank:] = 0
-    q_out[..., rank:rank + rot] = _rotate_halves(q[..., dim:], cs).to(q_out.dtype)
+    if q_out is not None:
+        q = z[:, :pre].float().view(T, heads, dim + rot)
+        q_out[..., rank:] = 0
+        q_out[..., rank:rank + rot] = _rotate_halves(q[..., dim:], cs).to(q_out.dtype)
     row = torch.zeros(T, DK)
     row[:, :rank] = head_rms(z[:, pre:pre + rank], w_c, rank_true, eps)
     row[:, rank:rank + rot] = _rotate_halves(z[:, pre + rank:pre + rank + rot].float(), cs)
