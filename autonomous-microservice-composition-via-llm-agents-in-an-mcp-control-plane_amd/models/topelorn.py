@@ -379,7 +379,7 @@ class TopelornModel:
     tp_rank = 0
     supports_cascade = False      # a shared prefix leaves the window as a request goes on
     uses_host_step = True         # spans this long expand the latents they see
-    EXPAND_MIN, EXPAND_MAX_BYTES = 256, 4 << 30
+    EXPAND_MIN, EXPAND_MAX_BYTES = 192, 4 << 30
     logit_scale, logit_cap = 1.0, 0.0
 
     def __init__(self, cfg: TopelornConfig, weights: TopelornWeights, device):
