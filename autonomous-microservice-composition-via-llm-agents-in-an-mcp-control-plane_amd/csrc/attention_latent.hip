@@ -240,10 +240,10 @@ __global__ __launch_bounds__(256) void attn_latent_merge_kernel(const MaskedAttn
 }
 
 template <int DK, int DV>
-int launch_pair(const MaskedAttnArgs& a, int nwork, int nz, hipStream_t s) {
-  // one token's rows in the grid when keys are split (decoding: the blocks of further
-  // tokens would mostly find none, and hold a CU's LDS to see that), else the item's
-  const int rows = (nz > 1 ? 1 : a.item_tokens) * a.Hq;
+int launch_pair(const MaskedAttnArgs& a, int nwork, int form, int nz, hipStream_t s) {
+  // 1-wave items with split keys (decoding): one token's rows in the grid.  Blocks of
+  // further tokens would mostly find none, and hold a CU's LDS to see that
+  const int rows = (form == 1 && nz > 1 ? 1 : a.item_tokens) * a.Hq;
   if (a.Hq <= 16) attn_latent_kernel<DK, DV, 1><<<dim3(nwork, (rows + 15) / 16, nz), 256, 0, s>>>(a);
   else attn_latent_kernel<DK, DV, 2><<<dim3(nwork, (rows + 31) / 32, nz), 512, 0, s>>>(a);
   if (nz > 1) attn_latent_merge_kernel<<<dim3(nwork, (rows + 1) / 2), 256, 0, s>>>(a, nz);
@@ -412,21 +412,21 @@ int launch_prefill_dk(const LatentPrefillArgs& a, hipStream_t s) {
 }  // namespace
 
 // One work list; 3: a (DK, DV) pair without a kernel (the row form takes it)
-int launch_attn_latent(const MaskedAttnArgs& a, int nwork, int nz, hipStream_t s) {
+int launch_attn_latent(const MaskedAttnArgs& a, int nwork, int form, int nz, hipStream_t s) {
   if (nwork <= 0) return 0;
   if (a.Hkv != 1 || a.cap > 0.f || a.slopes) return 1;
   if (nz < 1 || nz > MAX_SPLITS || (nz > 1 && (!a.split_o || !a.split_ml))) return 2;
   switch (a.DK * 1024 + a.DV) {
-    case 64 * 1024 + 64: return launch_pair<64, 64>(a, nwork, nz, s);
-    case 128 * 1024 + 64: return launch_pair<128, 64>(a, nwork, nz, s);
-    case 128 * 1024 + 128: return launch_pair<128, 128>(a, nwork, nz, s);
-    case 192 * 1024 + 128: return launch_pair<192, 128>(a, nwork, nz, s);
-    case 192 * 1024 + 192: return launch_pair<192, 192>(a, nwork, nz, s);
-    case 256 * 1024 + 192: return launch_pair<256, 192>(a, nwork, nz, s);
-    case 256 * 1024 + 256: return launch_pair<256, 256>(a, nwork, nz, s);
-    case 320 * 1024 + 256: return launch_pair<320, 256>(a, nwork, nz, s);
-    case 448 * 1024 + 384: return launch_pair<448, 384>(a, nwork, nz, s);
-    case 576 * 1024 + 512: return launch_pair<576, 512>(a, nwork, nz, s);
+    case 64 * 1024 + 64: return launch_pair<64, 64>(a, nwork, form, nz, s);
+    case 128 * 1024 + 64: return launch_pair<128, 64>(a, nwork, form, nz, s);
+    case 128 * 1024 + 128: return launch_pair<128, 128>(a, nwork, form, nz, s);
+    case 192 * 1024 + 128: return launch_pair<192, 128>(a, nwork, form, nz, s);
+    case 192 * 1024 + 192: return launch_pair<192, 192>(a, nwork, form, nz, s);
+    case 256 * 1024 + 192: return launch_pair<256, 192>(a, nwork, form, nz, s);
+    case 256 * 1024 + 256: return launch_pair<256, 256>(a, nwork, form, nz, s);
+    case 320 * 1024 + 256: return launch_pair<320, 256>(a, nwork, form, nz, s);
+    case 448 * 1024 + 384: return launch_pair<448, 384>(a, nwork, form, nz, s);
+    case 576 * 1024 + 512: return launch_pair<576, 512>(a, nwork, form, nz, s);
     default: return 3;
   }
 }

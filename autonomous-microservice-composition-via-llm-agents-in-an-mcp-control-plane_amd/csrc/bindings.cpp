@@ -1110,7 +1110,7 @@ bool attention_masked(const at::Tensor& q, const at::Tensor& k_cache, const c10:
     a.split_ml = split_ml->data_ptr<float>();
   }
   const int rc = v_cache.has_value() ? launch_attn_masked(a, work_seq.numel(), (int)form, (int)nz, stream())
-                                     : launch_attn_latent(a, work_seq.numel(), (int)nz, stream());
+                                     : launch_attn_latent(a, work_seq.numel(), (int)form, (int)nz, stream());
   if (rc == 3) return false;
   TORCH_CHECK(rc == 0, "attention_masked: code ", rc);
   check_launch("attention_masked");

@@ -133,8 +133,8 @@ struct MaskedAttnArgs {
   int skip_q;                // > 0: sequences with this many new tokens are somebody else's (latent form)
 };
 int launch_attn_masked(const MaskedAttnArgs& a, int nwork, int form, int nz, hipStream_t s);
-// values are the first DV columns of the keys (vc is not read); either work list
-int launch_attn_latent(const MaskedAttnArgs& a, int nwork, int nz, hipStream_t s);
+// values are the first DV columns of the keys (vc is not read); either form may split
+int launch_attn_latent(const MaskedAttnArgs& a, int nwork, int form, int nz, hipStream_t s);
 // long prompt portions of latent attention: keys and values per head from expanded
 // rows [dim | DV] of every key, the rotated key part from the cache
 struct LatentPrefillArgs {

@@ -665,16 +665,16 @@ LATENT_SIZES = ((64, 64), (128, 64), (128, 128), (192, 128), (192, 192), (256, 1
                 (320, 256), (448, 384), (576, 512))
 
 
-def _latent_splits(meta, items: int, q, DV: int, window: int, keep_first: int) -> int:
-    """Key splits of an absorbed latent attention launch: one row group of 32
-    query heads per workgroup, one workgroup per CU, two tiles each at least.  A padded
-    (hipGraph) work list has fewer items than entries; the scheduler's split count
-    says how few."""
+def _latent_splits(meta, tokens: int, q, DV: int, window: int, keep_first: int) -> int:
+    """Key splits of an absorbed latent attention launch over ``tokens`` tokens (an
+    item of the 1-wave list counts as one): a workgroup per 32 rows, one per CU, two
+    key tiles each at least.  A padded (hipGraph) work list has fewer items than
+    entries; the scheduler's split count says how few."""
     tiles = meta.block_table.shape[1]
     if window:
         tiles = min(tiles, -(-window // 64) + 1 + -(-keep_first // 64))
     want = 4 * int(meta.kv_splits) if meta.padded else \
-        -(-_num_cus(q.device) // max(1, items * -(-q.shape[1] // 32)))
+        -(-_num_cus(q.device) // max(1, tokens * -(-q.shape[1] // 32)))
     room = (256 << 20) // max(1, 4 * DV * q.shape[0] * q.shape[1])
     return max(1, min(want, -(-tiles // 2), room, 64))
 
@@ -712,7 +712,8 @@ def masked_attention(q, k_cache, v_cache, meta, scale, group: int, soft_cap: flo
             for nw, ws, wq in meta.work_lists():
                 nz, so, sm = 1, None, None
                 if shared and int(meta.kv_splits) > 1:
-                    nz = _latent_splits(meta, ws.numel(), q, DV, window, keep_first)
+                    nz = _latent_splits(meta, ws.numel() * (1 if nw == 1 else nw * (16 // group)), q, DV, window,
+                                        keep_first)
                 elif nw == 1 and int(meta.kv_splits) > 1:
                     # (the partials are addressed with 31 bits; 4 waves take a tile each)
                     nz = min(int(meta.kv_splits), (1 << 31) // max(1, 4 * out.numel()) - 1)

@@ -203,6 +203,8 @@ def test_latent_windows(window, splits):
     _check(MIXED, 20, 1, 192, 128, window, 0, slopes=False, sinks=False, seed=window, splits=splits, amp=2.0, shared=True)
     _check([(1500, 1), (70, 1), (0, 2), (999, 6), (640, 1)], 40, 1, 576, 512, window, 0, slopes=False, sinks=False,
            seed=window, splits=splits, shared=True)
+    _check([(900, 17), (700, 1), (800, 12)], 24, 1, 320, 256, window, 0, slopes=False, sinks=False, splits=splits,
+           shared=True)
     _check(MIXED, 8, 1, 128, 64, max(window, 1), 3, slopes=False, seed=window, splits=splits, shared=True)
 
 
